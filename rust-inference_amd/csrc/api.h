@@ -185,6 +185,9 @@ int ri_experts_combine(float* out, const void* y, const int32_t* dest, const flo
 // [experts * 2 * ff, dim] (every expert's gate rows, then its up rows); down [dim, experts * ff]; ids and weights
 // [tokens, top] from ri_experts_route; act: workspace [tokens * top, ff] bfloat16; out: float32 [tokens, dim], the
 // weighted sum of the chosen experts' outputs, added in the order chosen.
+// experts without a gate, as ri_experts_few_tokens: up [experts, ff, dim] rows, kind: the activation
+int ri_experts_few_tokens_plain(float* out, void* act, const void* x, const void* up, const void* down, const int32_t* ids,
+                                const float* weights, int tokens, int experts, int top, int ff, int dim, int kind, void* stream);
 int ri_experts_few_tokens(float* out, void* act, const void* x, const void* gu, const void* down, const int32_t* ids,
                           const float* weights, int tokens, int experts, int top, int ff, int dim, float limit,
                           void* stream);
@@ -478,6 +481,25 @@ int ri_ssd_scan_cols(float* out, const float* xbc, int channels, int b_off, int 
                      void* stream);
 int ri_group_rms_norm(void* out, int out_dtype, const float* x, const float* gain, float eps, int rows, int width, int parts,
                       void* stream);
+
+// Biases, rotation in halves and the cache write (qk_half_bias_kv.hip).
+int ri_qk_half_bias_kv_write(void* proj, int act_dtype, long row_len, int q_off, int k_off, int v_off, const float* q_bias,
+                             const float* k_bias, const float* v_bias, const float* inv_freq, int half, float amplitude,
+                             const int32_t* tok_pos, const int32_t* tok_seq, const int32_t* cu_seqlens, int seqs, int max_new,
+                             const int32_t* page_table, int table_width, void* k_pages, void* v_pages, int cache_dtype,
+                             int tokens, int heads, int kv_heads, int dim, int vdim, int page_size, void* stream);
+
+// out[t, :] = table[ids[t], :] + pairs[row, :], row = buckets for a sequence's first token, else
+// (token before * mul_prev + ids[t] * mul_cur) mod buckets; last[slot]: a sequence's last token, from step to step.
+int ri_embed_bigram(float* out, const void* table, const void* pairs, int table_dtype, const int32_t* ids,
+                    const int32_t* tok_pos, const int32_t* tok_seq, const int32_t* cu_seqlens, const int32_t* slots,
+                    int32_t* last, long buckets, long mul_prev, long mul_cur, int tokens, int dim, void* stream);
+
+// ri_branch_norm_add with the norm in front of the next sublayer in the same kernel: act = rms_norm(new residual) *
+// next_gain (next_gain NULL: the new residual itself); tiled: act in the order of tiled_at.
+int ri_branch_norm_add_norm(float* residual, void* act, int act_dtype, const void* y, int y_dtype, int parts,
+                            const float* gain, const float* bias, float eps, int kind, const float* layer_scale,
+                            const float* next_gain, float next_eps, int tiled, int rows, int dim, void* stream);
 
 #ifdef __cplusplus
 }

@@ -1,10 +1,12 @@
 // Row-wise kernels around a sublayer whose norm sits on its output, and around mixers that run side by side:
 //
 //   embed_scaled:     r = E[id] * scale (float32), and a copy of r in the activations' format;
+//   embed_bigram:     r = E[id] + B[row of the pair (token before, token)], the token before kept per sequence;
 //   branch_norm_add:  r += layer_scale * norm(y), the norm (layer norm with gain and bias, or RMS norm with gain) over the
 //                     sublayer's output y, which may come as parts of a split product that are added in order;
 //                     again with a copy of the new r in the activations' format, which the next sublayer reads
-//                     (the sublayers read r itself: there is no norm before them);
+//                     (the sublayers read r itself: there is no norm before them), or, where a norm sits in front of the
+//                     next sublayer too, with that norm of the new r: act = r / sqrt(mean(r^2) + next_eps) * next_gain;
 //   gate_rows:        out = scale * x * gate(g), element by element, into columns of a wider row (the heads of
 //                     several mixers side by side, for one output product);
 //   row_norm_gate:    out = scale * x / sqrt(mean(x^2) + eps) * gain * gate(g), the mean over the whole row (all heads
@@ -81,12 +83,65 @@ extern "C" int ri_embed_scaled(float* out, void* act, int act_dtype, const void*
     return 0;
 }
 
+// Row `buckets` (the last) for a sequence's first token; else row (before * mul_prev + id * mul_cur) mod buckets, both
+// factors already reduced modulo buckets (every product then fits 64 bits).  A workgroup a token; the workgroup of a
+// sequence's first new token alone reads the token kept from the step before, and it alone puts the step's last token in
+// its place, after it has read.
+template <typename TW, bool VEC>
+__global__ void __launch_bounds__(256)
+embed_bigram_kernel(float* __restrict__ out, const TW* __restrict__ table, const TW* __restrict__ pairs,
+                    const int32_t* __restrict__ ids, const int32_t* __restrict__ tok_pos, const int32_t* __restrict__ tok_seq,
+                    const int32_t* __restrict__ cu_seqlens, const int32_t* __restrict__ slots, int32_t* __restrict__ last,
+                    long buckets, long mul_prev, long mul_cur, int dim) {
+    const int t = blockIdx.x, b = tok_seq[t], slot = slots[b];
+    const bool opens = t == cu_seqlens[b];                   // the sequence's first token of this step
+    const long id = ids[t];
+    long row = buckets;
+    if (tok_pos[t] > 0) {
+        const long before = opens ? last[slot] : ids[t - 1];
+        row = (before * mul_prev + id * mul_cur) % buckets;
+    }
+    const TW* a = table + (size_t)id * dim;
+    const TW* p = pairs + (size_t)row * dim;
+    float* o = out + (size_t)t * dim;
+    if (VEC) {
+        for (int d = threadIdx.x * 4; d < dim; d += 1024) {
+            const float4 u = ld4(a + d), v = ld4(p + d);
+            st4(o + d, make_float4(u.x + v.x, u.y + v.y, u.z + v.z, u.w + v.w));
+        }
+    } else {
+        for (int d = threadIdx.x; d < dim; d += 256) o[d] = to_f32(a[d]) + to_f32(p[d]);
+    }
+    if (!opens) return;
+    __syncthreads();                                         // every thread has read the kept token
+    if (threadIdx.x == 0) last[slot] = ids[cu_seqlens[b + 1] - 1];
+}
+
+extern "C" int ri_embed_bigram(float* out, const void* table, const void* pairs, int table_dtype, const int32_t* ids,
+                               const int32_t* tok_pos, const int32_t* tok_seq, const int32_t* cu_seqlens, const int32_t* slots,
+                               int32_t* last, long buckets, long mul_prev, long mul_cur, int tokens, int dim, void* stream) {
+    RI_REQUIRE(tokens > 0 && dim > 0, "embed_bigram: tokens %d, dim %d", tokens, dim);
+    RI_REQUIRE(buckets >= 1 && buckets <= 2147483647L && mul_prev >= 0 && mul_prev < buckets && mul_cur >= 0 && mul_cur < buckets,
+               "embed_bigram: %ld buckets, factors %ld and %ld (reduced modulo the buckets)", buckets, mul_prev, mul_cur);
+    RI_REQUIRE(table_dtype == RI_F32 || table_dtype == RI_BF16, "embed_bigram: table dtype %d", table_dtype);
+    hipStream_t s = (hipStream_t)stream;
+#define RI_GO(TW, VEC)                                                                                                  \
+    embed_bigram_kernel<TW, VEC><<<tokens, 256, 0, s>>>(out, (const TW*)table, (const TW*)pairs, ids, tok_pos, tok_seq,    \
+                                                       cu_seqlens, slots, last, buckets, mul_prev, mul_cur, dim)
+    if (table_dtype == RI_F32) { if (dim % 4 == 0) RI_GO(float, true); else RI_GO(float, false); }
+    else                       { if (dim % 4 == 0) RI_GO(bf16_t, true); else RI_GO(bf16_t, false); }
+#undef RI_GO
+    RI_LAUNCH_CHECK("embed_bigram");
+    return 0;
+}
+
 // The row's y is kept in LDS as float32 between the passes (parts added once, in order).
 template <typename TY, typename TA>
 __global__ void __launch_bounds__(256)
 branch_norm_add_kernel(float* __restrict__ residual, TA* __restrict__ act, const TY* __restrict__ y, int parts,
                        size_t part_stride, const float* __restrict__ gain, const float* __restrict__ bias, float eps,
-                       int kind, const float* __restrict__ layer_scale, int dim) {
+                       int kind, const float* __restrict__ layer_scale, int dim, const float* __restrict__ next_gain,
+                       float next_eps) {
     extern __shared__ float row[];                           // dim floats
     __shared__ float scratch[16];
     const size_t at = (size_t)blockIdx.x * dim;
@@ -105,27 +160,36 @@ branch_norm_add_kernel(float* __restrict__ residual, TA* __restrict__ act, const
         ss += c * c;
     }
     const float inv = 1.0f / sqrtf(block_sum(ss, scratch) / (float)dim + eps);
+    float rr = 0.f;
     for (int d = threadIdx.x; d < dim; d += blockDim.x) {
         float v = (row[d] - mean) * inv * gain[d];
         if (bias) v += bias[d];
         if (layer_scale) v *= layer_scale[d];
         const float r = residual[at + d] + v;
         residual[at + d] = r;
-        if (act) from_f32(act + at + d, r);
+        if (next_gain) {                                     // (a thread's own columns: no barrier needed for them)
+            row[d] = r;
+            rr += r * r;
+        } else if (act) from_f32(act + at + d, r);
     }
+    if (!next_gain) return;
+    const float next_inv = 1.0f / sqrtf(block_sum(rr, scratch) / (float)dim + next_eps);
+    for (int d = threadIdx.x; d < dim; d += blockDim.x) from_f32(act + at + d, row[d] * next_inv * next_gain[d]);
 }
 
 // The same for rows of up to 8,192 elements, a multiple of 4: a thread asks for all its 16-byte pieces of the residual
 // and of every part of y up front and keeps them in registers, so that a row is one trip to memory and not one an
-// element; the parts are added in their order, the row's sums taken in an order that the width alone fixes.
-template <typename TY, typename TA, int VPT>
+// element; the parts are added in their order, the row's sums taken in an order that the width alone fixes.  `tiled`
+// (with NEXT): act in the order of tiled_at.
+template <typename TY, typename TA, int VPT, bool NEXT>
 __global__ void __launch_bounds__(256)
 branch_norm_add_vec_kernel(float* __restrict__ residual, TA* __restrict__ act, const TY* __restrict__ y, int parts,
                            size_t part_stride, const float* __restrict__ gain, const float* __restrict__ bias, float eps,
-                           int kind, const float* __restrict__ layer_scale, int dim) {
+                           int kind, const float* __restrict__ layer_scale, int dim, const float* __restrict__ next_gain,
+                           float next_eps, int tiled) {
     __shared__ float scratch[16];
     const size_t at = (size_t)blockIdx.x * dim;
-    float4 r[VPT], v[VPT];
+    float4 r[VPT], v[VPT], ng[NEXT ? VPT : 1];
     int col[VPT];
     bool ok[VPT];
 #pragma unroll
@@ -135,6 +199,7 @@ branch_norm_add_vec_kernel(float* __restrict__ residual, TA* __restrict__ act, c
         col[i] = ok[i] ? c : 0;                              // a column pulled back inside the row: the load is issued anyway
         r[i] = ld4(residual + at + col[i]);
         v[i] = ld4(y + at + col[i]);
+        if (NEXT) ng[i] = ld4(next_gain + col[i]);
     }
     for (int p = 1; p < parts; ++p) {
 #pragma unroll
@@ -160,6 +225,7 @@ branch_norm_add_vec_kernel(float* __restrict__ residual, TA* __restrict__ act, c
         }
     }
     const float inv = 1.0f / sqrtf(block_sum(ss, scratch) / (float)dim + eps);
+    float rr = 0.f;
 #pragma unroll
     for (int i = 0; i < VPT; ++i) {
         if (!ok[i]) continue;
@@ -176,16 +242,30 @@ branch_norm_add_vec_kernel(float* __restrict__ residual, TA* __restrict__ act, c
         }
         o = make_float4(r[i].x + o.x, r[i].y + o.y, r[i].z + o.z, r[i].w + o.w);
         st4(residual + at + col[i], o);
-        if (act) st4(act + at + col[i], o);
+        if (NEXT) {
+            r[i] = o;
+            rr += (o.x * o.x + o.y * o.y) + (o.z * o.z + o.w * o.w);
+        } else if (act) st4(act + at + col[i], o);
     }
+    if (!NEXT) return;
+    const float next_inv = 1.0f / sqrtf(block_sum(rr, scratch) / (float)dim + next_eps);
+#pragma unroll
+    for (int i = 0; i < VPT; ++i)
+        if (ok[i])                                           // four columns of one chunk of eight, tiled or not
+            st4(tiled ? act + tiled_at(blockIdx.x, col[i], (dim + 31) / 32) : act + at + col[i],
+                make_float4(r[i].x * next_inv * ng[NEXT ? i : 0].x, r[i].y * next_inv * ng[NEXT ? i : 0].y,
+                            r[i].z * next_inv * ng[NEXT ? i : 0].z, r[i].w * next_inv * ng[NEXT ? i : 0].w));
 }
 
-extern "C" int ri_branch_norm_add(float* residual, void* act, int act_dtype, const void* y, int y_dtype, int parts,
-                                  const float* gain, const float* bias, float eps, int kind, const float* layer_scale,
-                                  int rows, int dim, void* stream) {
+extern "C" int ri_branch_norm_add_norm(float* residual, void* act, int act_dtype, const void* y, int y_dtype, int parts,
+                                       const float* gain, const float* bias, float eps, int kind, const float* layer_scale,
+                                       const float* next_gain, float next_eps, int tiled, int rows, int dim, void* stream) {
     RI_REQUIRE(rows > 0 && dim > 0 && parts >= 1, "branch_norm_add: %d rows of %d in %d parts", rows, dim, parts);
     RI_REQUIRE(kind == BR_NORM_RMS || kind == BR_NORM_LAYER, "branch_norm_add: norm kind %d", kind);
     RI_REQUIRE(gain && residual && y, "branch_norm_add: a gain, a residual and a branch output are needed");
+    RI_REQUIRE(!next_gain || act, "branch_norm_add: the next norm's rows need a place");
+    RI_REQUIRE(!tiled || (next_gain && act_dtype == RI_BF16 && rows <= 64 && dim % 4 == 0 && dim <= 8192),
+               "branch_norm_add: tiled rows are the next norm's, at most 64 (%d of %d), in bfloat16", rows, dim);
     RI_REQUIRE((size_t)dim * sizeof(float) <= 64 * 1024, "branch_norm_add: rows of %d exceed the kernel's 16384", dim);
     RI_REQUIRE((y_dtype == RI_F32 || y_dtype == RI_BF16) && (act_dtype == RI_F32 || act_dtype == RI_BF16),
                "branch_norm_add: dtypes %d and %d", y_dtype, act_dtype);
@@ -193,16 +273,25 @@ extern "C" int ri_branch_norm_add(float* residual, void* act, int act_dtype, con
     hipStream_t s = (hipStream_t)stream;
     const size_t lds = (size_t)dim * sizeof(float), stride = (size_t)rows * dim;
 #define RI_VEC(TY, TA, VPT)                                                                                             \
-    branch_norm_add_vec_kernel<TY, TA, VPT><<<rows, 256, 0, s>>>(residual, (TA*)act, (const TY*)y, parts, stride, gain,   \
-                                                                 bias, eps, kind, layer_scale, dim)
+    do {                                                                                                                \
+        if (next_gain)                                                                                                  \
+            branch_norm_add_vec_kernel<TY, TA, VPT, true><<<rows, 256, 0, s>>>(                                           \
+                residual, (TA*)act, (const TY*)y, parts, stride, gain, bias, eps, kind, layer_scale, dim, next_gain,      \
+                next_eps, tiled);                                                                                       \
+        else                                                                                                            \
+            branch_norm_add_vec_kernel<TY, TA, VPT, false><<<rows, 256, 0, s>>>(                                          \
+                residual, (TA*)act, (const TY*)y, parts, stride, gain, bias, eps, kind, layer_scale, dim, nullptr, 0.f, 0); \
+    } while (0)
 #define RI_GO(TY, TA)                                                                                                   \
-    if (dim % 4 == 0 && dim <= 1024) RI_VEC(TY, TA, 1);                                                                 \
-    else if (dim % 4 == 0 && dim <= 2048) RI_VEC(TY, TA, 2);                                                            \
-    else if (dim % 4 == 0 && dim <= 4096) RI_VEC(TY, TA, 4);                                                            \
-    else if (dim % 4 == 0 && dim <= 8192) RI_VEC(TY, TA, 8);                                                            \
-    else                                                                                                                \
-    branch_norm_add_kernel<TY, TA><<<rows, 256, lds, s>>>(residual, (TA*)act, (const TY*)y, parts, stride, gain, bias, eps, \
-                                                         kind, layer_scale, dim)
+    do {                                                                                                                \
+        if (dim % 4 == 0 && dim <= 1024) RI_VEC(TY, TA, 1);                                                             \
+        else if (dim % 4 == 0 && dim <= 2048) RI_VEC(TY, TA, 2);                                                        \
+        else if (dim % 4 == 0 && dim <= 4096) RI_VEC(TY, TA, 4);                                                        \
+        else if (dim % 4 == 0 && dim <= 8192) RI_VEC(TY, TA, 8);                                                        \
+        else                                                                                                            \
+            branch_norm_add_kernel<TY, TA><<<rows, 256, lds, s>>>(residual, (TA*)act, (const TY*)y, parts, stride, gain,  \
+                                                                 bias, eps, kind, layer_scale, dim, next_gain, next_eps); \
+    } while (0)
     if (lds > 48 * 1024) {
         static bool asked = false;
         if (!asked) {
@@ -219,6 +308,13 @@ extern "C" int ri_branch_norm_add(float* residual, void* act, int act_dtype, con
 #undef RI_VEC
     RI_LAUNCH_CHECK("branch_norm_add");
     return 0;
+}
+
+extern "C" int ri_branch_norm_add(float* residual, void* act, int act_dtype, const void* y, int y_dtype, int parts,
+                                  const float* gain, const float* bias, float eps, int kind, const float* layer_scale,
+                                  int rows, int dim, void* stream) {
+    return ri_branch_norm_add_norm(residual, act, act_dtype, y, y_dtype, parts, gain, bias, eps, kind, layer_scale, nullptr, 0.f,
+                                   0, rows, dim, stream);
 }
 
 __device__ __forceinline__ float gate_of(float g, int kind) {

@@ -6,6 +6,7 @@
 // sum over the chosen experts is the one product's sum over K, with the weight of an expert that was not chosen
 // being zero.
 #include "api.h"
+#include "activations.h"
 #include "common.h"
 
 #define EXPERTS_MAX 1024
@@ -14,7 +15,7 @@
 // token's own row on, times its weight; it has no matrices and is the business of whoever adds the experts up).
 //   scores:  s = sigmoid(z) or softmax(z) over all outputs (float32; the softmax with its maximum taken off);
 //   choice:  by s + correction; with groups, the outputs form `groups` equal runs of neighbours, a group's score is
-//            its largest choice score, and only outputs of the `keep` best groups can be chosen (the others count as
+//            the sum of its `best_of` (1 or 2) largest choice scores, and only outputs of the `keep` best groups can be chosen (the others count as
 //            minus infinity); the `top` largest, the lower index on a tie;
 //   weights: the chosen outputs' s, divided by their sum (+ 1e-20) when `normalize`.
 // z rows have z_stride >= outs columns; with `extra`, extra[t, 0] is the sum of the weights of the identity experts
@@ -26,7 +27,7 @@ __global__ void __launch_bounds__(64)
 experts_route_kernel(int32_t* __restrict__ ids, float* __restrict__ weights, float* __restrict__ dense,
                      float* __restrict__ extra, const float* __restrict__ z, int z_stride,
                      const float* __restrict__ correction, int outs, int experts, int top, int kind, int normalize,
-                     int groups, int keep) {
+                     int groups, int keep, int best_of) {
     __shared__ float sc[EXPERTS_MAX], ch[EXPERTS_MAX], gbest[EXPERTS_MAX];
     const int t = blockIdx.x, lane = threadIdx.x;
     const float* zt = z + (size_t)t * z_stride;
@@ -54,9 +55,13 @@ experts_route_kernel(int32_t* __restrict__ ids, float* __restrict__ weights, flo
     if (groups > 1 && keep < groups) {
         const int per = outs / groups;
         for (int g = lane; g < groups; g += RI_WAVE) {
-            float best = -INFINITY;
-            for (int e = g * per; e < (g + 1) * per; ++e) best = fmaxf(best, ch[e]);
-            gbest[g] = best;
+            float best = -INFINITY, second = -INFINITY;
+            for (int e = g * per; e < (g + 1) * per; ++e) {
+                const float c = ch[e];
+                second = fmaxf(second, fminf(best, c));
+                best = fmaxf(best, c);
+            }
+            gbest[g] = best_of > 1 && per > 1 ? best + second : best;
         }
         __syncthreads();
         for (int g = lane; g < groups; g += RI_WAVE) {
@@ -202,6 +207,55 @@ experts_down_rows_kernel(float* __restrict__ out, const bf16_t* __restrict__ act
     if (lane == 0) out[(size_t)t * dim + n] = acc + own;
 }
 
+// The same for experts without a gate: up row i alone, u: [experts, ff, dim] rows.
+__global__ void __launch_bounds__(256)
+experts_up_rows_kernel(bf16_t* __restrict__ act, const bf16_t* __restrict__ x, const bf16_t* __restrict__ up,
+                       const int32_t* __restrict__ ids, const float* __restrict__ weights, int top, int ff, int dim, int kind) {
+    const int lane = threadIdx.x & 63, i = blockIdx.x * 4 + (threadIdx.x >> 6), pair = blockIdx.y;
+    if (i >= ff) return;                                      // (whole wavefronts)
+    const bf16_t* xr = x + (size_t)(pair / top) * dim;
+    const bf16_t* ur = up + ((size_t)ids[pair] * ff + i) * dim;
+    float u = 0.f;
+    for (int c = lane * 8; c < dim; c += 2048) {              // four pieces a turn, all asked for before any is used
+        uint4 b[4], v[4];
+#pragma unroll
+        for (int q = 0; q < 4; ++q) {
+            const int at = c + q * 512 < dim ? c + q * 512 : c;        // past the row's end: a piece that is there, not used
+            b[q] = load_stream16(ur + at);
+            v[q] = *reinterpret_cast<const uint4*>(xr + at);
+        }
+#pragma unroll
+        for (int q = 0; q < 4; ++q) {
+            if (c + q * 512 >= dim) continue;
+            const uint32_t bw[4] = {b[q].x, b[q].y, b[q].z, b[q].w}, vw[4] = {v[q].x, v[q].y, v[q].z, v[q].w};
+#pragma unroll
+            for (int k = 0; k < 4; ++k)
+                u += __uint_as_float(bw[k] << 16) * __uint_as_float(vw[k] << 16) +
+                     __uint_as_float(bw[k] & 0xFFFF0000u) * __uint_as_float(vw[k] & 0xFFFF0000u);
+        }
+    }
+    u = wave_sum(u);
+    // (the product's result passes through bfloat16, as it does where the product is a kernel of its own)
+    if (lane == 0) act[(size_t)pair * ff + i] = f32_to_bf16(weights[pair] * pn_activate(bf16_to_f32(f32_to_bf16(u)), kind));
+}
+
+extern "C" int ri_experts_few_tokens_plain(float* out, void* act, const void* x, const void* up, const void* down,
+                                           const int32_t* ids, const float* weights, int tokens, int experts, int top, int ff,
+                                           int dim, int kind, void* stream) {
+    RI_REQUIRE(tokens > 0 && experts >= 1 && top >= 1, "experts_few_tokens: %d tokens, %d of %d experts", tokens, top, experts);
+    RI_REQUIRE(ff >= 8 && ff % 8 == 0 && dim >= 8 && dim % 8 == 0, "experts_few_tokens: sizes %d and %d must be multiples of 8", ff, dim);
+    RI_REQUIRE((long)tokens * top <= 65535 && tokens <= 65535, "experts_few_tokens: %d tokens exceed one launch", tokens);
+    RI_REQUIRE(kind >= PN_ACT_GELU_ERF && kind <= PN_ACT_RELU2, "experts_few_tokens: activation %d", kind);
+    hipStream_t s = (hipStream_t)stream;
+    experts_up_rows_kernel<<<dim3((ff + 3) / 4, tokens * top), 256, 0, s>>>((bf16_t*)act, (const bf16_t*)x, (const bf16_t*)up, ids,
+                                                                          weights, top, ff, dim, kind);
+    RI_LAUNCH_CHECK("experts_few_tokens (up)");
+    experts_down_rows_kernel<<<dim3((dim + 3) / 4, tokens), 256, 0, s>>>(out, (const bf16_t*)act, (const bf16_t*)down, ids,
+                                                                       top, ff, dim, experts, (const bf16_t*)x, weights);
+    RI_LAUNCH_CHECK("experts_few_tokens (down)");
+    return 0;
+}
+
 extern "C" int ri_experts_few_tokens(float* out, void* act, const void* x, const void* gu, const void* down,
                                      const int32_t* ids, const float* weights, int tokens, int experts, int top, int ff,
                                      int dim, float limit, void* stream) {
@@ -339,7 +393,8 @@ extern "C" int ri_experts_combine(float* out, const void* y, const int32_t* dest
 
 extern "C" int ri_experts_route_general(int32_t* ids, float* weights, float* dense, float* extra, const float* z, int z_stride,
                                         const float* correction, int tokens, int outs, int experts, int top, int kind,
-                                        int normalize, int groups, int keep, void* stream) {
+                                        int normalize, int groups, int keep, int best_of, void* stream) {
+    RI_REQUIRE(best_of == 1 || best_of == 2, "experts_route: groups scored by their %d best", best_of);
     RI_REQUIRE(tokens > 0 && experts >= 0 && experts <= outs && outs >= 1 && outs <= EXPERTS_MAX && top >= 1 && top <= outs,
                "experts_route: %d tokens, the %d best of %d outputs (%d experts; at most %d)", tokens, top, outs, experts, EXPERTS_MAX);
     RI_REQUIRE(kind == ROUTE_SIGMOID || kind == ROUTE_SOFTMAX, "experts_route: score kind %d", kind);
@@ -347,7 +402,7 @@ extern "C" int ri_experts_route_general(int32_t* ids, float* weights, float* den
                "experts_route: %d outputs in %d groups of which %d stay, for the %d best", outs, groups, keep, top);
     RI_REQUIRE(z_stride >= outs, "experts_route: logit rows of %d for %d outputs", z_stride, outs);
     experts_route_kernel<<<tokens, 64, 0, (hipStream_t)stream>>>(ids, weights, dense, extra, z, z_stride, correction, outs,
-                                                                  experts, top, kind, normalize, groups, keep);
+                                                                  experts, top, kind, normalize, groups, keep, best_of);
     RI_LAUNCH_CHECK("experts_route");
     return 0;
 }
@@ -355,7 +410,7 @@ extern "C" int ri_experts_route_general(int32_t* ids, float* weights, float* den
 extern "C" int ri_experts_route(int32_t* ids, float* weights, float* dense, const float* z, const float* correction,
                                 int tokens, int experts, int top, void* stream) {
     return ri_experts_route_general(ids, weights, dense, nullptr, z, experts, correction, tokens, experts, experts, top,
-                                    ROUTE_SIGMOID, 1, 1, 1, stream);
+                                    ROUTE_SIGMOID, 1, 1, 1, 1, stream);
 }
 
 extern "C" int ri_experts_activate_strided(void* out, const void* gu, int dtype, const float* dense, int dense_stride,

@@ -12,6 +12,7 @@
 // The residual, the statistics, alpha and every activation are float32; a value is rounded once, when it is stored in
 // the activations' format.  One workgroup a row; a row's sums are taken in an order that the row's width alone fixes.
 #include "api.h"
+#include "activations.h"
 #include "common.h"
 
 #define PN_NORM_RMS 1
@@ -241,17 +242,6 @@ extern "C" int ri_glu_clamped_bias(void* out, const void* gu, int dtype, const f
 }
 
 // ------------------------------------------------------------------ experts without a gate
-#define PN_ACT_GELU_ERF 0
-#define PN_ACT_GELU_TANH 1
-#define PN_ACT_RELU2 2
-
-__device__ __forceinline__ float pn_activate(float v, int kind) {
-    if (kind == PN_ACT_GELU_ERF) return 0.5f * v * (1.f + erff(v * 0.7071067811865476f));
-    if (kind == PN_ACT_GELU_TANH) return 0.5f * v * (1.f + tanhf(0.7978845608028654f * (v + 0.044715f * v * v * v)));
-    const float r = fmaxf(v, 0.f);
-    return r * r;
-}
-
 template <typename T>
 __global__ void __launch_bounds__(256)
 experts_activate_plain_kernel(T* __restrict__ out, const T* __restrict__ u, const float* __restrict__ dense,

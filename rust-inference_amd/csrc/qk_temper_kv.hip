@@ -11,6 +11,7 @@
 // the general kernel; prompts of head sizes that allow it go through the 16-byte kernels further down.
 #include "api.h"
 #include "common.h"
+#include "kv_pages.h"
 
 #define QT_MAX_PER_LANE 8    // head sizes up to 64 * 8
 
@@ -69,33 +70,6 @@ __global__ void qk_norm_temper_kv_write_kernel(
 // power-of-two fraction (dim 8, 16, ... 512): a lane takes eight consecutive elements of a q or k head, so dim / 8
 // lanes make a head and a wavefront works on 512 / dim heads at once, every load and store 16 bytes (32 for
 // float32); one workgroup a token.  Values are written by the page-wise kernel below.
-template <typename T> struct Eight;
-template <> struct Eight<float> {
-    __device__ static void load(const float* p, float* o) {
-        const float4 a = *reinterpret_cast<const float4*>(p), b = *reinterpret_cast<const float4*>(p + 4);
-        o[0] = a.x; o[1] = a.y; o[2] = a.z; o[3] = a.w; o[4] = b.x; o[5] = b.y; o[6] = b.z; o[7] = b.w;
-    }
-    __device__ static void store(float* p, const float* v) {
-        *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]);
-        *reinterpret_cast<float4*>(p + 4) = make_float4(v[4], v[5], v[6], v[7]);
-    }
-};
-template <> struct Eight<bf16_t> {
-    __device__ static void load(const bf16_t* p, float* o) {
-        const uint4 v = *reinterpret_cast<const uint4*>(p);
-        const uint32_t w[4] = {v.x, v.y, v.z, v.w};
-#pragma unroll
-        for (int i = 0; i < 4; ++i) {
-            o[2 * i] = __uint_as_float(w[i] << 16);
-            o[2 * i + 1] = __uint_as_float(w[i] & 0xFFFF0000u);
-        }
-    }
-    __device__ static void store(bf16_t* p, const float* v) {
-        *reinterpret_cast<uint4*>(p) = make_uint4(pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3]),
-                                                  pack_bf16x2(v[4], v[5]), pack_bf16x2(v[6], v[7]));
-    }
-};
-
 template <typename TA, typename TC>
 __global__ void __launch_bounds__(256)
 qk_norm_temper_k_write_vec_kernel(TA* __restrict__ qkv, const float* __restrict__ q_gain, const float* __restrict__ k_gain,
@@ -142,59 +116,6 @@ qk_norm_temper_k_write_vec_kernel(TA* __restrict__ qkv, const float* __restrict_
     }
 }
 
-// Values into their pages, a page at a time: one workgroup per (32 positions touched by this step, sequence, kv
-// head) reads the new tokens' value heads as rows, turns them through LDS and writes channel rows.
-#define QT_TOKENS 32
-template <typename TA, typename TC>
-__global__ void __launch_bounds__(256)
-values_to_pages_kernel(const TA* __restrict__ qkv, size_t row_len, size_t v_off, const int32_t* __restrict__ cu_seqlens,
-                       const int32_t* __restrict__ tok_pos, const int32_t* __restrict__ page_table, int table_width,
-                       TC* __restrict__ v_pages, int kv_heads, int vdim, int page_size) {
-    extern __shared__ float tile[];                          // [QT_TOKENS][vdim + 1]
-    const int b = blockIdx.y, kvh = blockIdx.z;
-    const int t_begin = cu_seqlens[b], n = cu_seqlens[b + 1] - t_begin;
-    if (n <= 0) return;
-    const int start = tok_pos[t_begin];                      // the sequence's new tokens sit at start .. start + n - 1
-    const int first = (start / QT_TOKENS + blockIdx.x) * QT_TOKENS;
-    const int lo = max(first, start), hi = min(first + QT_TOKENS - 1, start + n - 1);
-    if (lo > hi) return;
-    const int stride = vdim + 1;
-    const TA* from = qkv + v_off + (size_t)kvh * vdim;
-    const bool whole = lo == first && hi == first + QT_TOKENS - 1;
-    if (sizeof(TA) == 2 && whole && vdim % 8 == 0 && (row_len % 8) == 0 && (v_off % 8) == 0) {
-        const int pieces = vdim / 8;
-        for (int e = threadIdx.x; e < QT_TOKENS * pieces; e += blockDim.x) {
-            const int tt = e / pieces, d = (e - tt * pieces) * 8;
-            float v[8];
-            Eight<TA>::load(from + (size_t)(t_begin + first - start + tt) * row_len + d, v);
-#pragma unroll
-            for (int j = 0; j < 8; ++j) tile[tt * stride + d + j] = v[j];
-        }
-    } else {
-        for (int e = threadIdx.x; e < (hi - lo + 1) * vdim; e += blockDim.x) {
-            const int tt = e / vdim, d = e - tt * vdim;
-            tile[(lo - first + tt) * stride + d] = to_f32(from[(size_t)(t_begin + lo - start + tt) * row_len + d]);
-        }
-    }
-    __syncthreads();
-    const int page = page_table[(size_t)b * table_width + first / page_size];
-    TC* base = v_pages + ((size_t)page * kv_heads + kvh) * page_size * vdim + first % page_size;
-    if (whole && page_size % 8 == 0) {
-        for (int e = threadIdx.x; e < vdim * (QT_TOKENS / 8); e += blockDim.x) {
-            const int d = e / (QT_TOKENS / 8), t8 = (e - d * (QT_TOKENS / 8)) * 8;
-            float v[8];
-#pragma unroll
-            for (int j = 0; j < 8; ++j) v[j] = tile[(t8 + j) * stride + d];
-            Eight<TC>::store(base + (size_t)d * page_size + t8, v);
-        }
-    } else {
-        for (int e = threadIdx.x; e < vdim * QT_TOKENS; e += blockDim.x) {
-            const int d = e / QT_TOKENS, tt = e - d * QT_TOKENS;
-            if (first + tt >= lo && first + tt <= hi) from_f32(base + (size_t)d * page_size + tt, tile[tt * stride + d]);
-        }
-    }
-}
-
 template <typename TA, typename TC>
 static void launch_qk_temper(void* qkv, const float* q_gain, const float* k_gain, float eps, float temp_coef, int temp_every,
                              const int32_t* tok_pos, const int32_t* tok_seq, const int32_t* cu_seqlens, int seqs, int max_new,
@@ -212,7 +133,7 @@ static void launch_qk_temper(void* qkv, const float* q_gain, const float* k_gain
         dim3 grid((max_new + QT_TOKENS - 2) / QT_TOKENS + 1, seqs, kv_heads);      // the 32-position pieces a sequence may touch
         values_to_pages_kernel<TA, TC><<<grid, 256, QT_TOKENS * (vdim + 1) * sizeof(float), s>>>(
             (const TA*)qkv, row_len, (size_t)(heads + kv_heads) * dim, cu_seqlens, tok_pos, page_table, table_width,
-            (TC*)v_pages, kv_heads, vdim, page_size);
+            (TC*)v_pages, kv_heads, vdim, page_size, nullptr);
         return;
     }
     const long items = (long)tokens * (heads + 2 * kv_heads);
@@ -437,7 +358,7 @@ extern "C" int ri_qk_pairs_norm_kv_write(void* proj, int act_dtype, long row_len
     values_to_pages_kernel<T, T><<<dim3((max_new + QT_TOKENS - 2) / QT_TOKENS + 1, seqs, kv_heads), 256,                   \
                                    QT_TOKENS * (vdim + 1) * sizeof(float), s>>>(                                          \
         (const T*)proj, (size_t)row_len, (size_t)v_off, cu_seqlens, tok_pos, page_table, table_width, (T*)v_pages,        \
-        kv_heads, vdim, page_size)
+        kv_heads, vdim, page_size, nullptr)
         if (act_dtype == RI_F32) { RI_VEC(float); } else { RI_VEC(bf16_t); }
 #undef RI_VEC
         RI_LAUNCH_CHECK("qk_pairs_norm_kv_write");
@@ -458,7 +379,7 @@ extern "C" int ri_qk_pairs_norm_kv_write(void* proj, int act_dtype, long row_len
         dim3 grid((max_new + QT_TOKENS - 2) / QT_TOKENS + 1, seqs, kv_heads);                                            \
         values_to_pages_kernel<T, T><<<grid, 256, QT_TOKENS * (vdim + 1) * sizeof(float), s>>>(                           \
             (const T*)proj, (size_t)row_len, (size_t)v_off, cu_seqlens, tok_pos, page_table, table_width, (T*)v_pages,    \
-            kv_heads, vdim, page_size);                                                                                 \
+            kv_heads, vdim, page_size, nullptr);                                                                        \
     }
     if (act_dtype == RI_F32) { RI_GO(float) } else { RI_GO(bf16_t) }
 #undef RI_GO

@@ -253,7 +253,8 @@ def build_emulated(out_dir: str, patches: dict | None = None) -> str:
     os.makedirs(gen, exist_ok=True)
     for name in os.listdir(CSRC):
         if name.endswith(".h"):
-            shutil.copy(os.path.join(CSRC, name), os.path.join(gen, name))
+            with open(os.path.join(CSRC, name)) as f, open(os.path.join(gen, name), "w") as g:
+                g.write(_rewrite_launches(f.read()))
     objs = []
     jobs = []
     for src in sources():

@@ -118,12 +118,21 @@ _SIGNATURES = {
     "ri_embed_scaled": [c_void_p, c_void_p, c_int, c_void_p, c_int, c_void_p, c_float, c_int, c_int, c_void_p],
     "ri_branch_norm_add": [c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_void_p, c_void_p, c_float, c_int, c_void_p,
                            c_int, c_int, c_void_p],
+    "ri_branch_norm_add_norm": [c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_void_p, c_void_p, c_float, c_int, c_void_p,
+                                c_void_p, c_float, c_int, c_int, c_int, c_void_p],
+    "ri_embed_bigram": [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
+                        ctypes.c_long, ctypes.c_long, ctypes.c_long, c_int, c_int, c_void_p],
+    "ri_qk_half_bias_kv_write": [c_void_p, c_int, ctypes.c_long, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int,
+                                 c_float, c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p, c_int, c_void_p, c_void_p, c_int,
+                                 c_int, c_int, c_int, c_int, c_int, c_int, c_void_p],
+    "ri_experts_few_tokens_plain": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int,
+                                    c_int, c_int, c_int, c_void_p],
     "ri_gate_rows": [c_void_p, c_int, c_int, c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_float, c_int, c_int, c_int,
                      c_void_p],
     "ri_row_norm_gate": [c_void_p, c_int, c_int, c_void_p, c_void_p, c_float, c_void_p, c_int, c_int, c_int, c_float, c_int,
                          c_int, c_int, c_void_p],
     "ri_experts_route_general": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_int,
-                                 c_int, c_int, c_int, c_int, c_int, c_void_p],
+                                 c_int, c_int, c_int, c_int, c_int, c_int, c_void_p],
     "ri_experts_activate_strided": [c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_int, c_float, c_void_p],
     "ri_experts_finish": [c_void_p, c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_int, c_void_p, c_int, c_int,
                           c_void_p],
@@ -252,6 +261,40 @@ def branch_norm_add(residual: torch.Tensor, y: torch.Tensor, gain, bias, eps: fl
           _opt(bias, "bias", torch.float32, (dim,)), float(eps), int(norm_kind),
           _opt(layer_scale, "layer_scale", torch.float32, (dim,)), rows, dim, _stream())
     return act
+
+
+def branch_norm_add_norm(residual: torch.Tensor, y: torch.Tensor, gain, bias, eps: float, norm_kind: int, layer_scale,
+                         next_gain: torch.Tensor, next_eps: float, act_dtype, tiled: bool = False):
+    """``branch_norm_add`` and, of the new residual, the RMS norm in front of the next sublayer, in one kernel: returns
+    ``residual / sqrt(mean(residual^2) + next_eps) * next_gain`` in ``act_dtype`` (with ``tiled`` as ``TiledRows``)."""
+    rows, dim = residual.shape
+    parts = y.shape[0] if y.dim() == 3 else 1
+    if tuple(y.shape[-2:]) != (rows, dim):
+        raise ShapeError(f"a branch output of {list(y.shape)} for a residual of {list(residual.shape)}")
+    out = TiledRows.empty(rows, dim, residual.device) if tiled else torch.empty((rows, dim), dtype=act_dtype, device=residual.device)
+    _call("ri_branch_norm_add_norm", _dev(residual, "residual", torch.float32), _dev(out.data if tiled else out, "out"), code(act_dtype),
+          _dev(y, "y"), code(y.dtype), parts, _dev(gain, "gain", torch.float32, (dim,)), _opt(bias, "bias", torch.float32, (dim,)),
+          float(eps), int(norm_kind), _opt(layer_scale, "layer_scale", torch.float32, (dim,)),
+          _dev(next_gain, "next_gain", torch.float32, (dim,)), float(next_eps), int(tiled), rows, dim, _stream())
+    return out
+
+
+def embed_bigram(table: torch.Tensor, pairs: torch.Tensor, ids, tok_pos, tok_seq, cu_seqlens, slots, last, mul_prev: int,
+                 mul_cur: int) -> torch.Tensor:
+    """float32 ``table[id] + pairs[row]`` for every token of a step: ``row`` is the last one for a token at position 0, else
+    ``(token before * mul_prev + id * mul_cur) mod buckets`` (``pairs`` has ``buckets + 1`` rows).  ``last`` (int32 ``[slots, 1]``)
+    holds every sequence's last token from step to step and is moved on."""
+    tokens, dim, seqs = ids.shape[0], table.shape[1], slots.shape[0]
+    buckets = pairs.shape[0] - 1
+    if buckets < 1 or pairs.shape[1] != dim or pairs.dtype != table.dtype:
+        raise ShapeError(f"a table of pairs of {list(pairs.shape)} {pairs.dtype} beside tokens of {list(table.shape)} {table.dtype}")
+    out = torch.empty((tokens, dim), dtype=torch.float32, device=table.device)
+    _call("ri_embed_bigram", _dev(out, "out"), _dev(table, "table"), _dev(pairs, "pairs"), code(table.dtype),
+          _dev(ids, "ids", torch.int32, (tokens,)), _dev(tok_pos, "tok_pos", torch.int32, (tokens,)),
+          _dev(tok_seq, "tok_seq", torch.int32, (tokens,)), _dev(cu_seqlens, "cu_seqlens", torch.int32, (seqs + 1,)),
+          _dev(slots, "slots", torch.int32, (seqs,)), _dev(last, "last", torch.int32, (last.shape[0], 1)), buckets,
+          int(mul_prev) % buckets, int(mul_cur) % buckets, tokens, dim, _stream())
+    return out
 
 
 def gate_rows(out: torch.Tensor, out_off: int, x: torch.Tensor, proj: torch.Tensor, g_off: int, scale: float,
@@ -475,6 +518,33 @@ def qk_pairs_norm_kv_write(proj, q_off: int, k_off: int, v_off: int, inv_freq, q
           _dev(k_pages, "k_pages", proj.dtype, (pages, kv_heads, page_size, dim)),
           _dev(v_pages, "v_pages", proj.dtype, (pages, kv_heads, vdim, page_size)), code(k_pages.dtype),
           tokens, heads, kv_heads, dim, vdim, page_size, _stream())
+
+
+def qk_half_bias_kv_write(proj, q_off: int, k_off: int, v_off: int, bias, inv_freq, amplitude: float, tok_pos, tok_seq, page_table,
+                          k_pages, v_pages, heads: int, kv_heads: int, dim: int, vdim: int, cu_seqlens=None,
+                          max_new: int = 0) -> None:
+    """In place on the projection rows ``proj [T, row]`` (q heads at column ``q_off``, k heads at ``k_off``, v heads at ``v_off``):
+    the biases (float32, q's then k's then v's, or None) are added, the elements ``(i, i + r)`` of every q and k head, ``r =
+    len(inv_freq)``, turn by ``pos * inv_freq[i]`` with cosine and sine times ``amplitude``; q stays in ``proj``, k and v go to their
+    pages.  ``kv_heads`` 0: queries alone (their layer reads another one's keys and values)."""
+    tokens, row = proj.shape
+    seqs = cu_seqlens.shape[0] - 1 if cu_seqlens is not None else 0
+    half = 0 if inv_freq is None else inv_freq.shape[0]
+    widths = (heads * dim, kv_heads * dim, kv_heads * vdim)
+    q_bias = k_bias = v_bias = None
+    if bias is not None:
+        q_bias = _dev(bias, "bias", torch.float32, (sum(widths),))
+        k_bias, v_bias = q_bias + 4 * widths[0], q_bias + 4 * (widths[0] + widths[1])
+    page_size, kv = 0, (None, None, proj.dtype)
+    if kv_heads:
+        pages, _, page_size, _ = k_pages.shape
+        kv = (_dev(k_pages, "k_pages", proj.dtype, (pages, kv_heads, page_size, dim)),
+              _dev(v_pages, "v_pages", proj.dtype, (pages, kv_heads, vdim, page_size)), k_pages.dtype)
+    _call("ri_qk_half_bias_kv_write", _dev(proj, "proj"), code(proj.dtype), row, int(q_off), int(k_off), int(v_off), q_bias, k_bias,
+          v_bias, _opt(inv_freq, "inv_freq", torch.float32), half, float(amplitude), _dev(tok_pos, "tok_pos", torch.int32, (tokens,)),
+          _dev(tok_seq, "tok_seq", torch.int32, (tokens,)), _opt(cu_seqlens, "cu_seqlens", torch.int32), seqs, int(max_new),
+          _dev(page_table, "page_table", torch.int32), page_table.shape[1], kv[0], kv[1], code(kv[2]), tokens, heads, kv_heads, dim,
+          vdim, page_size, _stream())
 
 
 def qk_norm_temper_kv_write(qkv, q_gain, k_gain, eps: float, temper, tok_pos, tok_seq, page_table, k_pages, v_pages,
@@ -792,10 +862,11 @@ ROUTE_SIGMOID, ROUTE_SOFTMAX = 0, 1
 
 
 def experts_route_general(z: torch.Tensor, correction: torch.Tensor, outs: int, experts: int, top: int, kind: int,
-                          normalize: bool, groups: int = 1, keep: int = 1):
+                          normalize: bool, groups: int = 1, keep: int = 1, best_of: int = 1):
     """The general router from float32 logits ``z [T, >= outs]``: scores ``s`` are the sigmoid or the softmax over the
     ``outs`` outputs (``experts`` real ones, then identity experts); the choice is by ``s + correction`` among the outputs of
-    the ``keep`` best of ``groups`` equal runs of neighbours (a group's score: its largest choice score); weights are the
+    the ``keep`` best of ``groups`` equal runs of neighbours (a group's score: the sum of its ``best_of``, one or two, largest
+    choice scores); weights are the
     chosen ``s``, over their sum with ``normalize``.  Returns ``ids``, ``weights`` ``[T, top]``, ``dense [T, outs]`` and
     ``extra [T, 2]`` (the identity experts' weight; the sigmoid of column ``outs`` of ``z`` where it has one)."""
     tokens, stride = z.shape
@@ -805,7 +876,7 @@ def experts_route_general(z: torch.Tensor, correction: torch.Tensor, outs: int, 
     extra = torch.empty((tokens, 2), dtype=torch.float32, device=z.device)
     _call("ri_experts_route_general", _dev(ids, "ids"), _dev(weights, "weights"), _dev(dense, "dense"), _dev(extra, "extra"),
           _dev(z, "z", torch.float32), stride, _dev(correction, "correction", torch.float32, (outs,)), tokens, outs, experts,
-          int(top), int(kind), int(bool(normalize)), int(groups), int(keep), _stream())
+          int(top), int(kind), int(bool(normalize)), int(groups), int(keep), int(best_of), _stream())
     return ids, weights, dense, extra
 
 
@@ -892,6 +963,22 @@ def experts_few_tokens(x, gate_up, down, ids, weights, ff: int, limit: float) ->
           _dev(gate_up, "gate_up", torch.bfloat16), _dev(down, "down", torch.bfloat16),
           _dev(ids, "ids", torch.int32, (tokens, top)), _dev(weights, "weights", torch.float32, (tokens, top)),
           tokens, experts, top, ff, dim, float(limit), _stream())
+    return out
+
+
+def experts_few_tokens_plain(x, up, down, ids, weights, ff: int, activation: str) -> torch.Tensor:
+    """``experts_few_tokens`` for experts without a gate: ``up [E * ff, dim]``."""
+    tokens, dim = x.shape
+    top = ids.shape[1]
+    experts = up.shape[0] // ff
+    if tuple(up.shape) != (experts * ff, dim) or tuple(down.shape) != (dim, experts * ff):
+        raise ShapeError(f"experts' matrices {list(up.shape)} and {list(down.shape)} for rows of {dim} and experts of {ff}")
+    out = torch.empty((tokens, dim), dtype=torch.float32, device=x.device)
+    act = torch.empty((tokens * top, ff), dtype=torch.bfloat16, device=x.device)
+    _call("ri_experts_few_tokens_plain", _dev(out, "out"), _dev(act, "act"), _dev(x, "x", torch.bfloat16),
+          _dev(up, "up", torch.bfloat16), _dev(down, "down", torch.bfloat16), _dev(ids, "ids", torch.int32, (tokens, top)),
+          _dev(weights, "weights", torch.float32, (tokens, top)), tokens, experts, top, ff, dim, PLAIN_ACTIVATIONS[activation],
+          _stream())
     return out
 
 

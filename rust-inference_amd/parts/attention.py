@@ -61,6 +61,13 @@ class GroupedQueryAttention(Mixer):
     heads of their own size are welcome there.  Such a mixer can also run beside another one on one input and one
     output product (``parts.parallel.ParallelMixers``): ``in_matrix``, ``core`` and ``out_matrix`` are its three
     steps taken apart.
+
+    A fourth family rotates halves like the first and may differ from it in all of this: biases on q, k and v beside a
+    ``v_dim``, a ``softcap``, a ``window`` (with ``keep_first``) and sinks; a rotation with an ``amplitude`` or over part of a head;
+    ``sinks="zero"``, a sink whose score is 0 for every head and which has no tensor (the softmax's denominator grows by
+    one); ``reads_kv``, a layer without keys and values of its own: its run names the cache entry of an earlier layer of
+    the same geometry, whose keys it reads as they lie there, rotated, with its own queries.  ``sinks="zero"``, ``reads_kv``
+    or a rotation with an amplitude sends the mixer through ``ops.qk_half_bias_kv_write``.
     """
 
     links_norms = True
@@ -69,7 +76,8 @@ class GroupedQueryAttention(Mixer):
                  eps: float = 1e-6, position: PartSpec | None = None, window: int | None = None,
                  qkv_bias: bool = False, o_bias: bool = False, v_dim: int | None = None, scale: float | None = None,
                  softcap: float | None = None, q_temper: tuple | None = None, names: dict | None = None,
-                 distance_slopes: tuple | None = None, keep_first: int = 0, sinks: bool = False, gate: str | None = None):
+                 distance_slopes: tuple | None = None, keep_first: int = 0, sinks: bool | str = False, gate: str | None = None,
+                 reads_kv: bool = False):
         if heads < 1 or kv_heads < 1 or heads % kv_heads:
             raise ConfigError(f"{heads} attention heads not divisible by {kv_heads} kv heads")
         if not 1 <= head_dim <= ops.MAX_HEAD_DIM:
@@ -94,14 +102,22 @@ class GroupedQueryAttention(Mixer):
             raise ConfigError(f"{len(self.distance_slopes)} distance slopes for {heads} heads")
         self.tempered = self.v_dim != head_dim or self.q_temper is not None or self.distance_slopes is not None
         self.position = build_part("position", position or PartSpec("none"))
-        self.keep_first, self.sinks, self.gate = int(keep_first or 0), bool(sinks), gate
+        self.zero_sink = sinks == "zero"
+        self.keep_first, self.sinks, self.gate = int(keep_first or 0), bool(sinks) and not self.zero_sink, gate
+        self.reads_kv, self.amplitude = bool(reads_kv), float(getattr(self.position, "amplitude", 1.0))
+        # biases, halves and the rest in one kernel: the fourth family
+        self.halved = self.zero_sink or self.reads_kv or self.amplitude != 1.0
+        if self.halved and (qk_norm or gate is not None or self.q_temper is not None or o_bias
+                            or getattr(self.position, "pairs", False) or getattr(self.position, "acts_after_norm", False)):
+            raise ConfigError("an attention that reads another layer's keys, has a sink of score 0 or a rotation with an "
+                              "amplitude takes no q/k norm, gate, query temperature or output bias, and rotates halves or not at all")
         if gate not in (None, "sigmoid", "silu"):
             raise ConfigError(f"an output gate {gate!r} is neither 'sigmoid' nor 'silu'")
         if self.keep_first < 0 or (self.keep_first and window is None):
             raise ConfigError(f"{keep_first} first tokens kept behind a window of {window}")
         # rotation of neighbours, unit norm, kept first tokens, sinks or a gate: the third family
-        self.paired = (getattr(self.position, "pairs", False) or qk_norm == "unit" or self.keep_first > 0 or self.sinks
-                       or gate is not None)
+        self.paired = not self.halved and (getattr(self.position, "pairs", False) or qk_norm == "unit" or self.keep_first > 0
+                                           or self.sinks or gate is not None)
         if self.paired and (self.q_temper is not None or qkv_bias or o_bias):
             raise ConfigError("an attention with a rotation of neighbours, kept first tokens, sinks or a gate takes no "
                               "query temperature and no biases")
@@ -109,22 +125,24 @@ class GroupedQueryAttention(Mixer):
             raise ConfigError("an attention with kept first tokens, sinks or a gate rotates neighbours or not at all")
         if self.paired and head_dim > 512:
             raise ConfigError(f"head_dim {head_dim}: the kernel that rotates neighbours takes up to 512")
-        if not self.paired and (self.tempered or self.softcap is not None) and (position is not None and position.kind != "none"):
+        if (not self.paired and not self.halved and (self.tempered or self.softcap is not None)) and (position is not None and position.kind != "none"):
             raise ConfigError("an attention with a score cap, a query temperature or value heads of their own size "
                               "takes no position encoding")
-        if (self.tempered or self.softcap is not None) and (qkv_bias or o_bias):
+        if not self.halved and (self.tempered or self.softcap is not None) and (qkv_bias or o_bias):
             raise ConfigError("an attention with a score cap, a query temperature or value heads of their own size "
                               "takes no biases")
         p = prefix
         self.names = {"q": p + "q_proj.weight", "k": p + "k_proj.weight", "v": p + "v_proj.weight",
                       "o": p + "o_proj.weight", "q_norm": p + "q_norm.weight", "k_norm": p + "k_norm.weight",
-                      "sink": p + "sink", "g": p + "g_proj.weight"}
+                      "sink": p + "sink", "g": p + "g_proj.weight", "q_bias": p + "q_proj.bias", "k_bias": p + "k_proj.bias",
+                      "v_bias": p + "v_proj.bias"}
         self.names.update(names or {})
         self.unit_norm = qk_norm == "unit"
         self.q_width, self.k_width, self.v_width = heads * head_dim, kv_heads * head_dim, kv_heads * self.v_dim
         self.out_width = heads * self.v_dim
         # the columns of this mixer's input product: q, k, v and, with a gate, g
-        self.in_width = self.q_width + self.k_width + self.v_width + (self.out_width if gate else 0)
+        self.projected = ("q",) if self.reads_kv else ("q", "k", "v", "g") if gate else ("q", "k", "v")
+        self.in_width = self.q_width + (0 if self.reads_kv else self.k_width + self.v_width) + (self.out_width if gate else 0)
 
     def tensors(self):
         p, d, dh, n = self.prefix, self.hidden, self.head_dim, self.names
@@ -134,6 +152,8 @@ class GroupedQueryAttention(Mixer):
             n["v"]: TensorSpec((self.kv_heads * self.v_dim, d), MATRIX),
             n["o"]: TensorSpec((d, self.heads * self.v_dim), MATRIX),
         }
+        if self.reads_kv:
+            del t[n["k"]], t[n["v"]]
         if self.qk_norm and not self.unit_norm:
             t[n["q_norm"]] = TensorSpec((dh,), GAIN)
             t[n["k_norm"]] = TensorSpec((dh,), GAIN)
@@ -142,9 +162,8 @@ class GroupedQueryAttention(Mixer):
         if self.gate:
             t[n["g"]] = TensorSpec((self.heads * self.v_dim, d), MATRIX)
         if self.qkv_bias:
-            t[p + "q_proj.bias"] = TensorSpec((self.heads * dh,), BIAS)
-            t[p + "k_proj.bias"] = TensorSpec((self.kv_heads * dh,), BIAS)
-            t[p + "v_proj.bias"] = TensorSpec((self.kv_heads * dh,), BIAS)
+            for x, width in zip(self.projected, (self.q_width, self.k_width, self.v_width)):
+                t[n[x + "_bias"]] = TensorSpec((width,), BIAS)
         if self.o_bias:
             t[p + "o_proj.bias"] = TensorSpec((d,), BIAS)
         t.update(self.position.tensors())
@@ -152,8 +171,7 @@ class GroupedQueryAttention(Mixer):
 
     def in_matrix(self, weights):
         """The rows of this mixer's input product, ``[q; k; v]`` and, with a gate, ``g``."""
-        n = self.names
-        return torch.cat([weights[n[x]] for x in (("q", "k", "v", "g") if self.gate else ("q", "k", "v"))], 0)
+        return torch.cat([weights[self.names[x]] for x in self.projected], 0)
 
     def out_matrix(self, weights):
         return weights[self.names["o"]]
@@ -170,9 +188,11 @@ class GroupedQueryAttention(Mixer):
         self.q_gain = rt.place_gain(weights[n["q_norm"]]) if gains else None
         self.k_gain = rt.place_gain(weights[n["k_norm"]]) if gains else None
         self.sink = rt.place_gain(weights[n["sink"]]) if self.sinks else None
+        if self.zero_sink:
+            self.sink = torch.zeros((self.heads,), dtype=torch.float32, device=rt.device)
         self.b_qkv = self.b_o = None
         if self.qkv_bias:
-            self.b_qkv = rt.place_gain(torch.cat([weights[p + n + "_proj.bias"] for n in "qkv"], 0))
+            self.b_qkv = rt.place_gain(torch.cat([weights[n[x + "_bias"]] for x in self.projected if x != "g"], 0))
         if self.o_bias:
             self.b_o = rt.place_gain(weights[p + "o_proj.bias"])
         self.position.bind(weights, rt)
@@ -180,6 +200,9 @@ class GroupedQueryAttention(Mixer):
                        if self.distance_slopes is not None else None)
 
     def bind_plain(self, weights):
+        if self.halved:
+            raise ConfigError("an attention that reads another layer's keys, has a sink of score 0 or a rotation with an "
+                              "amplitude has no plain form")
         if self.tempered or self.softcap is not None:
             raise ConfigError("an attention with a score cap, a query temperature or value heads of their own size has "
                               "no plain form")
@@ -226,8 +249,10 @@ class GroupedQueryAttention(Mixer):
         rt = self.rt
         with profiler.section(profiler.QKV_PROJECTION):
             qkv = rt.linear_packed(x, self.w_qkv)
-            if self.b_qkv is not None:
+            if self.b_qkv is not None and not self.halved:
                 ops.add_bias(qkv, self.b_qkv)
+        if self.halved:
+            return self.forward_halved(ops.as_rows(qkv), ctx, store, page_table)
         if self.paired:
             proj = ops.as_rows(qkv)
             heads = torch.empty((proj.shape[0], self.out_width), dtype=proj.dtype, device=proj.device)
@@ -272,6 +297,19 @@ class GroupedQueryAttention(Mixer):
         with profiler.section(profiler.ATTENTION):
             o = self.attend(qkv, ctx, store, page_table)
         return self.project_out(o, link)
+
+    def forward_halved(self, proj, ctx, store, page_table):
+        """Biases, rotation in halves and the write of k and v in one kernel (queries alone where the keys are another
+        layer's), then the attention over the entry the run names."""
+        own = 0 if self.reads_kv else self.kv_heads
+        with profiler.section(profiler.QK_NORM_ROPE_APPEND):
+            ops.qk_half_bias_kv_write(proj, 0, self.q_width, self.q_width + self.k_width, self.b_qkv, self.position.rotation_table(),
+                                      self.amplitude, ctx.tok_pos, ctx.tok_seq, page_table, store.k_pages, store.v_pages, self.heads,
+                                      own, self.head_dim, self.v_dim, ctx.cu_seqlens, ctx.max_new)
+        with profiler.section(profiler.ATTENTION):
+            o = self.attend_kept(proj, 0, ctx, store, page_table)
+        with profiler.section(profiler.OUT_PROJECTION):
+            return self.rt.linear_packed(o, self.w_o, out_dtype=torch.float32, parts_ok=True)
 
     def core(self, proj, col0: int, ctx, store, page_table, out, out_col: int, out_scale: float) -> None:
         """The mixer between its two products: ``proj [T, row]`` holds this mixer's q, k, v (and g) from column

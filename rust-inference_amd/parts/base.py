@@ -34,7 +34,9 @@ class Part:
 class Embedding(Part):
     """``forward(ctx) -> [T, hidden]`` float32: what the residual stream starts from.  The part gets the whole
     step's context, so one that adds something by position (``ctx.tok_pos``) or by sequence (``ctx.tok_seq``,
-    ``ctx.slots``) to the rows of its table needs nothing from the model."""
+    ``ctx.slots``) to the rows of its table needs nothing from the model.  An embedding that keeps something per
+    sequence says what with ``cache_need()`` (one need) and is called as ``forward(ctx, store)`` with its entry's storage
+    (``ModelSpec.embedding_cache``)."""
 
     def forward(self, ctx):
         raise NotImplementedError

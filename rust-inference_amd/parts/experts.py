@@ -33,8 +33,8 @@ class RoutedExperts(FeedForward):
 
     Other routers and experts, by parameter.  ``scores="softmax"``: ``s`` is the softmax over all of the router's
     outputs.  ``normalize=False``: the weights are the chosen ``s`` themselves.  ``groups=(count, keep)``: the outputs
-    form ``count`` equal groups of neighbours, a group's score is its largest ``s + correction``, and only outputs of the
-    ``keep`` best groups can be chosen.  ``identity=n``: the router has ``n`` more outputs after the experts', which
+    form ``count`` equal groups of neighbours, a group's score is its largest ``s + correction`` (``group_score="best"``) or the sum
+    of its two largest (``"best_two"``), and only outputs of the ``keep`` best groups can be chosen.  ``identity=n``: the router has ``n`` more outputs after the experts', which
     stand for experts that hand the token's own row on (times the weight) and have no tensors; they are scored,
     grouped and chosen like the others.  ``limit=None``: an expert is ``W_down (silu(W_gate h) (W_up h))``.
     ``gated=False, activation=...``: an expert is ``W_down act(W_up h)`` (``<prefix>e<i>.up`` and ``.down`` alone), ``act`` one of
@@ -47,7 +47,8 @@ class RoutedExperts(FeedForward):
 
     def __init__(self, hidden: int, inter: int, experts: int, top: int, limit: float | None, prefix: str,
                  scores: str = "sigmoid", normalize: bool = True, groups: tuple | None = None, identity: int = 0,
-                 shared: int | None = None, gated: bool = True, activation: str | None = None, router_bias: bool = False):
+                 shared: int | None = None, gated: bool = True, activation: str | None = None, router_bias: bool = False,
+                 group_score: str = "best"):
         self.outs = experts + int(identity)
         self.gated, self.activation, self.router_bias = bool(gated), activation, bool(router_bias)
         if not self.gated:
@@ -66,6 +67,9 @@ class RoutedExperts(FeedForward):
         self.limit = float(limit) if limit is not None else 0.0          # 0: the plain gated form
         self.scores, self.normalize, self.identity, self.shared = scores, bool(normalize), int(identity), shared
         self.groups, self.keep = (int(groups[0]), int(groups[1])) if groups else (1, 1)
+        if group_score not in ("best", "best_two"):
+            raise ConfigError(f"a group's score {group_score!r} is neither 'best' nor 'best_two'")
+        self.best_of = 2 if group_score == "best_two" else 1
         if self.outs % self.groups or not 1 <= self.keep <= self.groups or top > self.keep * (self.outs // self.groups):
             raise ConfigError(f"{self.outs} router outputs in {self.groups} groups of which {self.keep} stay, for the {top} best")
         # the router of the first designs: one kernel call and no extras
@@ -132,15 +136,19 @@ class RoutedExperts(FeedForward):
             else:
                 ids, weights, dense, extra = ops.experts_route_general(
                     z, self.correction, self.outs, self.experts, self.top,
-                    ops.ROUTE_SOFTMAX if self.scores == "softmax" else ops.ROUTE_SIGMOID, self.normalize, self.groups, self.keep)
+                    ops.ROUTE_SOFTMAX if self.scores == "softmax" else ops.ROUTE_SIGMOID, self.normalize, self.groups, self.keep,
+                    self.best_of)
             tokens = z.shape[0]
             routed = (rt.dtype == torch.bfloat16 and not rt.invariant and self.top < self.experts
                       and self.hidden % 8 == 0 and self.inter % 8 == 0)
-            few = routed and self.gated          # the kernel that reads the chosen experts' rows alone knows gated experts
             own = self.identity > 0                   # whether the identity experts' share is still to be added
-            if few and tokens * self.top < self.experts:
-                y, own = ops.experts_few_tokens(rt.normed_now(x), self.w_gate_up.w, self.w_down.w, ids, weights, self.inter,
-                                                self.limit), False
+            if routed and tokens * self.top < self.experts:
+                if self.gated:
+                    y, own = ops.experts_few_tokens(rt.normed_now(x), self.w_gate_up.w, self.w_down.w, ids, weights, self.inter,
+                                                    self.limit), False
+                else:
+                    y = ops.experts_few_tokens_plain(rt.normed_now(x), self.w_gate_up.w, self.w_down.w, ids, weights, self.inter,
+                                                     self.activation)
             elif (routed and tokens >= self.SORTED_MIN_TOKENS and not ctx.is_decode
                     and not torch.cuda.is_current_stream_capturing()):
                 y, own = self.forward_sorted(rt.normed_now(x), ids, weights), False

@@ -6,7 +6,7 @@ from __future__ import annotations
 
 import torch
 
-from ..cache import Cache, KVNeed
+from ..cache import Cache, KVNeed, StateNeed
 from ..config import load_config
 from ..errors import ConfigError, ShapeError
 from .. import profiler
@@ -84,6 +84,35 @@ class PositionedEmbedding(Embedding):
         return ops.embed_positions_norm(self.table, self.positions, ctx.tokens, ctx.tok_pos,
                                         n.gain if n is not None else None, getattr(n, "bias", None),
                                         n.eps if n is not None else 0.0, n.kind if n is not None else ops.NORM_NONE)
+
+
+@register_part("embedding", "table_bigram")
+class BigramEmbedding(Embedding):
+    """``h[t, :] = E[id_t, :] + B[row_t, :]`` with a row for the pair of the token before and the token, ``row_t = (id_{t-1} *
+    mul_prev + id_t * mul_cur) mod buckets``, and the table's last row (``buckets``) for a sequence's first token.  The last token
+    of every sequence is kept from step to step (an int32 a slot), so that a prompt cut anywhere reads the rows it reads whole."""
+
+    def __init__(self, vocab: int, dim: int, name: str, bigram_name: str, buckets: int, mul_prev: int, mul_cur: int):
+        if buckets < 1 or mul_prev < 0 or mul_cur < 0:
+            raise ConfigError(f"pairs of tokens in {buckets} buckets with the factors {mul_prev} and {mul_cur}")
+        self.vocab, self.dim, self.name, self.bigram_name = vocab, dim, name, bigram_name
+        self.buckets, self.mul_prev, self.mul_cur = int(buckets), int(mul_prev), int(mul_cur)
+
+    def tensors(self):
+        return {self.name: TensorSpec((self.vocab, self.dim), MATRIX),
+                self.bigram_name: TensorSpec((self.buckets + 1, self.dim), MATRIX)}
+
+    def bind(self, weights, rt):
+        self.rt = rt
+        self.table = rt.place_matrix(weights[self.name])
+        self.pairs = rt.place_matrix(weights[self.bigram_name]).to(self.table.dtype)
+
+    def cache_need(self):
+        return StateNeed((1,), torch.int32)
+
+    def forward(self, ctx, last):
+        return ops.embed_bigram(self.table, self.pairs, ctx.tokens, ctx.tok_pos, ctx.tok_seq, ctx.cu_seqlens, ctx.slots, last,
+                                self.mul_prev, self.mul_cur)
 
 
 @register_part("head", "linear")
@@ -269,6 +298,8 @@ class DecoderModel:
                 if needs[entry] is not None and needs[entry] != need:
                     raise ConfigError(f"cache entry {entry} is used with two different needs")
                 needs[entry] = need
+        if self.spec.embedding_cache is not None:
+            needs[self.spec.embedding_cache] = self.embedding.cache_need()
         return needs
 
     def new_cache(self, max_tokens: int, num_slots: int, max_seq_len: int | None = None, **kw) -> Cache:
@@ -286,7 +317,8 @@ class DecoderModel:
         """float32 logits ``[n_want, vocab]`` for the wanted rows of this step's tokens."""
         rt = self.rt
         with profiler.section(profiler.EMBEDDING):
-            hidden = self.embedding.forward(ctx)
+            kept = self.spec.embedding_cache
+            hidden = self.embedding.forward(ctx) if kept is None else self.embedding.forward(ctx, cache.state(kept))
         if self.stream_kind is None or self.stream_kind.kind == "residual":
             stream = ResidualStream(hidden)
             stream.links_ok = not rt.invariant

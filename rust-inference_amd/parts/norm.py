@@ -4,7 +4,7 @@ from __future__ import annotations
 import torch
 
 from ..kernels import ops, plain
-from ..weights.loader import BIAS, GAIN, TensorSpec
+from ..weights.loader import BIAS, GAIN, OFFSET, TensorSpec
 from .base import Norm
 from .registry import register_part
 
@@ -12,25 +12,31 @@ from .registry import register_part
 @register_part("norm", "rmsnorm")
 class RMSNorm(Norm):
     """``y = x * (1 / sqrt(mean(x^2) + eps)) * w`` over the last axis, statistics in
-    float32 (the reference: src/ops/norm.rs:7-32; fused with the add: :35-62)."""
+    float32 (the reference: src/ops/norm.rs:7-32; fused with the add: :35-62).  ``from_one``: the stored weight is the
+    gain's distance from one, ``w = 1 + stored``; ``scale``: a constant on the norm's output.  Both go into the float32 gain
+    when the weights are bound."""
 
     accepts_parts = True
     kind = ops.NORM_RMS      # what the kernel that also writes and reads several residual streams calls this norm
     linkable = True          # gain, eps and dim are all a product needs to do this norm itself
     can_tile = True          # hands its rows on in the matrix cores' order when asked (up to 64 rows)
 
-    def __init__(self, dim: int, eps: float, name: str):
-        self.dim, self.eps, self.name = dim, eps, name
+    def __init__(self, dim: int, eps: float, name: str, from_one: bool = False, scale: float = 1.0):
+        self.dim, self.eps, self.name, self.from_one, self.scale = dim, eps, name, bool(from_one), float(scale)
 
     def tensors(self):
-        return {self.name: TensorSpec((self.dim,), GAIN)}
+        return {self.name: TensorSpec((self.dim,), OFFSET if self.from_one else GAIN)}
+
+    def _gain(self, stored):
+        g = 1.0 + stored.to(torch.float32) if self.from_one else stored.to(torch.float32)
+        return g if self.scale == 1.0 else g * self.scale
 
     def bind(self, weights, rt):
         self.rt = rt
-        self.gain = rt.place_gain(weights[self.name])
+        self.gain = rt.place_gain(self._gain(weights[self.name]))
 
     def bind_plain(self, weights):
-        self.gain_plain = weights[self.name].to(torch.float32).numpy()
+        self.gain_plain = self._gain(weights[self.name]).numpy()
 
     def plain(self, x):
         return plain.rms_norm(x, self.gain_plain, self.eps)

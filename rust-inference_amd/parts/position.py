@@ -1,6 +1,8 @@
 """Position encodings."""
 from __future__ import annotations
 
+import math
+
 import torch
 
 from ..errors import ConfigError
@@ -13,15 +15,44 @@ class RotateHalf(PositionEncoding):
     """Rotary encoding of the "default" kind over the whole head, pairs ``(d, d + dh/2)``.
     ``inv_freq[i] = 1 / theta^(2i / dh)`` in float32 (the reference: src/ops/rope.rs:20);
     the kernel forms the angle ``f32(pos) * inv_freq[i]`` in float32 (:39) and rotates
-    ``x'[d] = x[d] cos - x[d+half] sin``, ``x'[d+half] = x[d+half] cos + x[d] sin`` (:73-74)."""
+    ``x'[d] = x[d] cos - x[d+half] sin``, ``x'[d+half] = x[d+half] cos + x[d] sin`` (:73-74).
 
-    def __init__(self, head_dim: int, theta: float):
-        if head_dim % 2:
+    ``dims``: only the first ``dims`` elements of a head turn (pairs ``(d, d + dims/2)``), with ``theta^(-2i / dims)`` taken in
+    64-bit and rounded once.  ``stretch = {factor, original, fast, slow}`` slows the pairs down for contexts ``factor`` times
+    as long as ``original``: with ``i(t) = dims ln(original / (2 pi t)) / (2 ln theta)``, the place of a pair that turns ``t`` times
+    in the original context, a pair's frequency runs from its own (``i <= floor(i(fast))``) to ``1/factor`` of it (``i >=
+    ceil(i(slow))``), linearly in ``i`` between; and ``amplitude = 0.1 ln(factor) + 1`` multiplies cosine and sine."""
+
+    amplitude = 1.0
+
+    def __init__(self, head_dim: int, theta: float, dims: int | None = None, stretch: dict | None = None):
+        if head_dim % 2 and dims is None:
             raise ConfigError(f"head_dim {head_dim} must be even for a rotation in pairs")
-        self.head_dim, self.theta = head_dim, theta
+        if dims is not None and (dims % 2 or not 2 <= dims <= head_dim):
+            raise ConfigError(f"a rotation over {dims} of {head_dim} elements: an even number up to the head size")
+        self.head_dim, self.theta, self.dims, self.stretch = head_dim, theta, dims, stretch
+        if stretch is not None:
+            self.dims = dims or head_dim
+            self.amplitude = 0.1 * math.log(stretch["factor"]) + 1.0
+
+    def part_frequencies(self) -> torch.Tensor:
+        """The frequencies of a rotation over part of a head, stretched or not (float64)."""
+        dims, base = self.dims, float(self.theta)
+        i = torch.arange(dims // 2, dtype=torch.float64)
+        f = torch.pow(torch.tensor(base, dtype=torch.float64), -2.0 * i / dims)
+        if self.stretch is None:
+            return f
+        s = self.stretch
+        place = lambda turns: dims * math.log(s["original"] / (2.0 * math.pi * turns)) / (2.0 * math.log(base))
+        first, last = max(math.floor(place(s["fast"])), 0), min(math.ceil(place(s["slow"])), dims - 1)
+        ramp = ((i - first) / max(last - first, 0.001)).clamp(0.0, 1.0)
+        return f / s["factor"] * ramp + f * (1.0 - ramp)
 
     def bind(self, weights, rt):
         self.rt = rt
+        if self.dims is not None:
+            self.inv_freq = self.part_frequencies().to(torch.float32).to(rt.device).contiguous()
+            return
         i = torch.arange(self.head_dim // 2, dtype=torch.float32)
         expo = (2.0 * i) / torch.tensor(float(self.head_dim), dtype=torch.float32)
         theta = torch.tensor(self.theta, dtype=torch.float32)
@@ -29,6 +60,8 @@ class RotateHalf(PositionEncoding):
 
     def bind_plain(self, weights):
         from ..kernels import plain
+        if self.dims is not None:
+            raise ConfigError("a rotation over part of a head, or with stretched frequencies, has no plain form")
         self.inv_freq_plain = plain.rope_inv_freq(self.head_dim, self.theta)
 
     def plain(self, heads, positions):

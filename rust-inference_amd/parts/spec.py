@@ -85,8 +85,12 @@ class ModelSpec:
     max_positions: int
     # how the residual is kept between the layers: "residual" (one float32 sum) or a kind with several streams
     stream: PartSpec = PartSpec("residual")
+    # the cache entry of an embedding that keeps something per sequence (its last token, for instance)
+    embedding_cache: Optional[int] = None
 
     @property
     def num_cache_entries(self) -> int:
         used = [e for r in self.schedule for e in r.entries()]
+        if self.embedding_cache is not None:
+            used.append(self.embedding_cache)
         return max(used) + 1 if used else 0

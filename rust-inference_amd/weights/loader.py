@@ -21,6 +21,7 @@ from .safetensors_io import ModelFolder
 
 MATRIX = "matrix"     # linear and embedding weights: N(0, 0.02) when random
 GAIN = "gain"         # norm gains: 1 + N(0, 0.1) when random; always used in 32-bit
+OFFSET = "offset"     # a norm gain's distance from 1: N(0, 0.1) when random; used in 32-bit like gains
 TABLE = "table"       # integer tables
 BIAS = "bias"         # biases of products: drawn like matrices when random, used in 32-bit like gains
 MIXING = "mixing"     # small square matrices that mix residual streams: identity + N(0, 0.1) when random; used in 32-bit
