@@ -2,7 +2,7 @@
 """Decode and prefill throughput of the Qwen3-8B-shaped model on one MI355X.
 
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--layers L] [--batch B] [--context C] [--model 8b|0.6b|1.7b|4b|14b|32b]
-    python bench.py --design zidepel|pisulorn|zakelorn|dagezen [--size 0.6b|8b] [--layers L]      # another workload: see design_comparison below
+    python bench.py --design zidepel|pisulorn|zakelorn|dagezen|notadra [--size 0.6b|8b] [--layers L]      # another workload: see design_comparison below
 
 The default run has the layer sizes of Qwen3-8B with random weights
 (N(0, 0.02), norm gains 1 + N(0, 0.1), seed 2), a batch of 8 and prompts of 2,048 tokens in a
@@ -268,6 +268,22 @@ def dagezen_like(q, layers, vocab, context):
             "layers": [(lat, par, ssm, par)[i % 4] for i in range(layers)]}
 
 
+def notadra_like(q, layers, vocab, context, vdim=None):
+    """A Notadra configuration with the layer sizes of a Qwen3 one: the same width, heads and head size (``vdim``: value heads
+    of another size), half of every head turned with frequencies stretched four times; of every four layers the fourth reads
+    the third's keys and values; of every four the first, the second and the fourth have eight experts of three quarters of
+    Qwen3's width in four groups of which two stay, two experts a token (two matrices of that width hold what three of half
+    Qwen3's width do, the experts of the other designs), the third has no feed-forward."""
+    d, h, g, dh, ff = q["hidden_size"], q["num_attention_heads"], q["num_key_value_heads"], q["head_dim"], q["intermediate_size"]
+    mixer = {"heads": h, "kv_heads": g, "dim": dh, "vdim": vdim or dh, "scale": dh ** -0.5, "softcap": 30.0,
+             "rot": {"dims": dh // 2, "base": 1e6, "scaling": {"factor": 4.0, "original": 32768, "fast": 32.0, "slow": 1.0}}}
+    moe = {"kind": "moe", "expert": {"ff": ff * 3 // 4}, "router": {"experts": 8, "top": 2, "groups": {"count": 4, "keep": 2}}}
+    return {"architecture": "Notadra", "vocab": vocab, "width": d, "norm": {"eps": 1e-5}, "logit_scale": 0.5,
+            "embedding": {"bigram": {"buckets": vocab // 2 - 3, "mul_prev": 8191, "mul_cur": 131}},
+            "layers": [{"type": "attention", "mixer": {**mixer, "kv_from": i - 1} if i % 4 == 3 else mixer, "mlp": None if i % 4 == 2 else moe}
+                       for i in range(layers)]}
+
+
 def design_comparison(args) -> int:
     """`--design zidepel`, `--design pisulorn` or `--design zakelorn`: prefill and decode of a model of that design beside the Qwen3 model
     of the same layer sizes (and, for Pisulorn, beside the Zidepel model of those sizes, the design closest to it)
@@ -275,6 +291,30 @@ def design_comparison(args) -> int:
     the output matrix are what is timed).  One JSON line; the default workload and its line are not touched."""
     sizes = {"0.6b": QWEN3_0_6B, "8b": QWEN3_8B}
     layers, vocab, context = args.layers or 8, 32768, args.context
+    if args.design == "notadra":
+        out = {"metric": "prefill and decode of the Notadra design beside Zakelorn and Qwen3 at equal layer sizes", "unit": "tok/s",
+               "n_gpus": 1, "dtype": "bf16", "data": "synthetic: random weights, uniform random token ids", "layers": layers,
+               "vocab": vocab, "steps": args.steps, "warmup": args.warmup, "sizes": {}}
+        for size in ([args.size] if args.size else ["0.6b", "8b"]):
+            q = dict(sizes[size], num_hidden_layers=layers, vocab_size=vocab, max_position_embeddings=context,
+                     tie_word_embeddings=False)
+            got = {}
+            for name, cfg in (("qwen3", q), ("zakelorn", zakelorn_like(q, layers, vocab, context)),
+                              ("notadra", notadra_like(q, layers, vocab, context)),
+                              ("notadra_vdim_5_4", notadra_like(q, layers, vocab, context, q["head_dim"] * 5 // 4))):
+                if args.only and name != args.only:
+                    continue
+                b = ShapeBench(f"{name} at Qwen3-{size} layer sizes", cfg, vocab, 11, context, not args.no_graphs)
+                got[name] = b.measure(args.prompt, (1, 8, 32), args.steps, args.warmup)
+                b.close()
+            out["sizes"][size] = got
+        first = out["sizes"][next(iter(out["sizes"]))]
+        if "notadra" in first:
+            out["value"], out["higher_is_better"] = first["notadra"]["decode_b8"]["tok_s"], True
+        if "notadra" in first and "zakelorn" in first:
+            out["vs_zakelorn_decode_b8"] = round(first["notadra"]["decode_b8"]["tok_s"] / first["zakelorn"]["decode_b8"]["tok_s"], 3)
+        print(json.dumps(out))
+        return 0
     if args.design == "dagezen":
         out = {"metric": "prefill and decode of the Dagezen design beside Zakelorn and Qwen3 at equal layer sizes", "unit": "tok/s",
                "n_gpus": 1, "dtype": "bf16", "data": "synthetic: random weights, uniform random token ids", "layers": layers,
@@ -369,10 +409,10 @@ def main() -> int:
     ap.add_argument("--no-points", action="store_true", help="skip the batch 1 and 64 points and the other models")
     ap.add_argument("--no-other-models", action="store_true", help="skip the Qwen3-0.6B and Qwen3-32B points")
     ap.add_argument("--no-graphs", action="store_true", help="launch every kernel of a decode step from the host")
-    ap.add_argument("--design", choices=["zidepel", "pisulorn", "zakelorn", "dagezen"], default=None,
+    ap.add_argument("--design", choices=["zidepel", "pisulorn", "zakelorn", "dagezen", "notadra"], default=None,
                     help="another workload: this design beside Qwen3 at equal layer sizes (prefill, decode at batch 1, 8, 32)")
     ap.add_argument("--size", choices=["0.6b", "8b"], default=None, help="with --design: one of the two layer sizes only")
-    ap.add_argument("--only", default=None, help="with --design dagezen: one of the models only (qwen3, zakelorn, dagezen)")
+    ap.add_argument("--only", default=None, help="with --design dagezen or notadra: one of the models only (qwen3, zakelorn, dagezen, notadra, notadra_vdim_5_4)")
     args = ap.parse_args()
     if args.gpus != 1:
         print(f"bench.py measures one GPU: this library is single-GPU, --gpus {args.gpus} is not run")

@@ -226,7 +226,7 @@ int ri_attention_decode_bf16(void* out, float* workspace, const void* qkv, int q
                              int kv_heads, int head_dim, int page_size, int window, float scale, float softcap,
                              const float* slopes, int tiled_out, void* stream);
 // The same with the first keep_first keys visible behind a window and a number per head (sinks, may be NULL) whose
-// exponential joins the softmax's denominator; for steps that ri_attention_decode_streams says do not stream.
+// exponential joins the softmax's denominator; kept keys only in steps that ri_attention_decode_streams says do not stream.
 int ri_attention_decode_kept_bf16(void* out, float* workspace, const void* qkv, int q_stride, const void* k_pages,
                                   const void* v_pages, const int32_t* cu_seqlens, const int32_t* tok_pos,
                                   const int32_t* page_table, int table_width, int seqs, int max_chunks, int heads,
@@ -481,6 +481,20 @@ int ri_ssd_scan_cols(float* out, const float* xbc, int channels, int b_off, int 
                      void* stream);
 int ri_group_rms_norm(void* out, int out_dtype, const float* x, const float* gain, float eps, int rows, int width, int parts,
                       void* stream);
+
+// Matrix-core attention for key and value heads of their own sizes (attention_mfma_padded.hip): dim a multiple of 8 up to
+// 128, vdim a multiple of 4 up to 256; otherwise as ri_attention_prefill_kept_bf16 and ri_attention_decode_kept_bf16.
+int ri_attention_padded_fits(int dim, int vdim, int group, int decode);
+int ri_attention_prefill_padded_bf16(void* out, const void* qkv, int q_stride, const void* k_pages, const void* v_pages,
+                                     const int32_t* cu_seqlens, const int32_t* tok_pos, const int32_t* page_table,
+                                     int table_width, int seqs, int max_new, int heads, int kv_heads, int dim, int vdim,
+                                     int page_size, int window, float scale, float softcap, const float* slopes,
+                                     int keep_first, const float* sinks, void* stream);
+int ri_attention_decode_padded_bf16(void* out, float* workspace, const void* qkv, int q_stride, const void* k_pages,
+                                    const void* v_pages, const int32_t* tok_pos, const int32_t* page_table, int table_width,
+                                    int seqs, int max_chunks, int heads, int kv_heads, int dim, int vdim, int page_size,
+                                    int window, float scale, float softcap, const float* slopes, int tiled_out,
+                                    int keep_first, const float* sinks, void* stream);
 
 // Biases, rotation in halves and the cache write (qk_half_bias_kv.hip).
 int ri_qk_half_bias_kv_write(void* proj, int act_dtype, long row_len, int q_off, int k_off, int v_off, const float* q_bias,

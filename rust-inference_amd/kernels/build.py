@@ -33,7 +33,7 @@ HIPCC_FLAGS = ["-O3", f"--offload-arch={ARCH}", "-fPIC", "-std=c++17", "-Wno-unu
 # take them for numbers, it first passes every operand through an instruction that quiets signalling NaNs
 # (IEEE mode), which is a fifth of the softmax's vector instructions.  The kernels produce no NaN from
 # numbers: a masked score is -inf, and a column without a key uses 0 as its reference point.
-FILE_FLAGS = {"attention_mfma.hip": ["-fno-honor-nans"]}
+FILE_FLAGS = {"attention_mfma.hip": ["-fno-honor-nans"], "attention_mfma_padded.hip": ["-fno-honor-nans"]}
 
 _lib = None
 

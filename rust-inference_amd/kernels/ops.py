@@ -118,6 +118,13 @@ _SIGNATURES = {
     "ri_embed_scaled": [c_void_p, c_void_p, c_int, c_void_p, c_int, c_void_p, c_float, c_int, c_int, c_void_p],
     "ri_branch_norm_add": [c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_void_p, c_void_p, c_float, c_int, c_void_p,
                            c_int, c_int, c_void_p],
+    "ri_attention_padded_fits": [c_int, c_int, c_int, c_int],
+    "ri_attention_prefill_padded_bf16": [c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int,
+                                         c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_void_p, c_int,
+                                         c_void_p, c_void_p],
+    "ri_attention_decode_padded_bf16": [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int,
+                                        c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_void_p, c_int,
+                                        c_int, c_void_p, c_void_p],
     "ri_branch_norm_add_norm": [c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_void_p, c_void_p, c_float, c_int, c_void_p,
                                 c_void_p, c_float, c_int, c_int, c_int, c_void_p],
     "ri_embed_bigram": [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
@@ -1014,6 +1021,62 @@ def attention_prefill_bf16(qkv, k_pages, v_pages, cu_seqlens, tok_pos, page_tabl
     return out
 
 
+def padded_attention_fits(dtype, dim: int, vdim: int, group: int, page_size: int, decode: bool) -> bool:
+    """Whether ``attention_prefill_padded`` (or, with ``decode``, ``attention_decode_padded``) takes these head sizes."""
+    return (dtype == torch.bfloat16 and page_size == 32
+            and bool(_get("ri_attention_padded_fits")(int(dim), int(vdim), int(group), int(decode))))
+
+
+def _padded_sizes(k_pages, v_pages, heads: int, kv_heads: int, stride: int, q_off: int):
+    pages, hkv, page_size, dim = k_pages.shape
+    vdim = v_pages.shape[2]
+    if hkv != kv_heads or tuple(v_pages.shape) != (pages, hkv, vdim, page_size):
+        raise ShapeError(f"pages are {list(k_pages.shape)} / {list(v_pages.shape)}, the mixer has {kv_heads} kv heads")
+    if q_off < 0 or q_off + heads * dim > stride or q_off % 8:
+        raise ShapeError(f"attention: queries at column {q_off} of rows of {stride} for {heads} heads of {dim}")
+    return dim, vdim, page_size
+
+
+def attention_prefill_padded(qkv, k_pages, v_pages, cu_seqlens, tok_pos, page_table, seqs: int, max_new: int, heads: int,
+                             kv_heads: int, window: int | None, scale: float, softcap: float | None = None,
+                             slopes: torch.Tensor | None = None, keep_first: int = 0, sinks: torch.Tensor | None = None,
+                             q_off: int = 0) -> torch.Tensor:
+    """``attention_prefill_bf16`` for key and value heads of their own sizes, which the pages give."""
+    tokens, stride = qkv.shape
+    dim, vdim, page_size = _padded_sizes(k_pages, v_pages, heads, kv_heads, stride, q_off)
+    out = torch.empty((tokens, heads * vdim), dtype=torch.bfloat16, device=qkv.device)
+    _call("ri_attention_prefill_padded_bf16", _dev(out, "out"), _dev(qkv, "qkv", torch.bfloat16) + 2 * int(q_off), stride,
+          _dev(k_pages, "k_pages", torch.bfloat16), _dev(v_pages, "v_pages", torch.bfloat16),
+          _dev(cu_seqlens, "cu_seqlens", torch.int32, (seqs + 1,)), _dev(tok_pos, "tok_pos", torch.int32, (tokens,)),
+          _dev(page_table, "page_table", torch.int32), page_table.shape[1], seqs, max_new, heads, kv_heads, dim, vdim, page_size,
+          int(window or 0), float(scale), float(softcap or 0.0), _opt(slopes, "slopes", torch.float32, (heads,)),
+          int(keep_first or 0), _opt(sinks, "sinks", torch.float32, (heads,)), _stream())
+    return out
+
+
+def attention_decode_padded(qkv, k_pages, v_pages, tok_pos, page_table, seqs: int, max_len: int, heads: int, kv_heads: int,
+                            window: int | None, scale: float, tiled_out: bool = False, softcap: float | None = None,
+                            slopes: torch.Tensor | None = None, keep_first: int = 0, sinks: torch.Tensor | None = None,
+                            q_off: int = 0):
+    """``attention_decode_bf16`` for key and value heads of their own sizes, which the pages give."""
+    tokens, stride = qkv.shape
+    if tokens != seqs:
+        raise ShapeError(f"decode attention takes one token per sequence, got {tokens} tokens for {seqs} sequences")
+    dim, vdim, page_size = _padded_sizes(k_pages, v_pages, heads, kv_heads, stride, q_off)
+    chunks = _get("ri_attention_decode_chunks")(int(max_len))      # the kernels' own chunk size
+    out = (TiledRows.empty(tokens, heads * vdim, qkv.device) if tiled_out else
+           torch.empty((tokens, heads * vdim), dtype=torch.bfloat16, device=qkv.device))
+    pieces = _get("ri_attention_decode_pieces")(int(seqs), int(kv_heads), int(heads), chunks)
+    ws = torch.empty((seqs, heads, chunks * pieces, vdim + 2), dtype=torch.float32, device=qkv.device)
+    _call("ri_attention_decode_padded_bf16", _dev(out.data if tiled_out else out, "out"), _dev(ws, "workspace"),
+          _dev(qkv, "qkv", torch.bfloat16) + 2 * int(q_off), stride, _dev(k_pages, "k_pages", torch.bfloat16),
+          _dev(v_pages, "v_pages", torch.bfloat16), _dev(tok_pos, "tok_pos", torch.int32, (tokens,)),
+          _dev(page_table, "page_table", torch.int32), page_table.shape[1], seqs, chunks, heads, kv_heads, dim, vdim, page_size,
+          int(window or 0), float(scale), float(softcap or 0.0), _opt(slopes, "slopes", torch.float32, (heads,)), int(tiled_out),
+          int(keep_first or 0), _opt(sinks, "sinks", torch.float32, (heads,)), _stream())
+    return out
+
+
 def decode_attention_runs(seqs: int, kv_heads: int, max_len: int) -> int:
     """The runs per sequence in which the decode attention's streaming kernel walks a step of this size, or 0
     where it takes one workgroup per chunk of 256 keys instead (host code only: it needs no GPU)."""
@@ -1034,7 +1097,7 @@ def attention_decode_bf16(qkv, k_pages, v_pages, cu_seqlens, tok_pos, page_table
     """Matrix-core attention for one new token per sequence; ``max_len`` bounds every sequence's length
     after this step (it sizes the grid and the workspace, not the result).  ``tiled_out``: the result as
     ``TiledRows`` (at most 64 sequences).  ``softcap`` and ``slopes`` as in ``attention_prefill_bf16``; ``keep_first``,
-    ``sinks`` and ``q_off`` as in ``attention`` (in steps for which ``decode_attention_streams`` is false)."""
+    ``sinks`` and ``q_off`` as in ``attention`` (``keep_first`` in steps for which ``decode_attention_streams`` is false)."""
     tokens, stride = qkv.shape
     if tokens != seqs:
         raise ShapeError(f"decode attention takes one token per sequence, got {tokens} tokens for {seqs} sequences")

@@ -328,19 +328,32 @@ class GroupedQueryAttention(Mixer):
                           ops.GATE_SILU if self.gate == "silu" else ops.GATE_SIGMOID)
 
     def attend_kept(self, proj, q_at, ctx, store, page_table):
-        """The attention of the third family: window with kept first tokens, sinks, value heads of any size."""
+        """The attention of the third and the fourth family: window with kept first tokens, sinks, value heads of any size."""
         slopes = getattr(self, "slopes", None)
         group = self.heads // self.kv_heads
-        fits = self.v_dim == self.head_dim and proj.shape[1] % 8 == 0 and q_at % 8 == 0
+        aligned = proj.shape[1] % 8 == 0 and q_at % 8 == 0
+        # (heads that no gate follows may come in the output product's own order)
+        tiled = self.halved and ctx.is_decode and not self.rt.invariant and self.rt.takes_tiled(self.w_o, ctx.B, True)
+        if self.halved and (self.v_dim != self.head_dim or self.head_dim not in ops.MFMA_HEAD_DIMS):
+            args = (self.heads, self.kv_heads, self.window, self.scale)
+            kw = {"softcap": self.softcap, "slopes": slopes, "keep_first": self.keep_first, "sinks": self.sink, "q_off": q_at}
+            sizes = (proj.dtype, self.head_dim, self.v_dim, group, store.page_size)
+            if aligned and ctx.is_decode and not self.rt.invariant and ops.padded_attention_fits(*sizes, True):
+                return ops.attention_decode_padded(proj, store.k_pages, store.v_pages, ctx.tok_pos, page_table, ctx.B, ctx.max_len, *args,
+                                                   tiled_out=tiled, **kw)
+            if aligned and ops.padded_attention_fits(*sizes, False):
+                return ops.attention_prefill_padded(proj, store.k_pages, store.v_pages, ctx.cu_seqlens, ctx.tok_pos, page_table, ctx.B,
+                                                    ctx.max_new, *args, **kw)
+        fits = self.v_dim == self.head_dim and aligned
         if (fits and ctx.is_decode and not self.rt.invariant
                 and ops.mfma_attention_fits(proj.dtype, self.head_dim, group, store.page_size, True)
-                and not ops.decode_attention_streams(ctx.B, self.kv_heads, ctx.max_len)):
-            # one new token a sequence in a step that does not fill the machine: the keys in chunks side by side, then
-            # the join, which adds the kept keys' chunks and the sink
+                and (self.keep_first == 0 or not ops.decode_attention_streams(ctx.B, self.kv_heads, ctx.max_len))):
+            # one new token a sequence: the keys in chunks side by side, then the join, which adds the kept keys' chunks
+            # and the sink; without kept keys also a step that fills the machine, whose keys are walked in runs
             return ops.attention_decode_bf16(proj, store.k_pages, store.v_pages, ctx.cu_seqlens, ctx.tok_pos, page_table,
                                              ctx.B, ctx.max_len, self.heads, self.kv_heads, self.head_dim, self.window,
-                                             self.scale, softcap=self.softcap, slopes=slopes, keep_first=self.keep_first,
-                                             sinks=self.sink, q_off=q_at)
+                                             self.scale, tiled_out=tiled, softcap=self.softcap, slopes=slopes,
+                                             keep_first=self.keep_first, sinks=self.sink, q_off=q_at)
         if fits and ops.mfma_attention_fits(proj.dtype, self.head_dim, group, store.page_size, False):
             # the matrix cores' prompt kernel, also for the single tokens of a step that fills the machine: a
             # wavefront walks a sequence's pages in their order

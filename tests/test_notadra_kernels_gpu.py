@@ -244,6 +244,96 @@ def test_generic_attention_with_a_cap_and_a_sink_of_zero(ops, dtype, heads, kv, 
     assert np.allclose(want[75].reshape(heads, vdim), np.repeat(v[75], heads // kv, 0) * (1 / (1 + np.exp(-s)))[:, None])
 
 
+PADDED = [(8, 4, 64, 80), (4, 1, 128, 160), (2, 2, 24, 36), (6, 3, 96, 96), (16, 1, 40, 64), (3, 3, 128, 252), (4, 2, 64, 128), (2, 1, 8, 4), (4, 4, 128, 72)]
+
+
+@pytest.mark.parametrize("heads, kv, dim, vdim", PADDED)
+@pytest.mark.parametrize("form", ["prompts", "single tokens", "portions"])
+def test_matrix_core_attention_with_head_sizes_of_their_own(ops, form, heads, kv, dim, vdim):
+    """bfloat16, key and value heads of sizes of their own: prompts of unequal lengths, one new token each, the last tokens
+    of each as a portion; a cap, a sink of 0; a scale at which a key can stand out."""
+    rng = np.random.default_rng(dim + heads)
+    lens = [75, 1, 40] if form == "prompts" else [300, 33, 164]
+    scale = 2.0 / dim ** 0.5
+    q, k, v, cu, want = attention_case(rng, lens, heads, kv, dim, vdim, scale, 6.0)
+    kp, vp, table = paged_batch(k, v, lens, dim)
+    rows, pos, new_cu = rows_of(lens, cu, {"prompts": None, "single tokens": 1, "portions": 19}[form])
+    wide = np.concatenate([np.full((len(rows), 16), 9.0), q[rows].reshape(len(rows), -1), np.full((len(rows), 8), 9.0)], 1)
+    kw = {"softcap": 6.0, "sinks": t(np.zeros(heads)), "q_off": 16}
+    assert ops.padded_attention_fits(torch.bfloat16, dim, vdim, heads // kv, PAGE, False)
+    got = ops.attention_prefill_padded(t(wide, torch.bfloat16), kp, vp, t(new_cu, torch.int32), t(pos, torch.int32), table, len(lens),
+                                       int(np.diff(new_cu).max()), heads, kv, None, scale, **kw)
+    close(got, want[rows], BF16_OUT, form)
+    if form == "single tokens":                               # the same in chunks side by side and their join
+        for tiled in (False, True):
+            got = ops.attention_decode_padded(t(wide, torch.bfloat16), kp, vp, t(pos, torch.int32), table, len(lens), max(lens), heads, kv,
+                                              None, scale, tiled, **kw)
+            close(ops.as_rows(got), want[rows], BF16_OUT, "chunks and join")
+
+
+def test_which_head_sizes_the_padded_kernels_take(ops):
+    fits = lambda *a: ops.padded_attention_fits(torch.bfloat16, *a)
+    assert fits(64, 80, 4, 32, True) and fits(128, 256, 16, 32, False) and fits(8, 4, 32, 32, False)
+    assert not fits(12, 80, 4, 32, True) and not fits(64, 82, 4, 32, True) and not fits(136, 64, 1, 32, False)
+    assert not fits(64, 260, 1, 32, False) and not fits(64, 80, 4, 16, True) and not fits(64, 200, 32, 32, False)
+    assert not ops.padded_attention_fits(torch.float32, 64, 80, 4, 32, True)
+
+
+@pytest.mark.parametrize("dim, vdim", [(64, 80), (128, 128)])
+def test_one_far_key_and_the_sink_in_thousands_of_keys(ops, dim, vdim):
+    """5,000 keys, more chunks than the short join takes at once; one key 4,968 tokens back answers loudly, at a page's
+    border; a query that answers to nothing leaves most of its weight to no key only if the sink counts."""
+    rng = np.random.default_rng(12)
+    T, heads = 5000, 4
+    q, k, v = rng.normal(size=(1, heads, dim)) * 0.2, rng.normal(size=(T, 2, dim)) * 0.2, rng.normal(size=(T, 2, vdim))
+    q[0, :2, 5] = 5.0
+    k[:, :, 6] = -3.0
+    q[0, 2:, 6] = 5.0                                         # two heads whose every score is near -15
+    k[31, :, 5] = 5.0
+    k[32, :, 5] = -5.0
+    q, k, v = bf16_round(q), bf16_round(k), bf16_round(v)
+    want = P.capped_attention(q, k, v, T - 1, 1.0, 20.0).reshape(1, -1)
+    assert np.abs(want[0, :vdim] - v[31, 0]).max() < 0.1 and np.abs(want[0, 2 * vdim:]).max() < 1e-2
+    kp, vp, table = paged_batch(k, v, [T], 3)
+    row, pos = t(q.reshape(1, -1), torch.bfloat16), t([T - 1], torch.int32)
+    if dim == vdim:
+        got = ops.attention_decode_bf16(row, kp, vp, t([0, 1], torch.int32), pos, table, 1, T, heads, 2, dim, None, 1.0, softcap=20.0,
+                                        sinks=t(np.zeros(heads)))
+    else:
+        got = ops.attention_decode_padded(row, kp, vp, pos, table, 1, T, heads, 2, None, 1.0, softcap=20.0, sinks=t(np.zeros(heads)))
+    close(got, want, BF16_OUT)
+
+
+@pytest.mark.parametrize("dim, vdim", [(64, 80), (32, 32), (128, 120)])
+@pytest.mark.parametrize("wide", [False, True])
+def test_single_tokens_of_many_sequences_walk_their_keys_in_runs_with_a_sink(ops, dim, vdim, wide):
+    """As many (sequence, kv head) pairs as make the step stream (with eight wavefronts a workgroup or with four); sequences
+    of one key to 150, a cap and the sink."""
+    from rust_inference_amd.kernels.build import load
+    rng = np.random.default_rng(dim)
+    units = load().ri_compute_units()
+    kv = 8
+    seqs = -(-(units * 9 // 10 if wide else 2 * units) // kv)
+    heads = 2 * kv
+    lens = [int(n) for n in rng.integers(1, 150, seqs)]
+    lens[0] = 1
+    if not ops.decode_attention_streams(seqs, kv, max(lens)):
+        pytest.skip("this machine's size leaves no such step")
+    T = sum(lens)
+    q, k, v = (bf16_round(rng.normal(size=(T, n, d))) for n, d in ((heads, dim), (kv, dim), (kv, vdim)))
+    cu = np.concatenate([[0], np.cumsum(lens)])
+    last = cu[1:] - 1
+    want = np.concatenate([P.capped_attention(q[b - 1:b], k[a:b], v[a:b], b - 1 - a, 0.2, 5.0).reshape(1, -1) for a, b in zip(cu[:-1], cu[1:])])
+    kp, vp, table = paged_batch(k, v, lens, dim)
+    row, pos, sinks = t(q[last].reshape(seqs, -1), torch.bfloat16), t(np.array(lens) - 1, torch.int32), t(np.zeros(heads))
+    if dim == vdim:
+        got = ops.attention_decode_bf16(row, kp, vp, t(np.arange(seqs + 1), torch.int32), pos, table, seqs, max(lens), heads, kv, dim, None, 0.2,
+                                        softcap=5.0, sinks=sinks)
+    else:
+        got = ops.attention_decode_padded(row, kp, vp, pos, table, seqs, max(lens), heads, kv, None, 0.2, softcap=5.0, sinks=sinks)
+    close(got, want, BF16_OUT)
+
+
 # ---------------------------------------------------------------- the router and the experts
 def router_case(seed, tokens, experts, spread=1.0):
     rng = np.random.default_rng(seed)
