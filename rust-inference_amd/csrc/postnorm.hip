@@ -254,6 +254,31 @@ experts_activate_plain_kernel(T* __restrict__ out, const T* __restrict__ u, cons
         from_f32(out + at + i, w == 0.f ? 0.f : w * pn_activate(to_f32(u[at + i]), kind));
 }
 
+// Widths that are a multiple of 8, bfloat16: a thread takes eight neighbours, 16 bytes there and back; an expert that was
+// not chosen is not read.
+__global__ void __launch_bounds__(256)
+experts_activate_plain_vec_kernel(bf16_t* __restrict__ out, const bf16_t* __restrict__ u, const float* __restrict__ dense,
+                                  int dense_stride, int experts, int ff, int kind) {
+    const size_t t = blockIdx.y;
+    const int e = blockIdx.x;
+    const float w = dense ? dense[t * dense_stride + e] : 1.f;
+    const size_t at = (t * experts + e) * ff;
+    for (int i = threadIdx.x * 8; i < ff; i += 256 * 8) {
+        uint4 o = make_uint4(0, 0, 0, 0);
+        if (w != 0.f) {
+            const uint4 v = *reinterpret_cast<const uint4*>(u + at + i);
+            const uint32_t x[4] = {v.x, v.y, v.z, v.w};
+            uint32_t y[4];
+#pragma unroll
+            for (int k = 0; k < 4; ++k)
+                y[k] = pack_bf16x2(w * pn_activate(__uint_as_float(x[k] << 16), kind),
+                                   w * pn_activate(__uint_as_float(x[k] & 0xFFFF0000u), kind));
+            o = make_uint4(y[0], y[1], y[2], y[3]);
+        }
+        *reinterpret_cast<uint4*>(out + at + i) = o;
+    }
+}
+
 extern "C" int ri_experts_activate_plain(void* out, const void* u, int dtype, const float* dense, int dense_stride,
                                          int tokens, int experts, int ff, int kind, void* stream) {
     RI_REQUIRE(tokens > 0 && experts >= 1 && experts <= 65535 && ff >= 1, "experts_activate_plain: %d tokens, %d experts of %d",
@@ -270,6 +295,9 @@ extern "C" int ri_experts_activate_plain(void* out, const void* u, int dtype, co
         if (dtype == RI_F32)
             experts_activate_plain_kernel<float><<<grid, 256, 0, s>>>((float*)out + at, (const float*)u + at, d, dense_stride,
                                                                      experts, ff, kind);
+        else if (ff % 8 == 0 && ((uintptr_t)out | (uintptr_t)u) % 16 == 0)
+            experts_activate_plain_vec_kernel<<<grid, 256, 0, s>>>((bf16_t*)out + at, (const bf16_t*)u + at, d, dense_stride,
+                                                                  experts, ff, kind);
         else
             experts_activate_plain_kernel<bf16_t><<<grid, 256, 0, s>>>((bf16_t*)out + at, (const bf16_t*)u + at, d, dense_stride,
                                                                       experts, ff, kind);

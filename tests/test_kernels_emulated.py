@@ -61,8 +61,11 @@ SAMPLER_TESTS = os.path.join(HERE, "test_sampling_gpu.py")
 ZIDEPEL_TESTS = os.path.join(HERE, "test_zidepel_kernels_gpu.py")
 PISULORN_TESTS = os.path.join(HERE, "test_pisulorn_kernels_gpu.py")
 ZAKELORN_TESTS = os.path.join(HERE, "test_zakelorn_kernels_gpu.py")
+NOTADRA_TESTS = os.path.join(HERE, "test_notadra_kernels_gpu.py")
 DAGEZEN_TESTS = os.path.join(HERE, "test_dagezen_kernels_gpu.py")
 PISULORN_SELECT = "not two_equal_keys and not many_sequences"      # not the 1,300 keys and the 512 workgroups on the emulated matrix cores (minutes)
+NOTADRA_SELECT = ("not many_sequences and not thousands_of_keys and not (matrix_core and not (64-80 or 24-36 or 128-252 or 40-64))"
+                  " and not 8192 and not 8200 and not 4100")          # a size of every capacity, not every size (minutes each)
 SAMPLER_SELECT = "(same_token_as_the_plain_sampler or top_p_drops) and not large"     # not the 151,936 entries, not the engine
 
 
@@ -85,6 +88,9 @@ def runs():
         "pisulorn": _start([*PYTEST, *_workers(2), PISULORN_TESTS, "-k", PISULORN_SELECT]),
         "zakelorn": _start([*PYTEST, *_workers(2), ZAKELORN_TESTS, "-k", "not thousands_of_keys"]),
         "dagezen": _start([*PYTEST, *_workers(2), DAGEZEN_TESTS]),
+        "notadra": _start([*PYTEST, *_workers(3), NOTADRA_TESTS, "-k", NOTADRA_SELECT]),
+        # (eight compute units: the decode attention then walks whole runs of keys for a few sequences already)
+        "notadra, eight units": _start([*PYTEST, *_workers(2), NOTADRA_TESTS, "-k", "many_sequences and 64-80"], {"RI_EMU_COMPUTE_UNITS": "8"}),
         # (with one compute unit a prompt of 70 tokens already takes the form of the rotation kernel that gives a
         # wavefront four heads of a token)
         "zakelorn, one unit": _start([*PYTEST, ZAKELORN_TESTS, "-k", "rotation_unit_norm"], {"RI_EMU_COMPUTE_UNITS": "1"}),
@@ -146,6 +152,14 @@ def test_the_kernels_of_the_dagezen_design_pass_on_the_cpu_build_between_guard_p
     windowed attention whose heads talk (whole and in shares of the keys), the time mixing and the state-space mixer in
     both forms of their walks."""
     _passed(runs["dagezen"])
+
+
+def test_the_kernels_of_the_notadra_design_pass_on_the_cpu_build_between_guard_pages(runs):
+    """tests/test_notadra_kernels_gpu.py: the embedding of pairs, the norms around a sublayer, biases with the rotation in
+    halves and the cache write, attention with a cap and a sink of 0 (generic and on the emulated matrix cores, head
+    sizes of their own), groups scored by their two best, experts without gates."""
+    _passed(runs["notadra"])
+    _passed(runs["notadra, eight units"], 2)
 
 
 @pytest.mark.parametrize("units, tests", [("sixteen units", 7), ("one unit", 61)])

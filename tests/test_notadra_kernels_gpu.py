@@ -382,3 +382,19 @@ def test_few_tokens_read_the_chosen_experts_alone(ops, tokens, experts, top, ff,
     down = np.concatenate([w[f"e{e}.down"] for e in range(experts)], 1)
     got = ops.experts_few_tokens_plain(t(x, torch.bfloat16), t(up, torch.bfloat16), t(down, torch.bfloat16), t(ids, torch.int32), t(weights), ff, "relu2")
     close(got, want, 2e-2)
+
+
+@pytest.mark.parametrize("activation", ["relu2", "gelu_erf", "gelu_tanh"])
+@pytest.mark.parametrize("dtype, ff", [(torch.bfloat16, 24), (torch.bfloat16, 2056), (torch.bfloat16, 21), (torch.float32, 24)])
+def test_the_experts_activation_with_and_without_weights(ops, dtype, ff, activation):
+    rng = np.random.default_rng(ff)
+    tokens, experts = 5, 3
+    u = bf16_round(rng.normal(size=(tokens, experts * ff)) * 2)
+    dense = np.where(rng.random((tokens, experts + 1)) < 0.5, 0.0, rng.random((tokens, experts + 1)))
+    from math import erf
+    f = {"relu2": lambda z: np.maximum(z, 0) ** 2, "gelu_erf": lambda z: 0.5 * z * (1 + np.vectorize(erf)(z / 2 ** 0.5)),
+         "gelu_tanh": lambda z: 0.5 * z * (1 + np.tanh((2 / np.pi) ** 0.5 * (z + 0.044715 * z ** 3)))}[activation]
+    tol = 1e-6 if dtype == torch.float32 else 5e-3
+    got = ops.experts_activate_plain(t(u, dtype), t(dense), ff, activation)
+    close(got, np.repeat(dense[:, :experts], ff, 1) * f(u), tol)
+    close(ops.experts_activate_plain(t(u[:, :ff], dtype), None, ff, activation), f(u[:, :ff]), tol)
