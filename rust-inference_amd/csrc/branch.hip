@@ -88,7 +88,7 @@ extern "C" int ri_embed_scaled(float* out, void* act, int act_dtype, const void*
 // sequence's first new token alone reads the token kept from the step before, and it alone puts the step's last token in
 // its place, after it has read.
 template <typename TW, bool VEC>
-__global__ void __launch_bounds__(256)
+__global__ void __launch_bounds__(1024)
 embed_bigram_kernel(float* __restrict__ out, const TW* __restrict__ table, const TW* __restrict__ pairs,
                     const int32_t* __restrict__ ids, const int32_t* __restrict__ tok_pos, const int32_t* __restrict__ tok_seq,
                     const int32_t* __restrict__ cu_seqlens, const int32_t* __restrict__ slots, int32_t* __restrict__ last,
@@ -105,12 +105,12 @@ embed_bigram_kernel(float* __restrict__ out, const TW* __restrict__ table, const
     const TW* p = pairs + (size_t)row * dim;
     float* o = out + (size_t)t * dim;
     if (VEC) {
-        for (int d = threadIdx.x * 4; d < dim; d += 1024) {
+        for (int d = threadIdx.x * 4; d < dim; d += blockDim.x * 4) {
             const float4 u = ld4(a + d), v = ld4(p + d);
             st4(o + d, make_float4(u.x + v.x, u.y + v.y, u.z + v.z, u.w + v.w));
         }
     } else {
-        for (int d = threadIdx.x; d < dim; d += 256) o[d] = to_f32(a[d]) + to_f32(p[d]);
+        for (int d = threadIdx.x; d < dim; d += blockDim.x) o[d] = to_f32(a[d]) + to_f32(p[d]);
     }
     if (!opens) return;
     __syncthreads();                                         // every thread has read the kept token
@@ -125,8 +125,10 @@ extern "C" int ri_embed_bigram(float* out, const void* table, const void* pairs,
                "embed_bigram: %ld buckets, factors %ld and %ld (reduced modulo the buckets)", buckets, mul_prev, mul_cur);
     RI_REQUIRE(table_dtype == RI_F32 || table_dtype == RI_BF16, "embed_bigram: table dtype %d", table_dtype);
     hipStream_t s = (hipStream_t)stream;
+    // a row of up to 4,096 elements in one pass of the workgroup: every load of both rows in flight at once
+    const int threads = dim % 4 != 0 || dim <= 1024 ? 256 : dim <= 2048 ? 512 : 1024;
 #define RI_GO(TW, VEC)                                                                                                  \
-    embed_bigram_kernel<TW, VEC><<<tokens, 256, 0, s>>>(out, (const TW*)table, (const TW*)pairs, ids, tok_pos, tok_seq,    \
+    embed_bigram_kernel<TW, VEC><<<tokens, threads, 0, s>>>(out, (const TW*)table, (const TW*)pairs, ids, tok_pos, tok_seq,    \
                                                        cu_seqlens, slots, last, buckets, mul_prev, mul_cur, dim)
     if (table_dtype == RI_F32) { if (dim % 4 == 0) RI_GO(float, true); else RI_GO(float, false); }
     else                       { if (dim % 4 == 0) RI_GO(bf16_t, true); else RI_GO(bf16_t, false); }

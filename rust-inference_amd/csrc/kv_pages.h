@@ -57,12 +57,12 @@ values_to_pages_kernel(const TA* __restrict__ qkv, size_t row_len, size_t v_off,
             float v[8];
             Eight<TA>::load(from + (size_t)(t_begin + first - start + tt) * row_len + d, v);
 #pragma unroll
-            for (int j = 0; j < 8; ++j) tile[tt * stride + d + j] = v[j] + (add ? add[d + j] : 0.f);
+            for (int j = 0; j < 8; ++j) tile[tt * stride + d + j] = v[j];
         }
     } else {
         for (int e = threadIdx.x; e < (hi - lo + 1) * vdim; e += blockDim.x) {
             const int tt = e / vdim, d = e - tt * vdim;
-            tile[(lo - first + tt) * stride + d] = to_f32(from[(size_t)(t_begin + lo - start + tt) * row_len + d]) + (add ? add[d] : 0.f);
+            tile[(lo - first + tt) * stride + d] = to_f32(from[(size_t)(t_begin + lo - start + tt) * row_len + d]);
         }
     }
     __syncthreads();
@@ -71,15 +71,16 @@ values_to_pages_kernel(const TA* __restrict__ qkv, size_t row_len, size_t v_off,
     if (whole && page_size % 8 == 0) {
         for (int e = threadIdx.x; e < vdim * (QT_TOKENS / 8); e += blockDim.x) {
             const int d = e / (QT_TOKENS / 8), t8 = (e - d * (QT_TOKENS / 8)) * 8;
+            const float b = add ? add[d] : 0.f;
             float v[8];
 #pragma unroll
-            for (int j = 0; j < 8; ++j) v[j] = tile[(t8 + j) * stride + d];
+            for (int j = 0; j < 8; ++j) v[j] = tile[(t8 + j) * stride + d] + b;
             Eight<TC>::store(base + (size_t)d * page_size + t8, v);
         }
     } else {
         for (int e = threadIdx.x; e < vdim * QT_TOKENS; e += blockDim.x) {
             const int d = e / QT_TOKENS, tt = e - d * QT_TOKENS;
-            if (first + tt >= lo && first + tt <= hi) from_f32(base + (size_t)d * page_size + tt, tile[tt * stride + d]);
+            if (first + tt >= lo && first + tt <= hi) from_f32(base + (size_t)d * page_size + tt, tile[tt * stride + d] + (add ? add[d] : 0.f));
         }
     }
 }

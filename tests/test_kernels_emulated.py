@@ -64,7 +64,7 @@ ZAKELORN_TESTS = os.path.join(HERE, "test_zakelorn_kernels_gpu.py")
 NOTADRA_TESTS = os.path.join(HERE, "test_notadra_kernels_gpu.py")
 DAGEZEN_TESTS = os.path.join(HERE, "test_dagezen_kernels_gpu.py")
 PISULORN_SELECT = "not two_equal_keys and not many_sequences"      # not the 1,300 keys and the 512 workgroups on the emulated matrix cores (minutes)
-NOTADRA_SELECT = ("not many_sequences and not thousands_of_keys and not (matrix_core and not (64-80 or 24-36 or 128-252 or 40-64))"
+NOTADRA_SELECT = ("not many_sequences and not thousands_of_keys and not (matrix_core and not (64-88 or 24-36 or 128-252 or 40-64))"
                   " and not 8192 and not 8200 and not 4100")          # a size of every capacity, not every size (minutes each)
 SAMPLER_SELECT = "(same_token_as_the_plain_sampler or top_p_drops) and not large"     # not the 151,936 entries, not the engine
 
@@ -90,7 +90,7 @@ def runs():
         "dagezen": _start([*PYTEST, *_workers(2), DAGEZEN_TESTS]),
         "notadra": _start([*PYTEST, *_workers(3), NOTADRA_TESTS, "-k", NOTADRA_SELECT]),
         # (eight compute units: the decode attention then walks whole runs of keys for a few sequences already)
-        "notadra, eight units": _start([*PYTEST, *_workers(2), NOTADRA_TESTS, "-k", "many_sequences and 64-80"], {"RI_EMU_COMPUTE_UNITS": "8"}),
+        "notadra, eight units": _start([*PYTEST, *_workers(2), NOTADRA_TESTS, "-k", "many_sequences and 64-88"], {"RI_EMU_COMPUTE_UNITS": "8"}),
         # (with one compute unit a prompt of 70 tokens already takes the form of the rotation kernel that gives a
         # wavefront four heads of a token)
         "zakelorn, one unit": _start([*PYTEST, ZAKELORN_TESTS, "-k", "rotation_unit_norm"], {"RI_EMU_COMPUTE_UNITS": "1"}),

@@ -255,7 +255,7 @@ def changed(folder, **tensors):
 
 
 @pytest.mark.parametrize("dtype_name", ["float32", "bfloat16"])
-@pytest.mark.parametrize("dim, vdim, place, seed", [(16, 24, 64, 7), (64, 80, 63, 3), (64, 64, 31, 3), (128, 144, 0, 3)])
+@pytest.mark.parametrize("dim, vdim, place, seed", [(16, 24, 64, 7), (64, 88, 63, 3), (64, 64, 31, 3), (128, 144, 0, 3)])
 def test_a_far_key_among_hundreds(tmp_path_factory, dim, vdim, place, seed, dtype_name):
     """A score scale at which one key can take the softmax: the last logits must see a token 700 positions back, at a page's
     first or last place or at the sequence's start.  No pairs beside the tokens (one bucket), so that the key alone tells."""
@@ -280,7 +280,7 @@ def test_a_far_key_among_hundreds(tmp_path_factory, dim, vdim, place, seed, dtyp
 
 
 @pytest.mark.parametrize("dtype_name", ["float32", "bfloat16"])
-@pytest.mark.parametrize("dim, vdim", [(16, 24), (64, 64), (64, 80)])
+@pytest.mark.parametrize("dim, vdim", [(16, 24), (64, 64), (64, 88)])
 def test_the_sink_of_score_zero_at_the_first_tokens(tmp_path_factory, dim, vdim, dtype_name):
     """Scores near zero: the first tokens lose half, a third, a quarter of their weight to the sink, which the norm behind the
     sublayer would hide if the values were all there is; the value's bias is taken out and the residual kept small, and the
@@ -425,12 +425,12 @@ def drawn_config(seed):
             mixer = {**layers[j]["mixer"], "kv_from": j, "scale": float(rng.uniform(0.05, 0.4)), "softcap": float(pick([3.0, 10.0, 40.0]))}
         else:
             kv, dim = pick([1, 2, 3, 4]), pick([8, 12, 16, 32, 40, 64, 72, 128])
-            stretch = pick([None, (float(pick([1.5, 2.0, 8.0])), pick([40, 128, 1024]), float(pick([4.0, 32.0])), float(pick([0.5, 1.0, 2.0])))])
+            stretch = pick([None, (float(pick([1.5, 2.0, 8.0])), pick([40, 128, 900]), float(pick([4.0, 32.0])), float(pick([0.5, 1.0, 2.0])))])
             mixer = attention(kv * pick([1, 2, 4]), kv, dim, pick([8, 20, 32, 64, 96, 128, 160]), float(rng.uniform(0.05, 0.4)),
                               cap=pick([None, 3.0, 10.0, 30.0]), rot_dims=2 * int(rng.integers(0, dim // 2 + 1)), base=float(pick([50.0, 10000.0, 500000.0])),
                               stretch=stretch)
         layers.append(layer(mixer, mlp))
-    buckets = pick([1, 17, 509, 4099])
+    buckets = pick([1, 17, 503, 4099])
     return model(layers, vocab=int(rng.integers(50, 400)), width=pick([48, 80, 136, 192]), eps=pick([1e-5, 1e-6, 1e-3]),
                  logit_scale=float(rng.uniform(0.3, 3.0)), bigram=(buckets, int(rng.integers(0, 2000)), int(rng.integers(0, 2000))))
 
