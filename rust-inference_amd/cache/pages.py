@@ -4,7 +4,7 @@ Pages are handed out lazily as a sequence grows, lowest number first, and go bac
 to the pool when the slot is released (the reference hands out page 0 first and
 can only reset the whole cache: src/kvcache.rs:51, :115-124, :192-196).  A pool with
 a window gives pages back as soon as every position in them lies behind the window
-of all later queries.  The bookkeeping is native (csrc/host_cache.hip); ``tables`` is
+of all later queries, one with chunks as soon as the sequence's next position lies in a later chunk.  The bookkeeping is native (csrc/host_cache.hip); ``tables`` is
 a view of its memory.
 """
 from __future__ import annotations
@@ -19,7 +19,8 @@ UNMAPPED = -1
 
 class PagePool:
     def __init__(self, num_pages: int, page_size: int, num_slots: int, max_pages_per_slot: int,
-                 window: int | None = None, keep_first: int | None = None):
+                 window: int | None = None, keep_first: int | None = None,
+                 chunk: int | None = None):
         if page_size < 1 or num_pages < 1 or max_pages_per_slot < 1 or num_slots < 1:
             raise CacheError("page pool sizes must be positive")
         self.num_pages, self.page_size = num_pages, page_size
@@ -31,6 +32,9 @@ class PagePool:
         self.keep_first = int(keep_first or 0)          # a sequence's first tokens, which a window never drops
         if self.keep_first:
             native.check(self._lib.ri_pool_keep_first(self.handle, self.keep_first))
+        self.chunk = int(chunk or 0)                    # a query sees its own run of this many positions alone
+        if self.chunk:
+            native.check(self._lib.ri_pool_chunk(self.handle, self.chunk))
         # slot -> its pages by logical number, -1 where none is mapped: the pool's own memory
         self.tables = np.ctypeslib.as_array(self._lib.ri_pool_tables(self.handle), shape=(num_slots, max_pages_per_slot))
 

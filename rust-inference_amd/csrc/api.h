@@ -104,6 +104,9 @@ int ri_gla_scan(float* out, const void* proj, int act_dtype, int row, int q_off,
 // from proj rows at column g_off; out of act_dtype [tokens, heads * vdim].
 int ri_gla_norm_gate(void* out, const float* o, const void* proj, int act_dtype, int row, int g_off, const float* gain,
                      float eps, int tokens, int heads, int vdim, void* stream);
+// The same with the gate in a format of its own (float32, or act_dtype) and, with `sigmoid`, sigmoid(gate) for silu(gate).
+int ri_head_norm_gate(void* out, int act_dtype, const float* o, const void* gate, int gate_dtype, int row, int g_off,
+                      const float* gain, float eps, int tokens, int heads, int vdim, int sigmoid, void* stream);
 
 // One new token a sequence (token b is sequence b's): the recurrence's step, the per-head RMS norm and the gate in
 // one kernel; out of act_dtype [seqs, heads * vdim].  ri_gla_step_fits: whether it takes these head sizes.
@@ -156,6 +159,22 @@ int ri_delta_step(void* out, const void* proj, int act_dtype, int row, int q_off
                   float* tails, const float* ab, const float* a_log, const float* dt_bias, float* state,
                   const int32_t* cu_seqlens, const int32_t* slots, const float* gain, float eps, int seqs, int heads,
                   int kv_heads, int dim, int vdim, void* stream);
+
+// The same with a decay per head and key channel: z [tokens or seqs, z_row] float32 holds heads * dim pre-activations from
+// column 0 on, g = exp(-exp(a_log_h) * softplus(z + dt_bias)) with dt_bias [heads * dim]; b, rows of b_row elements of act_dtype,
+// the logits of beta; gates [tokens, heads * dim + heads] (decays, then betas).  The step's output gate is the sigmoid of the
+// heads * vdim elements of z's rows from column gate_at on.
+int ri_delta_prepare_channels(float* qkv, float* gates, const void* proj, int act_dtype, int row, int q_off, const float* taps,
+                              int ntaps, float* tails, const float* z, int z_row, const void* b, int b_row, const float* a_log,
+                              const float* dt_bias, const int32_t* tok_seq, const int32_t* cu_seqlens, const int32_t* slots,
+                              int seqs, int tokens, int heads, int kv_heads, int dim, int vdim, void* stream);
+int ri_delta_scan_channels(float* out, const float* qkv, const float* gates, float* state, const int32_t* cu_seqlens,
+                           const int32_t* slots, int seqs, int tokens, int heads, int kv_heads, int dim, int vdim, int slices,
+                           void* stream);
+int ri_delta_step_channels(void* out, const void* proj, int act_dtype, int row, int q_off, const float* taps, int ntaps,
+                           float* tails, const float* z, int z_row, int gate_at, const void* b, int b_row, const float* a_log,
+                           const float* dt_bias, float* state, const int32_t* cu_seqlens, const int32_t* slots, const float* gain,
+                           float eps, int seqs, int heads, int kv_heads, int dim, int vdim, void* stream);
 
 // A mixture of experts' router.  z: float32 [tokens, experts] router logits; s = sigmoid(z); the `top` experts with
 // the largest s + correction (the lower index on a tie) are chosen; their weights are their s divided by the sum of
@@ -230,7 +249,7 @@ int ri_attention_decode_bf16(void* out, float* workspace, const void* qkv, int q
 int ri_attention_decode_kept_bf16(void* out, float* workspace, const void* qkv, int q_stride, const void* k_pages,
                                   const void* v_pages, const int32_t* cu_seqlens, const int32_t* tok_pos,
                                   const int32_t* page_table, int table_width, int seqs, int max_chunks, int heads,
-                                  int kv_heads, int head_dim, int page_size, int window, float scale, float softcap,
+                                  int kv_heads, int head_dim, int page_size, int window, int chunk, float scale, float softcap,
                                   const float* slopes, int tiled_out, int keep_first, const float* sinks, void* stream);
 
 // tiled_out (both decode forms): the result [seqs, heads * head_dim] is written in the matrix cores' operand order
@@ -365,6 +384,8 @@ int ri_pool_reserve(void* pool, int slot, long length_before, long new_tokens);
 int ri_pool_trim(void* pool, int slot, long length);
 // The first `tokens` positions of every sequence stay mapped however far a window has moved on.
 int ri_pool_keep_first(void* pool, int tokens);
+// A query sees the keys of its own run of `tokens` positions alone (runs counted from position 0): pages of earlier runs go back.
+int ri_pool_chunk(void* pool, int tokens);
 int ri_pool_release(void* pool, int slot);
 int ri_pool_check(void* pool);
 // Slots, every slot's length, and the pools (not owned) that the slots hold pages in.
@@ -488,17 +509,29 @@ int ri_attention_padded_fits(int dim, int vdim, int group, int decode);
 int ri_attention_prefill_padded_bf16(void* out, const void* qkv, int q_stride, const void* k_pages, const void* v_pages,
                                      const int32_t* cu_seqlens, const int32_t* tok_pos, const int32_t* page_table,
                                      int table_width, int seqs, int max_new, int heads, int kv_heads, int dim, int vdim,
-                                     int page_size, int window, float scale, float softcap, const float* slopes,
+                                     int page_size, int window, int chunk, float scale, float softcap, const float* slopes,
                                      int keep_first, const float* sinks, void* stream);
 int ri_attention_decode_padded_bf16(void* out, float* workspace, const void* qkv, int q_stride, const void* k_pages,
                                     const void* v_pages, const int32_t* tok_pos, const int32_t* page_table, int table_width,
                                     int seqs, int max_chunks, int heads, int kv_heads, int dim, int vdim, int page_size,
-                                    int window, float scale, float softcap, const float* slopes, int tiled_out,
+                                    int window, int chunk, float scale, float softcap, const float* slopes, int tiled_out,
                                     int keep_first, const float* sinks, void* stream);
+
+// out (+)= a_scale * norm(a) * a_gain + b_scale * norm(b) * b_gain, row by row: RMS norms over `dim` of products' results a and b
+// ([parts, rows, dim] float32, added in order, or one part of either format; b may be NULL); out float32 [rows, dim].
+int ri_normed_sum(float* out, int accumulate, const void* a, int a_dtype, int a_parts, const float* a_gain, float a_scale,
+                  const void* b, int b_dtype, int b_parts, const float* b_gain, float b_scale, float eps, int rows, int dim,
+                  void* stream);
+
+// Experts by token: table int32 [vocab, top] (entries of a row differ, all below `experts`); ids [tokens, top], weights
+// [tokens, top] (all 1 / top) and, where not NULL, dense [tokens, experts] of the tokens' rows.
+int ri_experts_by_table(int32_t* ids, float* weights, float* dense, const int32_t* table, const int32_t* token_ids, int tokens,
+                        int vocab, int experts, int top, void* stream);
 
 // Biases, rotation in halves and the cache write (qk_half_bias_kv.hip).
 int ri_qk_half_bias_kv_write(void* proj, int act_dtype, long row_len, int q_off, int k_off, int v_off, const float* q_bias,
-                             const float* k_bias, const float* v_bias, const float* inv_freq, int half, float amplitude,
+                             const float* k_bias, const float* v_bias, const float* q_gain, const float* k_gain, float eps,
+                             const float* inv_freq, int half, float amplitude,
                              const int32_t* tok_pos, const int32_t* tok_seq, const int32_t* cu_seqlens, int seqs, int max_new,
                              const int32_t* page_table, int table_width, void* k_pages, void* v_pages, int cache_dtype,
                              int tokens, int heads, int kv_heads, int dim, int vdim, int page_size, void* stream);

@@ -5,7 +5,7 @@
 //
 // score_j = (q . k_j) * scale, then, with a cap c > 0, score_j <- c tanh(score_j / c), then, with a slope per
 // query head, score_j <- score_j - slope_h (p - j); the query at position p
-// sees keys lo..p with lo = 0 or p - window + 1, and with keep_first > 0 also the keys 0..keep_first-1 that lie
+// sees keys lo..p with lo = 0, p - window + 1 or the start of the chunk of positions that p lies in, and with keep_first > 0 also the keys 0..keep_first-1 that lie
 // before lo (the first tokens of a sequence stay visible behind the window); with a sink per query head the
 // softmax's denominator also holds exp(sink_h), which has no key and no value;
 // online softmax with running maximum m, running sum l and factor exp(m_old - m_new)
@@ -50,7 +50,7 @@ __global__ void __launch_bounds__(ATT_TILE)
 attention_generic_kernel(TA* __restrict__ out, const TA* __restrict__ q, int q_stride, const TC* __restrict__ k_pages,
                          const TC* __restrict__ v_pages, const int32_t* __restrict__ tok_pos,
                          const int32_t* __restrict__ tok_seq, const int32_t* __restrict__ page_table, int table_width,
-                         int heads, int kv_heads, int head_dim, int v_dim, int page_size, int window, float scale,
+                         int heads, int kv_heads, int head_dim, int v_dim, int page_size, Reach reach, float scale,
                          float softcap, const float* __restrict__ slopes, int keep_first,
                          const float* __restrict__ sinks) {
     extern __shared__ float qs[];                 // head_dim floats: the query
@@ -61,7 +61,7 @@ attention_generic_kernel(TA* __restrict__ out, const TA* __restrict__ q, int q_s
     const int t = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
     const int kvh = h / (heads / kv_heads);       // consecutive query heads share a kv head
     const int qpos = tok_pos[t];
-    const int lo = window > 0 ? max(0, qpos - window + 1) : 0;
+    const int lo = reach.first(qpos);
     const float slope = slopes ? slopes[h] : 0.f;
     const int32_t* table = page_table + (size_t)tok_seq[t] * table_width;
 
@@ -166,18 +166,20 @@ template <typename T, bool VEC>
 static void launch_attention(void* out, const void* q, int q_stride, const void* k_pages, const void* v_pages,
                              const int32_t* tok_pos, const int32_t* tok_seq, const int32_t* page_table,
                              int table_width, int tokens, int heads, int kv_heads, int head_dim, int v_dim,
-                             int page_size, int window, float scale, float softcap, const float* slopes, int keep_first,
+                             int page_size, Reach reach, float scale, float softcap, const float* slopes, int keep_first,
                              const float* sinks, hipStream_t s) {
     attention_generic_kernel<T, T, VEC><<<dim3(tokens, heads), ATT_TILE, (size_t)head_dim * sizeof(float), s>>>(
         (T*)out, (const T*)q, q_stride, (const T*)k_pages, (const T*)v_pages, tok_pos, tok_seq, page_table,
-        table_width, heads, kv_heads, head_dim, v_dim, page_size, window, scale, softcap, slopes, keep_first, sinks);
+        table_width, heads, kv_heads, head_dim, v_dim, page_size, reach, scale, softcap, slopes, keep_first, sinks);
 }
 
 extern "C" int ri_attention_kept(void* out, const void* q, int act_dtype, int q_stride, const void* k_pages,
                             const void* v_pages, int cache_dtype, const int32_t* tok_pos, const int32_t* tok_seq,
                             const int32_t* page_table, int table_width, int tokens, int heads, int kv_heads,
-                            int head_dim, int v_dim, int page_size, int window, float scale, float softcap,
+                            int head_dim, int v_dim, int page_size, int window, int chunk, float scale, float softcap,
                             const float* slopes, int keep_first, const float* sinks, void* stream) {
+    RI_REQUIRE(chunk >= 0 && (chunk == 0 || window <= 0), "attention: chunks of %d beside a window of %d", chunk, window);
+    const Reach reach = {window, chunk};
     RI_REQUIRE(keep_first >= 0, "attention: %d first tokens kept", keep_first);
     RI_REQUIRE(tokens > 0 && heads > 0 && kv_heads > 0 && heads % kv_heads == 0,
                "attention: tokens %d, heads %d, kv heads %d", tokens, heads, kv_heads);
@@ -195,7 +197,7 @@ extern "C" int ri_attention_kept(void* out, const void* q, int act_dtype, int q_
     // the pools themselves are 256-byte aligned allocations
     const bool vec = head_dim % (act_dtype == RI_F32 ? 4 : 8) == 0 && (uintptr_t)k_pages % 16 == 0 && (uintptr_t)v_pages % 16 == 0;
 #define RI_ATT_GO(T, V) launch_attention<T, V>(out, q, q_stride, k_pages, v_pages, tok_pos, tok_seq, page_table, \
-                                               table_width, tokens, heads, kv_heads, head_dim, v_dim, page_size, window, scale, \
+                                               table_width, tokens, heads, kv_heads, head_dim, v_dim, page_size, reach, scale, \
                                                softcap, slopes, window > 0 ? keep_first : 0, sinks, s)
     if (act_dtype == RI_F32) { if (vec) RI_ATT_GO(float, true); else RI_ATT_GO(float, false); }
     else                     { if (vec) RI_ATT_GO(bf16_t, true); else RI_ATT_GO(bf16_t, false); }
@@ -210,6 +212,6 @@ extern "C" int ri_attention(void* out, const void* q, int act_dtype, int q_strid
                             int head_dim, int v_dim, int page_size, int window, float scale, float softcap,
                             const float* slopes, void* stream) {
     return ri_attention_kept(out, q, act_dtype, q_stride, k_pages, v_pages, cache_dtype, tok_pos, tok_seq, page_table,
-                             table_width, tokens, heads, kv_heads, head_dim, v_dim, page_size, window, scale, softcap,
+                             table_width, tokens, heads, kv_heads, head_dim, v_dim, page_size, window, 0, scale, softcap,
                              slopes, 0, nullptr, stream);
 }

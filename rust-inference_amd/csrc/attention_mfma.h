@@ -14,7 +14,7 @@
 // after them lane group j (lanes 16 j .. 16 j + 15) holds the scores of keys 8 j .. 8 j + 7 of its
 // column: exactly the B operand of the second product, with no exchange between lanes.
 //
-// The mask is positional: the query at position p sees keys lo..p, lo = 0 or p - window + 1
+// The mask is positional: the query at position p sees keys lo..p, lo = 0, p - window + 1 or the start of p's chunk (Reach)
 // (the reference: src/attention.rs:73, :117-118).  Scores are scaled after the dot product
 // (src/attention.rs:28, :121-127); statistics and accumulators are float32; the weights enter the
 // second product rounded to bfloat16, the running sum is taken of them before the rounding.  (Letting
@@ -402,7 +402,7 @@ attn_prefill_mfma_kernel(bf16_t* __restrict__ out, const bf16_t* __restrict__ qk
                          const bf16_t* __restrict__ k_pages, const bf16_t* __restrict__ v_pages,
                          const int32_t* __restrict__ cu_seqlens, const int32_t* __restrict__ tok_pos,
                          const int32_t* __restrict__ page_table, int table_width, int heads, int kv_heads,
-                         int window, float scale_log2, float cap_pre, float cap_post,
+                         Reach reach, float scale_log2, float cap_pre, float cap_post,
                          const float* __restrict__ slopes, float inv_scale, int keep_first,
                          const float* __restrict__ sinks, int dim_ = DH, int vdim_ = DV) {
     // PAD: heads of dim and vdim elements (multiples of 8 and 4), up to DH and DV; what lies behind dim is zero in the
@@ -429,7 +429,7 @@ attn_prefill_mfma_kernel(bf16_t* __restrict__ out, const bf16_t* __restrict__ qk
     c.cap_pre = cap_pre;
     c.cap_post = cap_post;
     c.biased = slopes != nullptr;
-    c.keep = window > 0 ? keep_first : 0;
+    c.keep = reach.window > 0 ? keep_first : 0;
     const int jg = lane >> 4;
     float sink[NT];                                          // the column's sink in the exponents' units; -inf: none
 #pragma unroll
@@ -441,7 +441,7 @@ attn_prefill_mfma_kernel(bf16_t* __restrict__ out, const bf16_t* __restrict__ qk
         if (tl < nt) {
             const int tok = t0 + tl;
             c.qpos[j] = tok_pos[tok];
-            c.lo[j] = window > 0 ? max(0, c.qpos[j] - window + 1) : 0;
+            c.lo[j] = reach.first(c.qpos[j]);
             const bf16_t* qp = qkv + (long)tok * q_stride + (kvh * group + g) * dim + jg * 8;
 #pragma unroll
             for (int ks = 0; ks < DH / 32; ++ks)
@@ -450,13 +450,13 @@ attn_prefill_mfma_kernel(bf16_t* __restrict__ out, const bf16_t* __restrict__ qk
     }
     // pages the workgroup walks (every wavefront takes them all)
     const int wg_first = tok_pos[t_wg], wg_last = tok_pos[min(t_end, t_wg + 4 * tile_tokens) - 1];
-    const int p_lo = window > 0 ? max(0, wg_first - window + 1) / PAGE : 0;
+    const int p_lo = reach.first(wg_first) / PAGE;
     const int p_hi = wg_last / PAGE;
     // a page is open to the whole wavefront when its last key is at or before the first token's position
     // and its first key inside the last token's window; wavefronts with unused columns mask always
     const bool full = nt * group == 16 * NT;
     const int min_qpos = (nt > 0 && full) ? tok_pos[t0] : -1;
-    const int max_lo = (nt > 0 && window > 0) ? max(0, tok_pos[t0 + nt - 1] - window + 1) : 0;
+    const int max_lo = nt > 0 ? reach.first(tok_pos[t0 + nt - 1]) : 0;
     const int32_t* table = page_table + (long)b * table_width;
     // The walk: the pages that hold kept first tokens and lie before the window's first page, then the window's
     // pages.  Walk position W stands for the page RI_PG(W); a kept page is never taken for open (its keys from
@@ -606,7 +606,7 @@ __global__ void __launch_bounds__(CW * 64)
 attn_decode_mfma_kernel(float* __restrict__ ws, const bf16_t* __restrict__ qkv, int q_stride,
                         const bf16_t* __restrict__ k_pages, const bf16_t* __restrict__ v_pages,
                         const int32_t* __restrict__ tok_pos, const int32_t* __restrict__ page_table, int table_width,
-                        int heads, int kv_heads, int window, float scale_log2, int max_chunks, float cap_pre, float cap_post,
+                        int heads, int kv_heads, Reach reach, float scale_log2, int max_chunks, float cap_pre, float cap_post,
                         const float* __restrict__ slopes, float inv_scale, int keep_first, int dim_ = DH, int vdim_ = DV) {
     const int dim = PAD ? dim_ : DH, vdim = PAD ? vdim_ : DV;
     __shared__ float o_lds[CW][DV * 17];           // [d * 17 + col]: no bank conflicts either way
@@ -621,8 +621,8 @@ attn_decode_mfma_kernel(float* __restrict__ ws, const bf16_t* __restrict__ qkv, 
     const int page = chunk * CW + wave;   // this wavefront's page
     const int qpos = tok_pos[tok];
     const int phys = max(page_table[(long)b * table_width + min(page, table_width - 1)], 0);   // not mapped: page 0, unused
-    const int lo = window > 0 ? max(0, qpos - window + 1) : 0;
-    const int keep = window > 0 ? keep_first : 0;             // keys before it stay visible behind the window
+    const int lo = reach.first(qpos);
+    const int keep = reach.window > 0 ? keep_first : 0;             // keys before it stay visible behind the window
     if (chunk * (CW * PAGE) > qpos || (chunk * (CW * PAGE) + CW * PAGE - 1 < lo && chunk * (CW * PAGE) >= keep))
         return;                                              // whole workgroup
 
@@ -740,7 +740,7 @@ __device__ __forceinline__ void join_sum(const float* __restrict__ base, int cb,
 template <int DH, int PB, bool PAD = false>
 __global__ void __launch_bounds__(DH * PB)
 attn_decode_join_kernel(bf16_t* __restrict__ out, const float* __restrict__ ws, const int32_t* __restrict__ tok_pos,
-                        int heads, int window, int max_chunks, int chunk_keys, int tiled, int keep_first,
+                        int heads, Reach reach, int max_chunks, int chunk_keys, int tiled, int keep_first,
                         const float* __restrict__ sinks, int vdim_ = DH) {
     const int vdim = PAD ? vdim_ : DH;
     __shared__ float part_o[JOIN_PARTS][DH];
@@ -749,15 +749,15 @@ attn_decode_join_kernel(bf16_t* __restrict__ out, const float* __restrict__ ws, 
     const int tp = threadIdx.x / DH, d = PAD ? min((int)threadIdx.x % DH, vdim - 1) : threadIdx.x % DH;
     const bool mine = !PAD || (int)threadIdx.x % DH < vdim;
     const int qpos = tok_pos[b];
-    const int lo = window > 0 ? max(0, qpos - window + 1) : 0;
-    // window < 0: the entries are the runs of the streaming kernel, all of them written
-    const int c_lo = window < 0 ? 0 : lo / chunk_keys, c_hi = window < 0 ? max_chunks - 1 : qpos / chunk_keys;
+    const int lo = reach.first(qpos);
+    // reach.window < 0: the entries are the runs of the streaming kernel, all of them written
+    const int c_lo = reach.window < 0 ? 0 : lo / chunk_keys, c_hi = reach.window < 0 ? max_chunks - 1 : qpos / chunk_keys;
     const int n = c_hi - c_lo + 1;
     const int parts = n <= JOIN_SERIAL ? 1 : JOIN_PARTS;
     const int per = (n + parts - 1) / parts;
     const float* base = ws + ((long)b * heads + h) * max_chunks * (vdim + 2);
     // the chunks of the kept first keys that lie before the window's first chunk: the first run takes them first
-    const int k_hi = window > 0 && keep_first > 0 ? min((keep_first - 1) / chunk_keys, c_lo - 1) : -1;
+    const int k_hi = reach.window > 0 && keep_first > 0 ? min((keep_first - 1) / chunk_keys, c_lo - 1) : -1;
     // a sink joins the denominator alone, exp(sink - maximum) in the exponents' units
     const float sink = sinks ? sinks[h] * 1.4426950408889634f : -INFINITY;
     for (int p = tp; p < parts; p += PB) {
@@ -814,7 +814,7 @@ attn_decode_join_kernel(bf16_t* __restrict__ out, const float* __restrict__ ws, 
 template <int DH, int CAP, bool PAD = false>
 __global__ void __launch_bounds__(DH)
 attn_decode_join_small_kernel(bf16_t* __restrict__ out, const float* __restrict__ ws, const int32_t* __restrict__ tok_pos,
-                              int heads, int window, int max_chunks, int chunk_keys, int tiled, int keep_first,
+                              int heads, Reach reach, int max_chunks, int chunk_keys, int tiled, int keep_first,
                               const float* __restrict__ sinks, int vdim_ = DH) {
     const int vdim = PAD ? vdim_ : DH;
     const int b = blockIdx.x, h = blockIdx.y, d = PAD ? min((int)threadIdx.x, vdim - 1) : threadIdx.x;
@@ -832,12 +832,12 @@ attn_decode_join_small_kernel(bf16_t* __restrict__ out, const float* __restrict_
         }
     }
     const int qpos = tok_pos[b];
-    const int lo = window > 0 ? max(0, qpos - window + 1) : 0;
-    // window < 0: the entries are not chunks at fixed places but the runs of the streaming kernel, all of
+    const int lo = reach.first(qpos);
+    // reach.window < 0: the entries are not chunks at fixed places but the runs of the streaming kernel, all of
     // them written (an empty run as a maximum of -inf)
-    const int c_lo = window < 0 ? 0 : lo / chunk_keys, c_hi = window < 0 ? max_chunks - 1 : qpos / chunk_keys;
+    const int c_lo = reach.window < 0 ? 0 : lo / chunk_keys, c_hi = reach.window < 0 ? max_chunks - 1 : qpos / chunk_keys;
     // the chunks of the kept first keys count as well (those before the window's first chunk were written for them)
-    const int k_hi = window > 0 && keep_first > 0 ? min((keep_first - 1) / chunk_keys, c_hi) : -1;
+    const int k_hi = reach.window > 0 && keep_first > 0 ? min((keep_first - 1) / chunk_keys, c_hi) : -1;
     const float sink = sinks ? sinks[h] * 1.4426950408889634f : -INFINITY;
     float m = -INFINITY;
 #pragma unroll
@@ -859,17 +859,17 @@ attn_decode_join_small_kernel(bf16_t* __restrict__ out, const float* __restrict_
 }
 
 template <int DH, bool PAD = false>
-static void launch_join(bf16_t* out, const float* ws, const int32_t* tok_pos, int seqs, int heads, int window,
+static void launch_join(bf16_t* out, const float* ws, const int32_t* tok_pos, int seqs, int heads, Reach reach,
                         int max_chunks, int tiled, hipStream_t s, int chunk_keys = DECODE_CHUNK, int keep_first = 0,
                         const float* sinks = nullptr, int vdim = DH) {
     constexpr int PB = DH * JOIN_PARTS <= 1024 ? JOIN_PARTS : JOIN_PARTS / 2;
     if (max_chunks <= JOIN_SERIAL)
-        attn_decode_join_small_kernel<DH, JOIN_SERIAL, PAD><<<dim3(seqs, heads), DH, 0, s>>>(out, ws, tok_pos, heads, window,
+        attn_decode_join_small_kernel<DH, JOIN_SERIAL, PAD><<<dim3(seqs, heads), DH, 0, s>>>(out, ws, tok_pos, heads, reach,
                                                                                      max_chunks, chunk_keys, tiled,
                                                                                      keep_first, sinks, vdim);
     else
         attn_decode_join_kernel<DH, PB, PAD><<<dim3(seqs, heads), DH * PB, 0, s>>>(out, ws, tok_pos, heads,
-                                                                                           window, max_chunks, chunk_keys, tiled,
+                                                                                           reach, max_chunks, chunk_keys, tiled,
                                                                                            keep_first, sinks, vdim);
 }
 
@@ -950,7 +950,7 @@ attn_decode_stream_kernel(bf16_t* __restrict__ out, float* __restrict__ ws, cons
                           const float* __restrict__ q_gain, const float* __restrict__ k_gain, float eps,
                           const float* __restrict__ inv_freq, bf16_t* k_pages, bf16_t* v_pages,
                           const int32_t* __restrict__ tok_pos, const int32_t* __restrict__ page_table, int table_width,
-                          int heads, int kv_heads, int window, float scale_log2, int splits, int tiled, float cap_pre, float cap_post,
+                          int heads, int kv_heads, Reach reach, float scale_log2, int splits, int tiled, float cap_pre, float cap_post,
                           const float* __restrict__ slopes, float inv_scale, const float* __restrict__ sinks, int dim_ = DH,
                           int vdim_ = DV) {
     static_assert(!FUSED || (DH <= 128 && DV == DH && !PAD), "one (d, d + DH/2) pair per lane");
@@ -964,7 +964,7 @@ attn_decode_stream_kernel(bf16_t* __restrict__ out, float* __restrict__ ws, cons
     const int b = blockIdx.x, kvh = blockIdx.y, split = blockIdx.z;
     const int group = heads / kv_heads;
     const int qpos = tok_pos[b];                             // token b is sequence b's one new token
-    const int lo = window > 0 ? max(0, qpos - window + 1) : 0;
+    const int lo = reach.first(qpos);
     const int c_lo = lo / DECODE_CHUNK, c_hi = qpos / DECODE_CHUNK;
     const int per = (c_hi - c_lo + splits) / splits;         // chunks per run: by the sequence's own length
     const int c0 = c_lo + split * per, c1 = min(c_hi, c0 + per - 1);
@@ -1172,7 +1172,7 @@ attn_decode_fused_kernel(float* __restrict__ ws, const bf16_t* __restrict__ qkv,
                          const float* __restrict__ k_gain, float eps, const float* __restrict__ inv_freq,
                          bf16_t* __restrict__ k_pages, bf16_t* __restrict__ v_pages,
                          const int32_t* __restrict__ tok_pos, const int32_t* __restrict__ page_table, int table_width,
-                         int heads, int kv_heads, int window, float scale_log2, int max_chunks) {
+                         int heads, int kv_heads, Reach reach, float scale_log2, int max_chunks) {
     static_assert(DH <= 128, "one (d, d + DH/2) pair per lane");
     __shared__ float o_lds[CW][DH * 17];
     __shared__ float ml_lds[CW][2][16];
@@ -1196,7 +1196,7 @@ attn_decode_fused_kernel(float* __restrict__ ws, const bf16_t* __restrict__ qkv,
     const int page = chunk * CW + wave;
     const int qpos = tok_pos[b];                             // token b is sequence b's one new token
     const int phys = max(page_table[(long)b * table_width + min(page, table_width - 1)], 0);
-    const int lo = window > 0 ? max(0, qpos - window + 1) : 0;
+    const int lo = reach.first(qpos);
     if (chunk * (CW * PAGE) > qpos || chunk * (CW * PAGE) + CW * PAGE - 1 < lo) return;   // whole workgroup
     const bool owner = chunk == qpos / (CW * PAGE);         // this chunk holds the new token's position
 

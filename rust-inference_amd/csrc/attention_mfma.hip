@@ -43,9 +43,11 @@ static int prefill_tiles(int head_dim, int group, int max_new, int seqs, int kv_
 extern "C" int ri_attention_prefill_kept_bf16(void* out, const void* qkv, int q_stride, const void* k_pages,
                                               const void* v_pages, const int32_t* cu_seqlens, const int32_t* tok_pos,
                                               const int32_t* page_table, int table_width, int seqs, int max_new,
-                                              int heads, int kv_heads, int head_dim, int page_size, int window,
+                                              int heads, int kv_heads, int head_dim, int page_size, int window, int chunk,
                                               float scale, float softcap, const float* slopes, int keep_first,
                                               const float* sinks, void* stream) {
+    RI_REQUIRE(chunk >= 0 && (chunk == 0 || window <= 0), "attention_prefill: chunks of %d beside a window of %d", chunk, window);
+    const Reach reach = {window, chunk};
     RI_REQUIRE(keep_first >= 0, "attention_prefill_bf16: %d first tokens kept", keep_first);
     const float cap_pre = softcap > 0.f ? scale / softcap : 0.f, cap_post = softcap > 0.f ? softcap / scale : 0.f;
     RI_REQUIRE(scale > 0.f, "attention_prefill_bf16: the scale %g must be positive", (double)scale);
@@ -65,7 +67,7 @@ extern "C" int ri_attention_prefill_kept_bf16(void* out, const void* qkv, int q_
     case DH * 8 + NT:                                                                                            \
         attn_prefill_mfma_kernel<DH, NT><<<grid, 256, 0, s>>>(                                                   \
             (bf16_t*)out, (const bf16_t*)qkv, q_stride, (const bf16_t*)k_pages, (const bf16_t*)v_pages,          \
-            cu_seqlens, tok_pos, page_table, table_width, heads, kv_heads, window, scale_log2, cap_pre,          \
+            cu_seqlens, tok_pos, page_table, table_width, heads, kv_heads, reach, scale_log2, cap_pre,          \
             cap_post, slopes, 1.f / scale, keep_first, sinks);                                                   \
         break;
     switch (head_dim * 8 + nt_tiles) {
@@ -89,7 +91,7 @@ extern "C" int ri_attention_prefill_bf16(void* out, const void* qkv, int q_strid
                                          int heads, int kv_heads, int head_dim, int page_size, int window,
                                          float scale, float softcap, const float* slopes, void* stream) {
     return ri_attention_prefill_kept_bf16(out, qkv, q_stride, k_pages, v_pages, cu_seqlens, tok_pos, page_table, table_width,
-                                          seqs, max_new, heads, kv_heads, head_dim, page_size, window, scale, softcap, slopes,
+                                          seqs, max_new, heads, kv_heads, head_dim, page_size, window, 0, scale, softcap, slopes,
                                           0, nullptr, stream);
 }
 
@@ -107,8 +109,10 @@ extern "C" int ri_attention_decode_kept_bf16(void* out, float* workspace, const 
                                              const void* k_pages, const void* v_pages, const int32_t* cu_seqlens,
                                              const int32_t* tok_pos, const int32_t* page_table, int table_width, int seqs,
                                              int max_chunks, int heads, int kv_heads, int head_dim, int page_size,
-                                             int window, float scale, float softcap, const float* slopes, int tiled_out,
+                                             int window, int chunk, float scale, float softcap, const float* slopes, int tiled_out,
                                              int keep_first, const float* sinks, void* stream) {
+    RI_REQUIRE(chunk >= 0 && (chunk == 0 || window <= 0), "attention_decode: chunks of %d beside a window of %d", chunk, window);
+    const Reach reach = {window, chunk};
     RI_REQUIRE(keep_first >= 0, "attention_decode_bf16: %d first tokens kept", keep_first);
     RI_REQUIRE(keep_first == 0 || stream_splits(seqs, kv_heads, max_chunks) == 0,
                "attention_decode_bf16: kept first tokens in a step that streams (%d sequences)", seqs);
@@ -132,15 +136,15 @@ extern "C" int ri_attention_decode_kept_bf16(void* out, float* workspace, const 
         if (wide)                                                                                                 \
             attn_decode_stream_kernel<DH, false, 8><<<sgrid, 8 * 64, 0, s>>>(                                     \
                 (bf16_t*)out, workspace, (const bf16_t*)qkv, q_stride, nullptr, nullptr, 0.f, nullptr,            \
-                (bf16_t*)k_pages, (bf16_t*)v_pages, tok_pos, page_table, table_width, heads, kv_heads, window,    \
+                (bf16_t*)k_pages, (bf16_t*)v_pages, tok_pos, page_table, table_width, heads, kv_heads, reach,     \
                 scale_log2, splits, tiled_out, cap_pre, cap_post, slopes, 1.f / scale, sinks);                           \
         else                                                                                                      \
             attn_decode_stream_kernel<DH, false, 4><<<sgrid, 4 * 64, 0, s>>>(                                     \
                 (bf16_t*)out, workspace, (const bf16_t*)qkv, q_stride, nullptr, nullptr, 0.f, nullptr,            \
-                (bf16_t*)k_pages, (bf16_t*)v_pages, tok_pos, page_table, table_width, heads, kv_heads, window,    \
+                (bf16_t*)k_pages, (bf16_t*)v_pages, tok_pos, page_table, table_width, heads, kv_heads, reach,     \
                 scale_log2, splits, tiled_out, cap_pre, cap_post, slopes, 1.f / scale, sinks);                           \
         if (splits > 1)                                                                                          \
-            launch_join<DH>((bf16_t*)out, workspace, tok_pos, seqs, heads, -1, splits, tiled_out, s, DECODE_CHUNK, 0, sinks); \
+            launch_join<DH>((bf16_t*)out, workspace, tok_pos, seqs, heads, Reach{-1, 0}, splits, tiled_out, s, DECODE_CHUNK, 0, sinks); \
         break;
         switch (head_dim) {
             RI_STREAM_CASE(32)
@@ -157,9 +161,9 @@ extern "C" int ri_attention_decode_kept_bf16(void* out, float* workspace, const 
     case DH * 16 + CW:                                                                                            \
         attn_decode_mfma_kernel<DH, CW><<<pgrid, CW * 64, 0, s>>>(                                                \
             workspace, (const bf16_t*)qkv, q_stride, (const bf16_t*)k_pages, (const bf16_t*)v_pages,             \
-            tok_pos, page_table, table_width, heads, kv_heads, window, scale_log2, all, cap_pre, cap_post,       \
+            tok_pos, page_table, table_width, heads, kv_heads, reach, scale_log2, all, cap_pre, cap_post,       \
             slopes, 1.f / scale, keep_first);                                                                     \
-        launch_join<DH>((bf16_t*)out, workspace, tok_pos, seqs, heads, window, all, tiled_out, s, CW * PAGE,      \
+        launch_join<DH>((bf16_t*)out, workspace, tok_pos, seqs, heads, reach, all, tiled_out, s, CW * PAGE,      \
                         keep_first, sinks);                                                                       \
         break;
     switch (head_dim * 16 + DECODE_WAVES / pieces) {
@@ -185,7 +189,7 @@ extern "C" int ri_attention_decode_bf16(void* out, float* workspace, const void*
                                         int window, float scale, float softcap, const float* slopes, int tiled_out,
                                         void* stream) {
     return ri_attention_decode_kept_bf16(out, workspace, qkv, q_stride, k_pages, v_pages, cu_seqlens, tok_pos, page_table,
-                                         table_width, seqs, max_chunks, heads, kv_heads, head_dim, page_size, window, scale,
+                                         table_width, seqs, max_chunks, heads, kv_heads, head_dim, page_size, window, 0, scale,
                                          softcap, slopes, tiled_out, 0, nullptr, stream);
 }
 
@@ -197,6 +201,7 @@ extern "C" int ri_attention_decode_fused_bf16(void* out, float* workspace, const
                                               const int32_t* tok_pos, const int32_t* page_table, int table_width,
                                               int seqs, int max_chunks, int heads, int kv_heads, int head_dim,
                                               int page_size, int window, float scale, int tiled_out, void* stream) {
+    const Reach reach = {window, 0};
     if (check_common("attention_decode_fused_bf16", heads, kv_heads, head_dim, page_size, q_stride, table_width))
         return 1;
     RI_REQUIRE(!tiled_out || (seqs <= 64 && head_dim % 32 == 0), "attention_decode_fused_bf16: tiled rows are at most 64 (%d)", seqs);
@@ -218,14 +223,14 @@ extern "C" int ri_attention_decode_fused_bf16(void* out, float* workspace, const
         if (wide)                                                                                                 \
             attn_decode_stream_kernel<DH, true, 8><<<sgrid, 8 * 64, 0, s>>>(                                      \
                 (bf16_t*)out, workspace, (const bf16_t*)qkv, q_stride, q_gain, k_gain, eps, inv_freq,             \
-                (bf16_t*)k_pages, (bf16_t*)v_pages, tok_pos, page_table, table_width, heads, kv_heads, window,    \
+                (bf16_t*)k_pages, (bf16_t*)v_pages, tok_pos, page_table, table_width, heads, kv_heads, reach,     \
                 scale_log2, splits, tiled_out, 0.f, 0.f, nullptr, 0.f, nullptr);                                           \
         else                                                                                                      \
             attn_decode_stream_kernel<DH, true, 4><<<sgrid, 4 * 64, 0, s>>>(                                      \
                 (bf16_t*)out, workspace, (const bf16_t*)qkv, q_stride, q_gain, k_gain, eps, inv_freq,             \
-                (bf16_t*)k_pages, (bf16_t*)v_pages, tok_pos, page_table, table_width, heads, kv_heads, window,    \
+                (bf16_t*)k_pages, (bf16_t*)v_pages, tok_pos, page_table, table_width, heads, kv_heads, reach,     \
                 scale_log2, splits, tiled_out, 0.f, 0.f, nullptr, 0.f, nullptr);                                           \
-        if (splits > 1) launch_join<DH>((bf16_t*)out, workspace, tok_pos, seqs, heads, -1, splits, tiled_out, s); \
+        if (splits > 1) launch_join<DH>((bf16_t*)out, workspace, tok_pos, seqs, heads, Reach{-1, 0}, splits, tiled_out, s); \
         break;
         switch (head_dim) {
             RI_STREAM_CASE(32)
@@ -242,8 +247,8 @@ extern "C" int ri_attention_decode_fused_bf16(void* out, float* workspace, const
     case DH * 16 + CW:                                                                                            \
         attn_decode_fused_kernel<DH, CW><<<pgrid, CW * 64, 0, s>>>(                                               \
             workspace, (const bf16_t*)qkv, q_stride, q_gain, k_gain, eps, inv_freq, (bf16_t*)k_pages,             \
-            (bf16_t*)v_pages, tok_pos, page_table, table_width, heads, kv_heads, window, scale_log2, all);        \
-        launch_join<DH>((bf16_t*)out, workspace, tok_pos, seqs, heads, window, all, tiled_out, s, CW * PAGE);     \
+            (bf16_t*)v_pages, tok_pos, page_table, table_width, heads, kv_heads, reach, scale_log2, all);        \
+        launch_join<DH>((bf16_t*)out, workspace, tok_pos, seqs, heads, reach, all, tiled_out, s, CW * PAGE);     \
         break;
     switch (head_dim * 16 + DECODE_WAVES / pieces) {
         RI_FUSED_CASE(32, 8)

@@ -33,9 +33,11 @@ extern "C" int ri_attention_padded_fits(int dim, int vdim, int group, int decode
 extern "C" int ri_attention_prefill_padded_bf16(void* out, const void* qkv, int q_stride, const void* k_pages,
                                                 const void* v_pages, const int32_t* cu_seqlens, const int32_t* tok_pos,
                                                 const int32_t* page_table, int table_width, int seqs, int max_new,
-                                                int heads, int kv_heads, int dim, int vdim, int page_size, int window,
+                                                int heads, int kv_heads, int dim, int vdim, int page_size, int window, int chunk,
                                                 float scale, float softcap, const float* slopes, int keep_first,
                                                 const float* sinks, void* stream) {
+    RI_REQUIRE(chunk >= 0 && (chunk == 0 || window <= 0), "attention_prefill_padded: chunks of %d beside a window of %d", chunk, window);
+    const Reach reach = {window, chunk};
     RI_REQUIRE(keep_first >= 0, "attention_prefill_padded: %d first tokens kept", keep_first);
     if (check_padded("attention_prefill_padded", heads, kv_heads, dim, vdim, page_size, q_stride, table_width, scale)) return 1;
     const float cap_pre = softcap > 0.f ? scale / softcap : 0.f, cap_post = softcap > 0.f ? softcap / scale : 0.f;
@@ -58,7 +60,7 @@ extern "C" int ri_attention_prefill_padded_bf16(void* out, const void* qkv, int 
     case (DH * 8 + NT) * 512 + DV:                                                                                \
         attn_prefill_mfma_kernel<DH, NT, DV, true><<<grid, 256, 0, s>>>(                                           \
             (bf16_t*)out, (const bf16_t*)qkv, q_stride, (const bf16_t*)k_pages, (const bf16_t*)v_pages,          \
-            cu_seqlens, tok_pos, page_table, table_width, heads, kv_heads, window, scale_log2, cap_pre,          \
+            cu_seqlens, tok_pos, page_table, table_width, heads, kv_heads, reach, scale_log2, cap_pre,          \
             cap_post, slopes, 1.f / scale, keep_first, sinks, dim, vdim);                                         \
         break;
 #define RI_CASES(DH)                                                                                              \
@@ -79,9 +81,11 @@ extern "C" int ri_attention_prefill_padded_bf16(void* out, const void* qkv, int 
 extern "C" int ri_attention_decode_padded_bf16(void* out, float* workspace, const void* qkv, int q_stride,
                                                const void* k_pages, const void* v_pages, const int32_t* tok_pos,
                                                const int32_t* page_table, int table_width, int seqs, int max_chunks,
-                                               int heads, int kv_heads, int dim, int vdim, int page_size, int window,
+                                               int heads, int kv_heads, int dim, int vdim, int page_size, int window, int chunk,
                                                float scale, float softcap, const float* slopes, int tiled_out,
                                                int keep_first, const float* sinks, void* stream) {
+    RI_REQUIRE(chunk >= 0 && (chunk == 0 || window <= 0), "attention_decode_padded: chunks of %d beside a window of %d", chunk, window);
+    const Reach reach = {window, chunk};
     RI_REQUIRE(keep_first >= 0, "attention_decode_padded: %d first tokens kept", keep_first);
     if (check_padded("attention_decode_padded", heads, kv_heads, dim, vdim, page_size, q_stride, table_width, scale)) return 1;
     const float cap_pre = softcap > 0.f ? scale / softcap : 0.f, cap_post = softcap > 0.f ? softcap / scale : 0.f;
@@ -100,14 +104,14 @@ extern "C" int ri_attention_decode_padded_bf16(void* out, float* workspace, cons
 #define RI_STREAM(DH, W, DV)                                                                                      \
     attn_decode_stream_kernel<DH, false, W, DV, true><<<sgrid, W * 64, 0, s>>>(                                    \
         (bf16_t*)out, workspace, (const bf16_t*)qkv, q_stride, nullptr, nullptr, 0.f, nullptr, (bf16_t*)k_pages,  \
-        (bf16_t*)v_pages, tok_pos, page_table, table_width, heads, kv_heads, window, scale_log2, splits,          \
+        (bf16_t*)v_pages, tok_pos, page_table, table_width, heads, kv_heads, reach, scale_log2, splits,          \
         tiled_out, cap_pre, cap_post, slopes, 1.f / scale, sinks, dim, vdim)
 #define RI_CASE(DH, DV)                                                                                           \
     case DH * 512 + DV:                                                                                           \
         if (wide) RI_STREAM(DH, 8, DV);                                                                           \
         else RI_STREAM(DH, 4, DV);                                                                                \
         if (splits > 1)                                                                                           \
-            launch_join<DV, true>((bf16_t*)out, workspace, tok_pos, seqs, heads, -1, splits, tiled_out, s, DECODE_CHUNK, 0, \
+            launch_join<DV, true>((bf16_t*)out, workspace, tok_pos, seqs, heads, Reach{-1, 0}, splits, tiled_out, s, DECODE_CHUNK, 0, \
                                   sinks, vdim);                                                                   \
         break;
         switch (padded_dim(dim) * 512 + padded_vdim(vdim)) {
@@ -124,9 +128,9 @@ extern "C" int ri_attention_decode_padded_bf16(void* out, float* workspace, cons
     case (DH * 16 + CW) * 512 + DV:                                                                               \
         attn_decode_mfma_kernel<DH, CW, DV, true><<<pgrid, CW * 64, 0, s>>>(                                       \
             workspace, (const bf16_t*)qkv, q_stride, (const bf16_t*)k_pages, (const bf16_t*)v_pages, tok_pos,     \
-            page_table, table_width, heads, kv_heads, window, scale_log2, all, cap_pre, cap_post, slopes,         \
+            page_table, table_width, heads, kv_heads, reach, scale_log2, all, cap_pre, cap_post, slopes,         \
             1.f / scale, keep_first, dim, vdim);                                                                  \
-        launch_join<DV, true>((bf16_t*)out, workspace, tok_pos, seqs, heads, window, all, tiled_out, s, CW * PAGE,  \
+        launch_join<DV, true>((bf16_t*)out, workspace, tok_pos, seqs, heads, reach, all, tiled_out, s, CW * PAGE,  \
                               keep_first, sinks, vdim);                                                           \
         break;
 #define RI_CASE(DH, DV) RI_CHUNKS(DH, 8, DV) RI_CHUNKS(DH, 4, DV) RI_CHUNKS(DH, 2, DV)

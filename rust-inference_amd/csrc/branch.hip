@@ -11,6 +11,7 @@
 //                     several mixers side by side, for one output product);
 //   row_norm_gate:    out = scale * x / sqrt(mean(x^2) + eps) * gain * gate(g), the mean over the whole row (all heads
 //                     of a mixer together), likewise into columns of a wider row.
+//   normed_sum:       out = a_scale * norm(a) + b_scale * norm(b), RMS norms of two mixers' results over the model's width.
 //
 // The residual, the statistics of every norm, the layer scale and the gates' sigmoids are float32; a value is
 // rounded once, when it is stored in the activations' format.  One workgroup a row; a row's sums are taken in an
@@ -474,5 +475,109 @@ extern "C" int ri_row_norm_gate(void* out, int out_stride, int out_off, const fl
         row_norm_gate_kernel<bf16_t><<<rows, 256, 0, s>>>((bf16_t*)out + out_off, out_stride, x, gain, eps,
                                                           gate ? (const bf16_t*)gate + g_off : nullptr, gate_stride, scale, kind, width);
     RI_LAUNCH_CHECK("row_norm_gate");
+    return 0;
+}
+
+// ------------------------------------------------------------------ normed results of mixers side by side, added
+// out (+)= a_scale * rms_norm(a) * a_gain + b_scale * rms_norm(b) * b_gain: a and b are the results of two output products,
+// each [parts, rows, dim] (the parts added in order) or one part in the activations' format; b may be absent.
+template <typename T>
+__device__ __forceinline__ float4 parts4(const T* x, int parts, size_t stride, size_t at) {
+    float4 v = ld4(x + at);
+    for (int p = 1; p < parts; ++p) {
+        const float4 w = ld4(x + p * stride + at);
+        v = make_float4(v.x + w.x, v.y + w.y, v.z + w.z, v.w + w.w);
+    }
+    return v;
+}
+
+// Rows of up to 1,024 VPT elements in a multiple of 4: both rows in registers, one trip; one workgroup a row.
+template <typename TX, typename TY, int VPT>
+__global__ void __launch_bounds__(256)
+normed_sum_vec_kernel(float* __restrict__ out, int accumulate, const TX* __restrict__ a, int a_parts, const float* __restrict__ a_gain,
+                      float a_scale, const TY* __restrict__ b, int b_parts, const float* __restrict__ b_gain, float b_scale,
+                      float eps, size_t stride, int dim) {
+    __shared__ float scratch[16];
+    const size_t t = (size_t)blockIdx.x * dim;
+    float4 va[VPT], vb[VPT];
+    float sa = 0.f, sb = 0.f;
+#pragma unroll
+    for (int i = 0; i < VPT; ++i) {
+        const int c = (threadIdx.x + i * 256) * 4;
+        const bool ok = c < dim;
+        va[i] = parts4(a, a_parts, stride, t + (ok ? c : 0));
+        vb[i] = b ? parts4(b, b_parts, stride, t + (ok ? c : 0)) : make_float4(0.f, 0.f, 0.f, 0.f);
+        if (ok) {
+            sa += (va[i].x * va[i].x + va[i].y * va[i].y) + (va[i].z * va[i].z + va[i].w * va[i].w);
+            sb += (vb[i].x * vb[i].x + vb[i].y * vb[i].y) + (vb[i].z * vb[i].z + vb[i].w * vb[i].w);
+        }
+    }
+    const float fa = a_scale / sqrtf(block_sum(sa, scratch) / (float)dim + eps);
+    const float fb = b ? b_scale / sqrtf(block_sum(sb, scratch) / (float)dim + eps) : 0.f;
+#pragma unroll
+    for (int i = 0; i < VPT; ++i) {
+        const int c = (threadIdx.x + i * 256) * 4;
+        if (c >= dim) continue;
+        const float4 g = ld4(a_gain + c);
+        float4 v = make_float4(fa * va[i].x * g.x, fa * va[i].y * g.y, fa * va[i].z * g.z, fa * va[i].w * g.w);
+        if (b) {
+            const float4 h = ld4(b_gain + c);
+            v = make_float4(v.x + fb * vb[i].x * h.x, v.y + fb * vb[i].y * h.y, v.z + fb * vb[i].z * h.z, v.w + fb * vb[i].w * h.w);
+        }
+        if (accumulate) {
+            const float4 o = ld4(out + t + c);
+            v = make_float4(v.x + o.x, v.y + o.y, v.z + o.z, v.w + o.w);
+        }
+        st4(out + t + c, v);
+    }
+}
+
+template <typename T>
+__device__ __forceinline__ float parts1(const T* x, int parts, size_t stride, size_t at) {
+    float v = to_f32(x[at]);
+    for (int p = 1; p < parts; ++p) v += to_f32(x[p * stride + at]);
+    return v;
+}
+
+template <typename TX, typename TY>
+__global__ void __launch_bounds__(256)
+normed_sum_kernel(float* __restrict__ out, int accumulate, const TX* __restrict__ a, int a_parts, const float* __restrict__ a_gain,
+                  float a_scale, const TY* __restrict__ b, int b_parts, const float* __restrict__ b_gain, float b_scale, float eps,
+                  size_t stride, int dim) {
+    __shared__ float scratch[16];
+    const size_t t = (size_t)blockIdx.x * dim;
+    float sa = 0.f, sb = 0.f;
+    for (int d = threadIdx.x; d < dim; d += blockDim.x) {
+        const float x = parts1(a, a_parts, stride, t + d), y = b ? parts1(b, b_parts, stride, t + d) : 0.f;
+        sa += x * x;
+        sb += y * y;
+    }
+    const float fa = a_scale / sqrtf(block_sum(sa, scratch) / (float)dim + eps);
+    const float fb = b ? b_scale / sqrtf(block_sum(sb, scratch) / (float)dim + eps) : 0.f;
+    for (int d = threadIdx.x; d < dim; d += blockDim.x) {
+        float v = fa * parts1(a, a_parts, stride, t + d) * a_gain[d];
+        if (b) v += fb * parts1(b, b_parts, stride, t + d) * b_gain[d];
+        out[t + d] = accumulate ? out[t + d] + v : v;
+    }
+}
+
+extern "C" int ri_normed_sum(float* out, int accumulate, const void* a, int a_dtype, int a_parts, const float* a_gain, float a_scale,
+                             const void* b, int b_dtype, int b_parts, const float* b_gain, float b_scale, float eps, int rows,
+                             int dim, void* stream) {
+    RI_REQUIRE(out && a && a_gain && rows > 0 && dim > 0 && a_parts >= 1 && (!b || (b_gain && b_parts >= 1)),
+               "normed_sum: %d rows of %d, %d and %d parts", rows, dim, a_parts, b_parts);
+    RI_REQUIRE((a_dtype == RI_F32 || (a_dtype == RI_BF16 && a_parts == 1)) && (!b || b_dtype == RI_F32 || (b_dtype == RI_BF16 && b_parts == 1)),
+               "normed_sum: parts of a product are float32");
+    hipStream_t s = (hipStream_t)stream;
+    const size_t stride = (size_t)rows * dim;
+    const bool vec = dim % 4 == 0 && dim <= 8192;
+    const int vpt = (dim / 4 + 255) / 256;
+#define RI_ARGS(TX, TY) out, accumulate, (const TX*)a, a_parts, a_gain, a_scale, (const TY*)b, b_parts, b_gain, b_scale, eps, stride, dim
+#define RI_GO(TX, TY)                                                                                       if (!vec) normed_sum_kernel<TX, TY><<<rows, 256, 0, s>>>(RI_ARGS(TX, TY));                              else if (vpt <= 1) normed_sum_vec_kernel<TX, TY, 1><<<rows, 256, 0, s>>>(RI_ARGS(TX, TY));              else if (vpt <= 2) normed_sum_vec_kernel<TX, TY, 2><<<rows, 256, 0, s>>>(RI_ARGS(TX, TY));              else if (vpt <= 4) normed_sum_vec_kernel<TX, TY, 4><<<rows, 256, 0, s>>>(RI_ARGS(TX, TY));              else normed_sum_vec_kernel<TX, TY, 8><<<rows, 256, 0, s>>>(RI_ARGS(TX, TY))
+    if (a_dtype == RI_F32) { if (!b || b_dtype == RI_F32) { RI_GO(float, float); } else { RI_GO(float, bf16_t); } }
+    else                   { if (!b || b_dtype == RI_F32) { RI_GO(bf16_t, float); } else { RI_GO(bf16_t, bf16_t); } }
+#undef RI_GO
+#undef RI_ARGS
+    RI_LAUNCH_CHECK("normed_sum");
     return 0;
 }

@@ -99,6 +99,17 @@ __device__ __forceinline__ float block_max(float v, float* scratch) {
     return total;
 }
 
+// What the query at position p sees of the keys before it: all of them (both members 0), the last `window` with its own, or
+// those of the run of `chunk` positions that p lies in (runs are counted from the sequence's first position).  A negative
+// window limits nothing: the join of the attention's decode kernels takes it as a mark.
+struct Reach {
+    int window, chunk;
+    __device__ __forceinline__ int first(int p) const {
+        if (chunk > 0) return p - p % chunk;
+        return window > 0 ? max(0, p - window + 1) : 0;
+    }
+};
+
 // How a decode-size product is linked to the RMSNorms around it, so that the norms need no kernels
 // of their own.  y = W . norm(r) with norm(r) = r * inv * g is computed as inv * (W . (r * g)): the
 // producer of r leaves xg = bfloat16(r * g) and partial sums of r^2; the consumer adds the partial

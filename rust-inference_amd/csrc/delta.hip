@@ -6,6 +6,8 @@
 //     q <- q / sqrt(sum q^2 + 1e-6) * dim^(-1/2),   k <- k / sqrt(sum k^2 + 1e-6)      per head
 //     beta = sigmoid(b),   g = exp(-exp(A_log) * softplus(a + dt_bias))               per value head
 //     S <- g S;   u = beta (v - S^T k);   S <- S + k u^T;   o = S^T q.
+// With a decay per key channel (CH in the kernels) g is a number per head and row of S, g = exp(-exp(A_log_h) *
+// softplus(z + dt_bias)) of z [heads * dim], S <- diag(g) S, and the output gate is the sigmoid of a product's float32 result.
 // Everything after the projections is float32.  ri_delta_prepare makes q, k, v, g and beta of all tokens of a step
 // (a workgroup a token and head), ri_delta_tails then moves the convolutions' last inputs into the sequences' state, and
 // ri_delta_scan walks every sequence's tokens in order.  A token's sums are taken in the same order whatever step
@@ -24,18 +26,32 @@ __device__ __forceinline__ float softplus_f(float v) { return fmaxf(v, 0.f) + lo
 // turn waiting for its own loads: 22 us for a single token.)
 #define DELTA_V_UNIT 256
 
-template <typename T>
+// CH: ab holds z, rows of z_row elements, the logits of beta are those of bsrc (rows of b_row), and the units behind
+// those of v are stretches of DELTA_V_UNIT of the decays; gates is [heads * dim decays, heads betas] a token.
+template <typename T, bool CH>
 __global__ void __launch_bounds__(256)
 delta_prepare_kernel(float* __restrict__ qkv, float* __restrict__ gates, const T* __restrict__ proj, int row, int q_off,
                      const float* __restrict__ taps, int ntaps, const float* __restrict__ tails,
                      const float* __restrict__ ab, const float* __restrict__ a_log, const float* __restrict__ dt_bias,
                      const int32_t* __restrict__ tok_seq, const int32_t* __restrict__ cu_seqlens,
-                     const int32_t* __restrict__ slots, int heads, int kv_heads, int dim, int vdim) {
+                     const int32_t* __restrict__ slots, int heads, int kv_heads, int dim, int vdim, int z_row,
+                     const T* __restrict__ bsrc, int b_row) {
     extern __shared__ float conv[];
     __shared__ float scratch[16];
     const int t = blockIdx.x, unit = blockIdx.y, b = tok_seq[t];
     const int i = t - cu_seqlens[b];                          // the token's place among its sequence's new tokens
     const int qk = kv_heads * dim, channels = 2 * qk + heads * vdim;
+    if (CH) {
+        const int decays = heads * dim, at = (unit - 2 * kv_heads - (heads * vdim + DELTA_V_UNIT - 1) / DELTA_V_UNIT) * DELTA_V_UNIT;
+        float* to = gates + (size_t)t * (decays + heads);
+        if (at >= 0) {                                        // a stretch of decays (the whole workgroup)
+            const int e = at + threadIdx.x;
+            if (e < decays) to[e] = expf(-expf(a_log[e / dim]) * softplus_f(ab[(size_t)t * z_row + e] + dt_bias[e]));
+            return;
+        }
+        if (unit == 0)
+            for (int h = threadIdx.x; h < heads; h += blockDim.x) to[decays + h] = 1.f / (1.f + expf(-to_f32(bsrc[(size_t)t * b_row + h])));
+    }
     const bool normed = unit < 2 * kv_heads;
     const int first = normed ? unit * dim : 2 * qk + (unit - 2 * kv_heads) * DELTA_V_UNIT;
     const int count = normed ? dim : min(DELTA_V_UNIT, channels - first);
@@ -84,7 +100,7 @@ delta_prepare_kernel(float* __restrict__ qkv, float* __restrict__ gates, const T
     } else {
         for (int e = threadIdx.x; e < count; e += blockDim.x) out[e] = conv[e];
     }
-    if (unit == 0 && threadIdx.x < heads) {
+    if (!CH && unit == 0 && threadIdx.x < heads) {
         const int h = threadIdx.x;
         const float a = ab[(size_t)t * 2 * heads + h], bb = ab[(size_t)t * 2 * heads + heads + h];
         gates[(size_t)t * 2 * heads + h] = expf(-expf(a_log[h]) * softplus_f(a + dt_bias[h]));
@@ -134,7 +150,7 @@ __device__ __forceinline__ float slices_sum(float v) {
 // flight while a block is walked.  The two sums over rows of a token meet over the SL lanes of a column.  A token costs
 // a wavefront 4 RPT vector instructions and nothing hides them, so eight slices halve a token's time; they also
 // double the workgroups that each stage q and k, which is what counts once the machine is full: the launch chooses.
-template <int RPT, int SL>
+template <int RPT, int SL, bool CH>
 struct DeltaLds {
     static constexpr int DELTA_BLOCK = RPT * SL >= 256 ? 8 : 16;    // tokens a block: two buffers stay inside 64 KB
     static constexpr int QS = RPT + 4;                        // stride of a slice of q or k: no bank conflicts between the slices
@@ -142,16 +158,17 @@ struct DeltaLds {
     float q[DELTA_BLOCK][SL][QS];
     float k[DELTA_BLOCK][SL][QS];
     float v[DELTA_BLOCK][COLS];
-    float g[DELTA_BLOCK], beta[DELTA_BLOCK];
+    float g[CH ? 1 : DELTA_BLOCK], beta[DELTA_BLOCK];
+    float gk[CH ? DELTA_BLOCK : 1][SL][CH ? QS : 1];          // a decay a row
 };
 
-template <int RPT, int SL>
+template <int RPT, int SL, bool CH>
 __global__ void __launch_bounds__(256)
 delta_scan_kernel(float* __restrict__ out, const float* __restrict__ qkv, const float* __restrict__ gates,
                   float* __restrict__ state, const int32_t* __restrict__ cu_seqlens, const int32_t* __restrict__ slots,
                   int heads, int kv_heads, int dim, int vdim) {
-    __shared__ DeltaLds<RPT, SL> lds[2];
-    constexpr int DELTA_BLOCK = DeltaLds<RPT, SL>::DELTA_BLOCK, COLS = DeltaLds<RPT, SL>::COLS;
+    __shared__ DeltaLds<RPT, SL, CH> lds[2];
+    constexpr int DELTA_BLOCK = DeltaLds<RPT, SL, CH>::DELTA_BLOCK, COLS = DeltaLds<RPT, SL, CH>::COLS;
     constexpr int QR = DELTA_BLOCK * SL * RPT / 256;          // elements of q (and of k) a thread fetches per block
     constexpr int VR = DELTA_BLOCK * COLS / 256;
     const int b = blockIdx.x / heads, h = blockIdx.x % heads, col0 = blockIdx.y * COLS;
@@ -172,7 +189,8 @@ delta_scan_kernel(float* __restrict__ out, const float* __restrict__ qkv, const 
         S[i] = (has_col && rw < dim) ? v : 0.f;
     }
 
-    float fq[QR], fk[QR], fv[VR], fg = 0.f;
+    const int gate_row = CH ? heads * dim + heads : 2 * heads;
+    float fq[QR], fk[QR], fgk[CH ? QR : 1], fv[VR], fg = 0.f;
     auto fetch = [&](int first) {                             // the block of tokens first ..+DELTA_BLOCK, into registers
 #pragma unroll
         for (int e = 0; e < QR; ++e) {
@@ -182,6 +200,7 @@ delta_scan_kernel(float* __restrict__ out, const float* __restrict__ qkv, const 
             const float a = p[0], c = p[qk];
             fq[e] = ok ? a : 0.f;
             fk[e] = ok ? c : 0.f;
+            if (CH) fgk[e] = gates[(size_t)(t0 + min(first + tk, n - 1)) * gate_row + h * dim + min(rw, dim - 1)];
         }
 #pragma unroll
         for (int e = 0; e < VR; ++e) {
@@ -191,15 +210,16 @@ delta_scan_kernel(float* __restrict__ out, const float* __restrict__ qkv, const 
         }
         if (tid < 2 * DELTA_BLOCK) {
             const int tk = tid >> 1;
-            fg = gates[(size_t)(t0 + min(first + tk, n - 1)) * 2 * heads + (tid & 1) * heads + h];
+            fg = gates[(size_t)(t0 + min(first + tk, n - 1)) * gate_row + (CH ? heads * dim : (tid & 1) * heads) + h];
         }
     };
-    auto stage = [&](DeltaLds<RPT, SL>& l) {
+    auto stage = [&](DeltaLds<RPT, SL, CH>& l) {
 #pragma unroll
         for (int e = 0; e < QR; ++e) {
             const int at = e * 256 + tid, tk = at / (SL * RPT), rw = at % (SL * RPT);
             l.q[tk][rw / RPT][rw % RPT] = fq[e];
             l.k[tk][rw / RPT][rw % RPT] = fk[e];
+            if (CH) l.gk[tk][rw / RPT][rw % RPT] = fgk[e];
         }
 #pragma unroll
         for (int e = 0; e < VR; ++e) {
@@ -207,7 +227,7 @@ delta_scan_kernel(float* __restrict__ out, const float* __restrict__ qkv, const 
             l.v[at / COLS][at % COLS] = fv[e];
         }
         if (tid < 2 * DELTA_BLOCK) {
-            if (tid & 1) l.beta[tid >> 1] = fg; else l.g[tid >> 1] = fg;
+            if (tid & 1) l.beta[tid >> 1] = fg; else if (!CH) l.g[tid >> 1] = fg;
         }
     };
 
@@ -218,17 +238,17 @@ delta_scan_kernel(float* __restrict__ out, const float* __restrict__ qkv, const 
     for (int first = 0; first < n; first += DELTA_BLOCK) {
         const bool more = first + DELTA_BLOCK < n;
         fetch(more ? first + DELTA_BLOCK : first);            // (always issued: no load in a branch)
-        const DeltaLds<RPT, SL>& l = lds[cur];
+        const DeltaLds<RPT, SL, CH>& l = lds[cur];
         const int count = min(DELTA_BLOCK, n - first);
 #pragma unroll 2
         for (int tk = 0; tk < count; ++tk) {
-            const float g = l.g[tk], beta = l.beta[tk];
+            const float g = CH ? 1.f : l.g[tk], beta = l.beta[tk];
             // four partial sums each: a single one would be a chain of RPT dependent additions
             float kk[RPT], d4[4] = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
             for (int i = 0; i < RPT; ++i) {
                 kk[i] = l.k[tk][r][i];
-                S[i] *= g;
+                S[i] *= CH ? l.gk[tk][r][i] : g;
                 d4[i & 3] += S[i] * kk[i];
             }
             const float dot = slices_sum<SL>((d4[0] + d4[1]) + (d4[2] + d4[3]));
@@ -258,14 +278,16 @@ delta_scan_kernel(float* __restrict__ out, const float* __restrict__ qkv, const 
 // state, four columns each (16-byte loads and stores of whole lines), x 256 / groups slices of rows, a thread RPT rows
 // in registers.  The sums over rows meet through LDS, slice after slice.  The convolutions' tails are read here and
 // moved on by delta_tails_kernel afterwards (the heads that share a q/k head all read its tail).
-template <typename T, int RPT>
+// CH: ab holds z (rows of z_row elements, the gate's pre-activations from column gate_at of them on), the logits of beta
+// are those of bsrc, the gate is a sigmoid.
+template <typename T, int RPT, bool CH>
 __global__ void __launch_bounds__(256)
 delta_step_kernel(T* __restrict__ out, const T* __restrict__ proj, int row, int q_off, int g_off,
                   const float* __restrict__ taps, int ntaps, const float* __restrict__ tails, const float* __restrict__ ab,
                   const float* __restrict__ a_log, const float* __restrict__ dt_bias, float* __restrict__ state,
                   const int32_t* __restrict__ slots, const float* __restrict__ gain, float eps, int heads, int kv_heads,
-                  int dim, int vdim, int groups) {
-    __shared__ float qs[256], ks[256], vs[256], scratch[16];
+                  int dim, int vdim, int groups, int z_row, int gate_at, const T* __restrict__ bsrc, int b_row) {
+    __shared__ float qs[256], ks[256], vs[256], gs[CH ? 256 : 1], scratch[16];
     __shared__ float4 part[256];
     const int h = blockIdx.x, b = blockIdx.y, tid = threadIdx.x;
     const int hq = h / (heads / kv_heads), slot = slots[b];
@@ -284,14 +306,16 @@ delta_step_kernel(T* __restrict__ out, const T* __restrict__ proj, int row, int 
     const T* x = proj + (size_t)b * row;
     const float* tail = tails + (size_t)slot * (ntaps - 1) * channels;
     // everything the end of the kernel reads from memory is asked for here, so that no load is waited for on its own
-    const float a_in = ab[(size_t)b * 2 * heads + h], b_in = ab[(size_t)b * 2 * heads + heads + h];
-    const float a_exp = a_log[h], a_bias = dt_bias[h];
+    const float* zr = ab + (size_t)b * (CH ? z_row : 2 * heads);
+    const float a_in = CH ? 0.f : zr[h], b_in = CH ? to_f32(bsrc[(size_t)b * b_row + h]) : zr[heads + h];
+    const float a_exp = a_log[h], a_bias = CH ? 0.f : dt_bias[h];
     float gate[4], gain_c[4];
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
-        gate[j] = to_f32(x[g_off + h * vdim + min(c0, vdim - 4) + j]);
+        gate[j] = CH ? zr[gate_at + h * vdim + min(c0, vdim - 4) + j] : to_f32(x[g_off + h * vdim + min(c0, vdim - 4) + j]);
         gain_c[j] = gain[min(c0, vdim - 4) + j];
     }
+    if (CH && tid < dim) gs[tid] = expf(-expf(a_exp) * softplus_f(zr[h * dim + tid] + dt_bias[h * dim + tid]));      // (dim <= 256)
     for (int e = tid; e < 2 * dim + vdim; e += 256) {
         const int ch = e < dim ? hq * dim + e : e < 2 * dim ? qk + hq * dim + (e - dim) : 2 * qk + h * vdim + (e - 2 * dim);
         float y = 0.f;
@@ -323,7 +347,7 @@ delta_step_kernel(T* __restrict__ out, const T* __restrict__ proj, int row, int 
     sq = block_sum(sq, scratch);
     sk = block_sum(sk, scratch);
     const float fq = rsqrtf((float)dim) / sqrtf(sq + 1e-6f), fk = 1.f / sqrtf(sk + 1e-6f);
-    const float g = expf(-expf(a_exp) * softplus_f(a_in + a_bias));
+    const float g_head = CH ? 1.f : expf(-expf(a_exp) * softplus_f(a_in + a_bias));
     const float beta = 1.f / (1.f + expf(-b_in));
     float kk[RPT];
     float4 d = make_float4(0.f, 0.f, 0.f, 0.f);
@@ -331,6 +355,7 @@ delta_step_kernel(T* __restrict__ out, const T* __restrict__ proj, int row, int 
     for (int i = 0; i < RPT; ++i) {
         const int rw = r * RPT + i;
         kk[i] = rw < dim ? ks[rw] * fk : 0.f;
+        const float g = CH ? gs[min(rw, dim - 1)] : g_head;
         S[i].x *= g; S[i].y *= g; S[i].z *= g; S[i].w *= g;
         d.x += S[i].x * kk[i]; d.y += S[i].y * kk[i]; d.z += S[i].z * kk[i]; d.w += S[i].w * kk[i];
     }
@@ -365,10 +390,11 @@ delta_step_kernel(T* __restrict__ out, const T* __restrict__ proj, int row, int 
     if (r == 0 && has_col) {
         const float inv = 1.f / sqrtf(ss / (float)vdim + eps);
         T* to = out + (size_t)b * heads * vdim + (size_t)h * vdim + c0;
-        from_f32(to, o.x * inv * gain_c[0] * silu_f(gate[0]));
-        from_f32(to + 1, o.y * inv * gain_c[1] * silu_f(gate[1]));
-        from_f32(to + 2, o.z * inv * gain_c[2] * silu_f(gate[2]));
-        from_f32(to + 3, o.w * inv * gain_c[3] * silu_f(gate[3]));
+        auto open = [](float z) { return CH ? 1.f / (1.f + expf(-z)) : silu_f(z); };
+        from_f32(to, o.x * inv * gain_c[0] * open(gate[0]));
+        from_f32(to + 1, o.y * inv * gain_c[1] * open(gate[1]));
+        from_f32(to + 2, o.z * inv * gain_c[2] * open(gate[2]));
+        from_f32(to + 3, o.w * inv * gain_c[3] * open(gate[3]));
     }
 }
 
@@ -384,24 +410,26 @@ extern "C" int ri_delta_step_fits(int dim, int vdim) {
     return (dim + slices - 1) / slices <= 16;
 }
 
-extern "C" int ri_delta_step(void* out, const void* proj, int act_dtype, int row, int q_off, int g_off, const float* taps,
+template <bool CH>
+static int launch_delta_step(void* out, const void* proj, int act_dtype, int row, int q_off, int g_off, const float* taps,
                              int ntaps, float* tails, const float* ab, const float* a_log, const float* dt_bias,
                              float* state, const int32_t* cu_seqlens, const int32_t* slots, const float* gain, float eps,
-                             int seqs, int heads, int kv_heads, int dim, int vdim, void* stream) {
+                             int seqs, int heads, int kv_heads, int dim, int vdim, int z_row, int gate_at, const void* bsrc,
+                             int b_row, void* stream) {
     RI_REQUIRE(seqs > 0 && seqs <= 65535 && heads > 0 && heads <= 65535 && kv_heads > 0 && heads % kv_heads == 0,
                "delta_step: %d sequences, %d heads, %d kv heads", seqs, heads, kv_heads);
     RI_REQUIRE(ri_delta_step_fits(dim, vdim), "delta_step: heads of %d x %d", dim, vdim);
     RI_REQUIRE(ntaps >= 1 && ntaps <= DELTA_MAX_TAPS, "delta_step: %d taps, the kernels take 1 to %d", ntaps, DELTA_MAX_TAPS);
     const long channels = 2L * kv_heads * dim + (long)heads * vdim;
-    RI_REQUIRE(q_off >= 0 && q_off + channels <= row && g_off >= 0 && g_off + (long)heads * vdim <= row,
+    RI_REQUIRE(q_off >= 0 && q_off + channels <= row && (CH || (g_off >= 0 && g_off + (long)heads * vdim <= row)),
                "delta_step: %ld channels at column %d and the gate at %d of rows of %d", channels, q_off, g_off, row);
     RI_REQUIRE(act_dtype == RI_F32 || act_dtype == RI_BF16, "delta_step: dtype %d", act_dtype);
     hipStream_t s = (hipStream_t)stream;
     const int groups = delta_step_cols(vdim) / 4, slices = 256 / groups, rpt = (dim + slices - 1) / slices;
     const dim3 grid(heads, seqs);
-#define RI_DSTEP_GO(T, R) delta_step_kernel<T, R><<<grid, 256, 0, s>>>((T*)out, (const T*)proj, row, q_off, g_off, taps, ntaps, \
+#define RI_DSTEP_GO(T, R) delta_step_kernel<T, R, CH><<<grid, 256, 0, s>>>((T*)out, (const T*)proj, row, q_off, g_off, taps, ntaps, \
                                                                     tails, ab, a_log, dt_bias, state, slots, gain, eps, heads,   \
-                                                                    kv_heads, dim, vdim, groups)
+                                                                    kv_heads, dim, vdim, groups, z_row, gate_at, (const T*)bsrc, b_row)
     if (act_dtype == RI_F32) {
         if (rpt <= 4) RI_DSTEP_GO(float, 4); else if (rpt <= 8) RI_DSTEP_GO(float, 8); else RI_DSTEP_GO(float, 16);
     } else {
@@ -420,15 +448,42 @@ extern "C" int ri_delta_step(void* out, const void* proj, int act_dtype, int row
     return 0;
 }
 
-extern "C" int ri_delta_prepare(float* qkv, float* gates, const void* proj, int act_dtype, int row, int q_off,
+extern "C" int ri_delta_step(void* out, const void* proj, int act_dtype, int row, int q_off, int g_off, const float* taps,
+                             int ntaps, float* tails, const float* ab, const float* a_log, const float* dt_bias,
+                             float* state, const int32_t* cu_seqlens, const int32_t* slots, const float* gain, float eps,
+                             int seqs, int heads, int kv_heads, int dim, int vdim, void* stream) {
+    return launch_delta_step<false>(out, proj, act_dtype, row, q_off, g_off, taps, ntaps, tails, ab, a_log, dt_bias, state,
+                                    cu_seqlens, slots, gain, eps, seqs, heads, kv_heads, dim, vdim, 0, 0, nullptr, 0, stream);
+}
+
+// Rows of pre-activations of a decay per key channel: what both entry points below ask of them.
+static int check_channels(const char* name, const void* z, int z_row, const void* b, int b_row, int heads, int dim) {
+    RI_REQUIRE(z && b && z_row >= heads * dim && b_row >= heads, "%s: decays in rows of %d, betas in rows of %d for %d heads of %d", name,
+               z_row, b_row, heads, dim);
+    return 0;
+}
+
+extern "C" int ri_delta_step_channels(void* out, const void* proj, int act_dtype, int row, int q_off, const float* taps, int ntaps,
+                                      float* tails, const float* z, int z_row, int gate_at, const void* b, int b_row,
+                                      const float* a_log, const float* dt_bias, float* state, const int32_t* cu_seqlens,
+                                      const int32_t* slots, const float* gain, float eps, int seqs, int heads, int kv_heads,
+                                      int dim, int vdim, void* stream) {
+    if (check_channels("delta_step_channels", z, z_row, b, b_row, heads, dim)) return 1;
+    RI_REQUIRE(gate_at >= 0 && gate_at + (long)heads * vdim <= z_row, "delta_step_channels: the gate at %d of rows of %d", gate_at, z_row);
+    return launch_delta_step<true>(out, proj, act_dtype, row, q_off, 0, taps, ntaps, tails, z, a_log, dt_bias, state, cu_seqlens,
+                                   slots, gain, eps, seqs, heads, kv_heads, dim, vdim, z_row, gate_at, b, b_row, stream);
+}
+
+template <bool CH>
+static int launch_delta_prepare(float* qkv, float* gates, const void* proj, int act_dtype, int row, int q_off,
                                 const float* taps, int ntaps, float* tails, const float* ab, const float* a_log,
                                 const float* dt_bias, const int32_t* tok_seq, const int32_t* cu_seqlens,
                                 const int32_t* slots, int seqs, int tokens, int heads, int kv_heads, int dim, int vdim,
-                                void* stream) {
+                                int z_row, const void* bsrc, int b_row, void* stream) {
     RI_REQUIRE(tokens > 0 && seqs > 0 && heads > 0 && kv_heads > 0 && heads % kv_heads == 0 && dim > 0 && vdim > 0,
                "delta_prepare: tokens %d, sequences %d, heads %d, kv heads %d of %d x %d", tokens, seqs, heads, kv_heads,
                dim, vdim);
-    RI_REQUIRE(heads <= 256, "delta_prepare: %d heads, the kernel takes up to 256", heads);
+    RI_REQUIRE(CH || heads <= 256, "delta_prepare: %d heads, the kernel takes up to 256", heads);
     RI_REQUIRE(ntaps >= 1 && ntaps <= DELTA_MAX_TAPS, "delta_prepare: %d taps, the kernels take 1 to %d", ntaps, DELTA_MAX_TAPS);
     const long channels = 2L * kv_heads * dim + (long)heads * vdim;
     RI_REQUIRE(q_off >= 0 && q_off + channels <= row, "delta_prepare: %ld channels at column %d of rows of %d", channels, q_off, row);
@@ -436,17 +491,17 @@ extern "C" int ri_delta_prepare(float* qkv, float* gates, const void* proj, int 
     RI_REQUIRE(act_dtype == RI_F32 || act_dtype == RI_BF16, "delta_prepare: dtype %d", act_dtype);
     hipStream_t s = (hipStream_t)stream;
     const size_t shared = (size_t)(dim > DELTA_V_UNIT ? dim : DELTA_V_UNIT) * sizeof(float);
-    const int units = 2 * kv_heads + (heads * vdim + DELTA_V_UNIT - 1) / DELTA_V_UNIT;
+    const int units = 2 * kv_heads + (heads * vdim + DELTA_V_UNIT - 1) / DELTA_V_UNIT + (CH ? (heads * dim + DELTA_V_UNIT - 1) / DELTA_V_UNIT : 0);
     RI_REQUIRE(units <= 65535, "delta_prepare: %d units of channels exceed one launch", units);
     const dim3 pgrid(tokens, units);
     if (act_dtype == RI_F32) {
-        delta_prepare_kernel<float><<<pgrid, 256, shared, s>>>(qkv, gates, (const float*)proj, row, q_off, taps, ntaps, tails,
-                                                               ab, a_log, dt_bias, tok_seq, cu_seqlens, slots, heads,
-                                                               kv_heads, dim, vdim);
+        delta_prepare_kernel<float, CH><<<pgrid, 256, shared, s>>>(qkv, gates, (const float*)proj, row, q_off, taps, ntaps, tails,
+                                                                   ab, a_log, dt_bias, tok_seq, cu_seqlens, slots, heads,
+                                                                   kv_heads, dim, vdim, z_row, (const float*)bsrc, b_row);
     } else {
-        delta_prepare_kernel<bf16_t><<<pgrid, 256, shared, s>>>(qkv, gates, (const bf16_t*)proj, row, q_off, taps, ntaps,
-                                                                tails, ab, a_log, dt_bias, tok_seq, cu_seqlens, slots,
-                                                                heads, kv_heads, dim, vdim);
+        delta_prepare_kernel<bf16_t, CH><<<pgrid, 256, shared, s>>>(qkv, gates, (const bf16_t*)proj, row, q_off, taps, ntaps,
+                                                                    tails, ab, a_log, dt_bias, tok_seq, cu_seqlens, slots,
+                                                                    heads, kv_heads, dim, vdim, z_row, (const bf16_t*)bsrc, b_row);
     }
     RI_LAUNCH_CHECK("delta_prepare");
     if (ntaps > 1) {
@@ -460,9 +515,29 @@ extern "C" int ri_delta_prepare(float* qkv, float* gates, const void* proj, int 
     return 0;
 }
 
+extern "C" int ri_delta_prepare(float* qkv, float* gates, const void* proj, int act_dtype, int row, int q_off,
+                                const float* taps, int ntaps, float* tails, const float* ab, const float* a_log,
+                                const float* dt_bias, const int32_t* tok_seq, const int32_t* cu_seqlens,
+                                const int32_t* slots, int seqs, int tokens, int heads, int kv_heads, int dim, int vdim,
+                                void* stream) {
+    return launch_delta_prepare<false>(qkv, gates, proj, act_dtype, row, q_off, taps, ntaps, tails, ab, a_log, dt_bias, tok_seq,
+                                       cu_seqlens, slots, seqs, tokens, heads, kv_heads, dim, vdim, 0, nullptr, 0, stream);
+}
+
+extern "C" int ri_delta_prepare_channels(float* qkv, float* gates, const void* proj, int act_dtype, int row, int q_off,
+                                         const float* taps, int ntaps, float* tails, const float* z, int z_row, const void* b,
+                                         int b_row, const float* a_log, const float* dt_bias, const int32_t* tok_seq,
+                                         const int32_t* cu_seqlens, const int32_t* slots, int seqs, int tokens, int heads,
+                                         int kv_heads, int dim, int vdim, void* stream) {
+    if (check_channels("delta_prepare_channels", z, z_row, b, b_row, heads, dim)) return 1;
+    return launch_delta_prepare<true>(qkv, gates, proj, act_dtype, row, q_off, taps, ntaps, tails, z, a_log, dt_bias, tok_seq,
+                                      cu_seqlens, slots, seqs, tokens, heads, kv_heads, dim, vdim, z_row, b, b_row, stream);
+}
+
 extern "C" int ri_delta_max_dim() { return 256; }
 
-extern "C" int ri_delta_scan(float* out, const float* qkv, const float* gates, float* state, const int32_t* cu_seqlens,
+template <bool CH>
+static int launch_delta_scan(float* out, const float* qkv, const float* gates, float* state, const int32_t* cu_seqlens,
                              const int32_t* slots, int seqs, int tokens, int heads, int kv_heads, int dim, int vdim,
                              int slices, void* stream) {
     RI_REQUIRE(slices == 0 || slices == 4 || slices == 8, "delta_scan: %d slices of rows (4, 8, or 0 for the launch's choice)", slices);
@@ -477,7 +552,7 @@ extern "C" int ri_delta_scan(float* out, const float* qkv, const float* gates, f
     const int sl = eight ? 8 : 4, cols = 256 / sl;
     const dim3 grid((unsigned)(seqs * heads), (unsigned)((vdim + cols - 1) / cols));
     const int need = (dim + sl - 1) / sl;
-#define RI_DELTA_GO(R, SL) delta_scan_kernel<R, SL><<<grid, 256, 0, s>>>(out, qkv, gates, state, cu_seqlens, slots, heads, kv_heads, dim, vdim)
+#define RI_DELTA_GO(R, SL) delta_scan_kernel<R, SL, CH><<<grid, 256, 0, s>>>(out, qkv, gates, state, cu_seqlens, slots, heads, kv_heads, dim, vdim)
     if (eight) {
         if (need <= 4) RI_DELTA_GO(4, 8);
         else if (need <= 8) RI_DELTA_GO(8, 8);
@@ -493,4 +568,16 @@ extern "C" int ri_delta_scan(float* out, const float* qkv, const float* gates, f
 #undef RI_DELTA_GO
     RI_LAUNCH_CHECK("delta_scan");
     return 0;
+}
+
+extern "C" int ri_delta_scan(float* out, const float* qkv, const float* gates, float* state, const int32_t* cu_seqlens,
+                             const int32_t* slots, int seqs, int tokens, int heads, int kv_heads, int dim, int vdim,
+                             int slices, void* stream) {
+    return launch_delta_scan<false>(out, qkv, gates, state, cu_seqlens, slots, seqs, tokens, heads, kv_heads, dim, vdim, slices, stream);
+}
+
+extern "C" int ri_delta_scan_channels(float* out, const float* qkv, const float* gates, float* state, const int32_t* cu_seqlens,
+                                      const int32_t* slots, int seqs, int tokens, int heads, int kv_heads, int dim, int vdim,
+                                      int slices, void* stream) {
+    return launch_delta_scan<true>(out, qkv, gates, state, cu_seqlens, slots, seqs, tokens, heads, kv_heads, dim, vdim, slices, stream);
 }

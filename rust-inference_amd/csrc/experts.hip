@@ -443,9 +443,9 @@ template <typename TX, typename TS>
 __global__ void __launch_bounds__(256)
 experts_finish_kernel(float* __restrict__ out, const float* __restrict__ routed, int parts, size_t part_stride,
                       const TX* __restrict__ x, const TS* __restrict__ shared, int shared_parts,
-                      const float* __restrict__ extra, int dim) {
+                      const float* __restrict__ extra, const float* __restrict__ plus, int plus_parts, int dim) {
     const size_t at = (size_t)blockIdx.x * dim;
-    const float own = extra[(size_t)blockIdx.x * 2], gate = extra[(size_t)blockIdx.x * 2 + 1];
+    const float own = extra ? extra[(size_t)blockIdx.x * 2] : 1.f, gate = extra ? extra[(size_t)blockIdx.x * 2 + 1] : 1.f;
     for (int d = threadIdx.x; d < dim; d += blockDim.x) {
         float v = routed[at + d];
         for (int p = 1; p < parts; ++p) v += routed[p * part_stride + at + d];
@@ -455,6 +455,7 @@ experts_finish_kernel(float* __restrict__ out, const float* __restrict__ routed,
             for (int p = 1; p < shared_parts; ++p) sv += to_f32(shared[p * part_stride + at + d]);
             v += gate * sv;
         }
+        for (int p = 0; p < plus_parts; ++p) v += plus[p * part_stride + at + d];
         out[at + d] = v;
     }
 }
@@ -472,11 +473,11 @@ template <typename TX, typename TS>
 __global__ void __launch_bounds__(256)
 experts_finish_vec_kernel(float* __restrict__ out, const float* __restrict__ routed, int parts, size_t part_stride,
                           const TX* __restrict__ x, const TS* __restrict__ shared, int shared_parts,
-                          const float* __restrict__ extra, int dim) {
+                          const float* __restrict__ extra, const float* __restrict__ plus, int plus_parts, int dim) {
     const int d = (blockIdx.y * 256 + threadIdx.x) * 4;
     if (d >= dim) return;
     const size_t at = (size_t)blockIdx.x * dim + d;
-    const float own = extra[(size_t)blockIdx.x * 2], gate = extra[(size_t)blockIdx.x * 2 + 1];
+    const float own = extra ? extra[(size_t)blockIdx.x * 2] : 1.f, gate = extra ? extra[(size_t)blockIdx.x * 2 + 1] : 1.f;
     float4 v = fin_ld4(routed + at);
     for (int p = 1; p < parts; ++p) {
         const float4 w = fin_ld4(routed + p * part_stride + at);
@@ -494,12 +495,18 @@ experts_finish_vec_kernel(float* __restrict__ out, const float* __restrict__ rou
         }
         v = make_float4(v.x + gate * sv.x, v.y + gate * sv.y, v.z + gate * sv.z, v.w + gate * sv.w);
     }
+    for (int p = 0; p < plus_parts; ++p) {
+        const float4 w = fin_ld4(plus + p * part_stride + at);
+        v = make_float4(v.x + w.x, v.y + w.y, v.z + w.z, v.w + w.w);
+    }
     *reinterpret_cast<float4*>(out + at) = v;
 }
 
 extern "C" int ri_experts_finish(float* out, const float* routed, int parts, const void* x, int x_dtype, const void* shared,
-                                 int shared_dtype, int shared_parts, const float* extra, int tokens, int dim, void* stream) {
-    RI_REQUIRE(tokens > 0 && dim > 0 && parts >= 1 && shared_parts >= 1 && extra && routed, "experts_finish: %d tokens of %d", tokens, dim);
+                                 int shared_dtype, int shared_parts, const float* extra, const float* plus, int plus_parts,
+                                 int tokens, int dim, void* stream) {
+    RI_REQUIRE(plus_parts >= 0 && (plus_parts == 0 || plus), "experts_finish: %d more parts", plus_parts);
+    RI_REQUIRE(tokens > 0 && dim > 0 && parts >= 1 && shared_parts >= 1 && (extra || !x) && routed, "experts_finish: %d tokens of %d", tokens, dim);
     RI_REQUIRE((x_dtype == RI_F32 || x_dtype == RI_BF16) && (shared_dtype == RI_F32 || shared_dtype == RI_BF16),
                "experts_finish: dtypes %d and %d", x_dtype, shared_dtype);
     RI_REQUIRE(shared_parts == 1 || shared_dtype == RI_F32, "experts_finish: parts of a product are float32");
@@ -509,13 +516,41 @@ extern "C" int ri_experts_finish(float* out, const float* routed, int parts, con
 #define RI_GO(TX, TS)                                                                                                   \
     if (dim % 4 == 0 && vgrid.y <= 65535)                                                                               \
         experts_finish_vec_kernel<TX, TS><<<vgrid, 256, 0, s>>>(out, routed, parts, stride, (const TX*)x,                 \
-                                                                (const TS*)shared, shared_parts, extra, dim);            \
+                                                                (const TS*)shared, shared_parts, extra, plus, plus_parts, dim);            \
     else                                                                                                                \
         experts_finish_kernel<TX, TS><<<tokens, 256, 0, s>>>(out, routed, parts, stride, (const TX*)x,                    \
-                                                             (const TS*)shared, shared_parts, extra, dim)
+                                                             (const TS*)shared, shared_parts, extra, plus, plus_parts, dim)
     if (x_dtype == RI_F32) { if (shared_dtype == RI_F32) RI_GO(float, float); else RI_GO(float, bf16_t); }
     else                   { if (shared_dtype == RI_F32) RI_GO(bf16_t, float); else RI_GO(bf16_t, bf16_t); }
 #undef RI_GO
     RI_LAUNCH_CHECK("experts_finish");
+    return 0;
+}
+
+// Experts by token: no router, the token's row of a table of choices.  One wavefront a token.
+__global__ void __launch_bounds__(64)
+experts_by_table_kernel(int32_t* __restrict__ ids, float* __restrict__ weights, float* __restrict__ dense,
+                        const int32_t* __restrict__ table, const int32_t* __restrict__ token_ids, int vocab, int experts, int top) {
+    const int t = blockIdx.x, lane = threadIdx.x;
+    const int32_t* row = table + (size_t)min(max(token_ids[t], 0), vocab - 1) * top;      // (the engine refuses ids outside)
+    const float w = 1.f / (float)top;
+    for (int k = lane; k < top; k += RI_WAVE) {
+        ids[(size_t)t * top + k] = row[k];
+        weights[(size_t)t * top + k] = w;
+    }
+    if (!dense) return;
+    for (int e = lane; e < experts; e += RI_WAVE) {
+        float v = 0.f;
+        for (int k = 0; k < top; ++k) v = row[k] == e ? w : v;
+        dense[(size_t)t * experts + e] = v;
+    }
+}
+
+extern "C" int ri_experts_by_table(int32_t* ids, float* weights, float* dense, const int32_t* table, const int32_t* token_ids,
+                                   int tokens, int vocab, int experts, int top, void* stream) {
+    RI_REQUIRE(tokens > 0 && vocab > 0 && experts > 0 && top > 0 && top <= experts && ids && weights && table && token_ids,
+               "experts_by_table: %d tokens, %d of %d experts, %d rows", tokens, top, experts, vocab);
+    experts_by_table_kernel<<<tokens, 64, 0, (hipStream_t)stream>>>(ids, weights, dense, table, token_ids, vocab, experts, top);
+    RI_LAUNCH_CHECK("experts_by_table");
     return 0;
 }

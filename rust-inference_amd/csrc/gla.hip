@@ -286,21 +286,23 @@ extern "C" int ri_decay_scan(float* out, const void* proj, int act_dtype, int ro
                        slots, seqs, tokens, heads, dim, vdim, head_decay, stream);
 }
 
-// The scan's result per head through an RMS norm over vdim (one gain for all heads) and times silu(gate):
-// one wavefront per (token, head).
+// The scan's result per head through an RMS norm over vdim (one gain for all heads) and times silu(gate), or, with
+// `sigmoid`, times sigmoid(gate): one wavefront per (token, head).  The gate may have a format of its own (TG).
 #define GLA_NORM_PER_LANE 8      // vdim <= 64 * 8
 
-template <typename TA>
-__global__ void gla_norm_gate_kernel(TA* __restrict__ out, const float* __restrict__ o, const TA* __restrict__ proj,
+__device__ __forceinline__ float gate_open(float z, int sigmoid) { return (sigmoid ? 1.0f : z) / (1.0f + expf(-z)); }
+
+template <typename TA, typename TG>
+__global__ void gla_norm_gate_kernel(TA* __restrict__ out, const float* __restrict__ o, const TG* __restrict__ proj,
                                      int row, int g_off, const float* __restrict__ gain, float eps, long items,
-                                     int heads, int vdim) {
+                                     int heads, int vdim, int sigmoid) {
     const int lane = threadIdx.x & (RI_WAVE - 1);
     const long item = (long)blockIdx.x * (blockDim.x / RI_WAVE) + threadIdx.x / RI_WAVE;
     if (item >= items) return;
     const long t = item / heads;
     const int h = (int)(item % heads);
     const float* x = o + (size_t)item * vdim;
-    const TA* g = proj + (size_t)t * row + g_off + (size_t)h * vdim;
+    const TG* g = proj + (size_t)t * row + g_off + (size_t)h * vdim;
     float v[GLA_NORM_PER_LANE];
     float ss = 0.f;
 #pragma unroll
@@ -314,17 +316,16 @@ __global__ void gla_norm_gate_kernel(TA* __restrict__ out, const float* __restri
     for (int j = 0; j < GLA_NORM_PER_LANE; ++j) {
         const int i = lane + j * RI_WAVE;
         if (i >= vdim) continue;
-        const float gate = to_f32(g[i]);
-        from_f32(out + (size_t)item * vdim + i, v[j] * inv * gain[i] * (gate / (1.0f + expf(-gate))));
+        from_f32(out + (size_t)item * vdim + i, v[j] * inv * gain[i] * gate_open(to_f32(g[i]), sigmoid));
     }
 }
 
 // The same 16 bytes a lane, for value heads of 8 lanes' worth of eight elements or a power-of-two fraction (vdim 8,
 // 16, ... 512): vdim / 8 lanes make a head, a wavefront works on 512 / vdim heads at once.
-template <typename TA>
+template <typename TA, typename TG>
 __global__ void __launch_bounds__(256)
-gla_norm_gate_vec_kernel(TA* __restrict__ out, const float* __restrict__ o, const TA* __restrict__ proj, int row, int g_off,
-                         const float* __restrict__ gain, float eps, long items, int heads, int vdim) {
+gla_norm_gate_vec_kernel(TA* __restrict__ out, const float* __restrict__ o, const TG* __restrict__ proj, int row, int g_off,
+                         const float* __restrict__ gain, float eps, long items, int heads, int vdim, int sigmoid) {
     const int lanes_per_head = vdim / 8;
     const int heads_at_once = RI_WAVE / lanes_per_head;
     const int lane = threadIdx.x & (RI_WAVE - 1);
@@ -338,8 +339,8 @@ gla_norm_gate_vec_kernel(TA* __restrict__ out, const float* __restrict__ o, cons
     const float4 a = *reinterpret_cast<const float4*>(x), b = *reinterpret_cast<const float4*>(x + 4);
     float v[8] = {a.x, a.y, a.z, a.w, b.x, b.y, b.z, b.w};
     float gate[8];
-    const TA* g = proj + (size_t)t * row + g_off + (size_t)h * vdim + piece * 8;
-    if (sizeof(TA) == 2) {
+    const TG* g = proj + (size_t)t * row + g_off + (size_t)h * vdim + piece * 8;
+    if (sizeof(TG) == 2) {
         const uint4 w = *reinterpret_cast<const uint4*>(g);
         const uint32_t ww[4] = {w.x, w.y, w.z, w.w};
 #pragma unroll
@@ -360,7 +361,7 @@ gla_norm_gate_vec_kernel(TA* __restrict__ out, const float* __restrict__ o, cons
     const float gn[8] = {ga.x, ga.y, ga.z, ga.w, gb.x, gb.y, gb.z, gb.w};
     float r[8];
 #pragma unroll
-    for (int e = 0; e < 8; ++e) r[e] = v[e] * inv * gn[e] * (gate[e] / (1.0f + expf(-gate[e])));
+    for (int e = 0; e < 8; ++e) r[e] = v[e] * inv * gn[e] * gate_open(gate[e], sigmoid);
     TA* dst = out + (size_t)item * vdim + piece * 8;
     if (sizeof(TA) == 2) {
         *reinterpret_cast<uint4*>(dst) = make_uint4(pack_bf16x2(r[0], r[1]), pack_bf16x2(r[2], r[3]), pack_bf16x2(r[4], r[5]),
@@ -371,36 +372,41 @@ gla_norm_gate_vec_kernel(TA* __restrict__ out, const float* __restrict__ o, cons
     }
 }
 
+template <typename TA, typename TG>
+static void launch_norm_gate(TA* out, const float* o, const TG* gate, int row, int g_off, const float* gain, float eps, int tokens,
+                             int heads, int vdim, int sigmoid, hipStream_t s) {
+    const long items = (long)tokens * heads, blocks = (items + 3) / 4;
+    const int lph = vdim / 8;
+    if (vdim % 8 == 0 && lph <= 64 && (lph & (lph - 1)) == 0 && row % 8 == 0 && g_off % 8 == 0 && (uintptr_t)gate % 16 == 0) {
+        const long waves = (items + (64 / lph) - 1) / (64 / lph), vblocks = (waves + 3) / 4;
+        gla_norm_gate_vec_kernel<TA, TG><<<(unsigned)vblocks, 256, 0, s>>>(out, o, gate, row, g_off, gain, eps, items, heads, vdim, sigmoid);
+    } else {
+        gla_norm_gate_kernel<TA, TG><<<(unsigned)blocks, 256, 0, s>>>(out, o, gate, row, g_off, gain, eps, items, heads, vdim, sigmoid);
+    }
+}
+
+extern "C" int ri_head_norm_gate(void* out, int act_dtype, const float* o, const void* gate, int gate_dtype, int row, int g_off,
+                                 const float* gain, float eps, int tokens, int heads, int vdim, int sigmoid, void* stream) {
+    RI_REQUIRE(tokens > 0 && heads > 0 && vdim > 0 && vdim <= RI_WAVE * GLA_NORM_PER_LANE,
+               "head_norm_gate: %d tokens, %d heads of %d", tokens, heads, vdim);
+    RI_REQUIRE(g_off >= 0 && g_off + heads * vdim <= row, "head_norm_gate: the gate at %d does not fit rows of %d", g_off, row);
+    RI_REQUIRE((act_dtype == RI_F32 || act_dtype == RI_BF16) && (gate_dtype == RI_F32 || gate_dtype == act_dtype),
+               "head_norm_gate: dtypes %d and %d", act_dtype, gate_dtype);
+    RI_REQUIRE(((long)tokens * heads + 3) / 4 <= 2147483647L, "head_norm_gate: %ld heads exceed one launch", (long)tokens * heads);
+    hipStream_t s = (hipStream_t)stream;
+    if (act_dtype == RI_F32)
+        launch_norm_gate<float, float>((float*)out, o, (const float*)gate, row, g_off, gain, eps, tokens, heads, vdim, sigmoid, s);
+    else if (gate_dtype == RI_F32)
+        launch_norm_gate<bf16_t, float>((bf16_t*)out, o, (const float*)gate, row, g_off, gain, eps, tokens, heads, vdim, sigmoid, s);
+    else
+        launch_norm_gate<bf16_t, bf16_t>((bf16_t*)out, o, (const bf16_t*)gate, row, g_off, gain, eps, tokens, heads, vdim, sigmoid, s);
+    RI_LAUNCH_CHECK("head_norm_gate");
+    return 0;
+}
+
 extern "C" int ri_gla_norm_gate(void* out, const float* o, const void* proj, int act_dtype, int row, int g_off,
                                 const float* gain, float eps, int tokens, int heads, int vdim, void* stream) {
-    RI_REQUIRE(tokens > 0 && heads > 0 && vdim > 0 && vdim <= RI_WAVE * GLA_NORM_PER_LANE,
-               "gla_norm_gate: %d tokens, %d heads of %d", tokens, heads, vdim);
-    RI_REQUIRE(g_off >= 0 && g_off + heads * vdim <= row, "gla_norm_gate: the gate at %d does not fit rows of %d", g_off, row);
-    RI_REQUIRE(act_dtype == RI_F32 || act_dtype == RI_BF16, "gla_norm_gate: dtype %d", act_dtype);
-    const long items = (long)tokens * heads;
-    const long blocks = (items + 3) / 4;
-    RI_REQUIRE(blocks <= 2147483647L, "gla_norm_gate: %ld heads exceed one launch", items);
-    hipStream_t s = (hipStream_t)stream;
-    const int lph = vdim / 8;
-    if (vdim % 8 == 0 && lph <= 64 && (lph & (lph - 1)) == 0 && row % 8 == 0 && g_off % 8 == 0) {
-        const long waves = (items + (64 / lph) - 1) / (64 / lph), vblocks = (waves + 3) / 4;
-        if (act_dtype == RI_F32)
-            gla_norm_gate_vec_kernel<float><<<(unsigned)vblocks, 256, 0, s>>>((float*)out, o, (const float*)proj, row, g_off,
-                                                                              gain, eps, items, heads, vdim);
-        else
-            gla_norm_gate_vec_kernel<bf16_t><<<(unsigned)vblocks, 256, 0, s>>>((bf16_t*)out, o, (const bf16_t*)proj, row,
-                                                                               g_off, gain, eps, items, heads, vdim);
-        RI_LAUNCH_CHECK("gla_norm_gate");
-        return 0;
-    }
-    if (act_dtype == RI_F32)
-        gla_norm_gate_kernel<float><<<(unsigned)blocks, 256, 0, s>>>((float*)out, o, (const float*)proj, row, g_off, gain, eps,
-                                                                     items, heads, vdim);
-    else
-        gla_norm_gate_kernel<bf16_t><<<(unsigned)blocks, 256, 0, s>>>((bf16_t*)out, o, (const bf16_t*)proj, row, g_off, gain,
-                                                                      eps, items, heads, vdim);
-    RI_LAUNCH_CHECK("gla_norm_gate");
-    return 0;
+    return ri_head_norm_gate(out, act_dtype, o, proj, act_dtype, row, g_off, gain, eps, tokens, heads, vdim, 0, stream);
 }
 
 // ------------------------------------------------------------------ one new token a sequence

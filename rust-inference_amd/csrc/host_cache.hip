@@ -7,7 +7,7 @@
 // The reference keeps one page table per layer, hands out page 0 first, advances every sequence by the
 // same count and can only reset the whole cache (src/kvcache.rs:51, :106-135, :185-196).  Here a pool
 // serves all layers of one key/value geometry, sequences advance by their own counts, a slot gives its
-// pages back when its sequence ends, and a pool with a window gives pages back as soon as no later query
+// pages back when its sequence ends, and a pool with a window or with chunks gives pages back as soon as no later query
 // can see them.
 #include <stdint.h>
 #include <string.h>
@@ -25,6 +25,7 @@ constexpr int32_t UNMAPPED = -1;
 struct PagePool {
     int num_pages, page_size, num_slots, max_pages_per_slot, window;   // window 0: every key stays
     int keep_first = 0;                                                // the first tokens of a sequence stay behind a window too
+    int chunk = 0;                                                     // > 0: a query sees its own run of this many positions alone
     std::vector<int32_t> free_list;                                    // taken from the back: page 0 first
     std::vector<int32_t> owner;                                        // page -> slot, to catch double frees
     std::vector<int32_t> tables;                                       // [num_slots][max_pages_per_slot]
@@ -74,8 +75,8 @@ struct PagePool {
     }
     // Gives back the pages that no query at a position >= length can see.
     int trim_behind_window(int slot, long length) {
-        if (window <= 0) return 0;
-        const long first_visible = std::max<long>(0, length - window + 1);   // of the next query, at `length`
+        if (window <= 0 && chunk <= 0) return 0;
+        const long first_visible = chunk > 0 ? length - length % chunk : std::max<long>(0, length - window + 1);   // of the next query, at `length`
         const long kept_pages = ((long)keep_first + page_size - 1) / page_size;    // they hold the positions 0 .. keep_first - 1
         for (long p = kept_pages; p < first_visible / page_size && p < max_pages_per_slot; ++p)
             if (give_back(slot, (int)p)) return 1;
@@ -155,6 +156,12 @@ extern "C" int ri_pool_reserve(void* pool, int slot, long before, long n) { retu
 extern "C" int ri_pool_keep_first(void* pool, int tokens) {
     RI_REQUIRE(pool && tokens >= 0, "a pool keeps %d first tokens", tokens);
     ((PagePool*)pool)->keep_first = tokens;
+    return 0;
+}
+extern "C" int ri_pool_chunk(void* pool, int tokens) {
+    RI_REQUIRE(pool && tokens >= 0 && (tokens == 0 || (((PagePool*)pool)->window == 0 && ((PagePool*)pool)->keep_first == 0)),
+               "chunks of %d tokens in a pool with a window", tokens);
+    ((PagePool*)pool)->chunk = tokens;
     return 0;
 }
 extern "C" int ri_pool_trim(void* pool, int slot, long length) { return ((PagePool*)pool)->trim_behind_window(slot, length); }

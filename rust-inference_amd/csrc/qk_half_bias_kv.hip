@@ -2,11 +2,12 @@
 // first part of a head, in one pass over the projection's rows (q heads at q_off, k heads at k_off, v heads at v_off
 // of rows of row_len elements; the biases float32, one per column of q, k and v):
 //
-//   q, k: x += bias; the elements (i, i + half), i < half, turn by pos * inv_freq[i], cosine and sine times `amplitude`;
+//   q, k: x += bias; with gains, x <- x / sqrt(mean(x^2) + eps) * gain over a head (one gain of dim for all q heads, one for
+//         all k heads); the elements (i, i + half), i < half, turn by pos * inv_freq[i], cosine and sine times `amplitude`;
 //         what lies behind 2 half passes; q in place, k into k_pages [pages][kv_heads][page_size][dim];
 //   v:    v + bias into v_pages [pages][kv_heads][vdim][page_size] (transposed inside a page).
 //
-// Bias, angle, sine and cosine are float32; an element is rounded once.  kv_heads 0: a layer that reads another one's
+// Bias, norm, angle, sine and cosine are float32; an element is rounded once.  kv_heads 0: a layer that reads another one's
 // keys and values, queries alone.
 #include "api.h"
 #include "common.h"
@@ -17,8 +18,9 @@ template <typename T>
 __global__ void __launch_bounds__(256)
 qk_half_bias_kv_write_kernel(T* __restrict__ proj, size_t row_len, int q_off, int k_off, int v_off,
                              const float* __restrict__ q_bias, const float* __restrict__ k_bias,
-                             const float* __restrict__ v_bias, const float* __restrict__ inv_freq, int half, float amplitude,
-                             const int32_t* __restrict__ tok_pos, const int32_t* __restrict__ tok_seq,
+                             const float* __restrict__ v_bias, const float* __restrict__ q_gain,
+                             const float* __restrict__ k_gain, float eps, const float* __restrict__ inv_freq, int half,
+                             float amplitude, const int32_t* __restrict__ tok_pos, const int32_t* __restrict__ tok_seq,
                              const int32_t* __restrict__ page_table, int table_width, T* __restrict__ k_pages,
                              T* __restrict__ v_pages, int tokens, int heads, int kv_heads, int dim, int vdim, int page_size,
                              int write_values) {
@@ -44,11 +46,25 @@ qk_half_bias_kv_write_kernel(T* __restrict__ proj, size_t row_len, int q_off, in
     const float* bias = is_q ? q_bias : k_bias;
     if (bias) bias += (size_t)(is_q ? hh : kvh) * dim;
     T* to = is_q ? x : k_pages + (page_head * page_size + pos % page_size) * dim;
+    const float* gain = is_q ? q_gain : k_gain;
+    float inv = 1.f;
+    if (gain) {
+        float ss = 0.f;
+        for (int i = lane; i < dim; i += RI_WAVE) {
+            const float v = to_f32(x[i]) + (bias ? bias[i] : 0.f);
+            ss += v * v;
+        }
+        inv = 1.f / sqrtf(wave_sum(ss) / (float)dim + eps);
+    }
     for (int i = lane; i < half; i += RI_WAVE) {
         float u = to_f32(x[i]), v = to_f32(x[i + half]);
         if (bias) {
             u += bias[i];
             v += bias[i + half];
+        }
+        if (gain) {
+            u = u * inv * gain[i];
+            v = v * inv * gain[i + half];
         }
         float sn, cs;
         sincosf((float)pos * inv_freq[i], &sn, &cs);
@@ -57,21 +73,48 @@ qk_half_bias_kv_write_kernel(T* __restrict__ proj, size_t row_len, int q_off, in
         from_f32(to + i, u * cs - v * sn);
         from_f32(to + i + half, v * cs + u * sn);
     }
-    for (int i = 2 * half + lane; i < dim; i += RI_WAVE) from_f32(to + i, to_f32(x[i]) + (bias ? bias[i] : 0.f));
+    for (int i = 2 * half + lane; i < dim; i += RI_WAVE) {
+        const float v = to_f32(x[i]) + (bias ? bias[i] : 0.f);
+        from_f32(to + i, gain ? v * inv * gain[i] : v);
+    }
 }
 
 // A prompt whose halves and head sizes 16-byte pieces divide: a workgroup a token.  The token's sines and cosines are
-// made once, in LDS; a thread then takes a piece of eight from each half of a head (or one of the part that passes), every
+// made once, in LDS, as are, with gains, the heads' factors (a wavefront a head); a thread then takes a piece of eight from each half of a head (or one of the part that passes), every
 // load and store 16 bytes (32 for float32).  The values go a page at a time (values_to_pages_kernel).
 template <typename T>
 __global__ void __launch_bounds__(256)
 qk_half_bias_k_write_vec_kernel(T* __restrict__ proj, size_t row_len, int q_off, int k_off, const float* __restrict__ q_bias,
-                                const float* __restrict__ k_bias, const float* __restrict__ inv_freq, int half, float amplitude,
-                                const int32_t* __restrict__ tok_pos, const int32_t* __restrict__ tok_seq,
+                                const float* __restrict__ k_bias, const float* __restrict__ q_gain,
+                                const float* __restrict__ k_gain, float eps, const float* __restrict__ inv_freq, int half,
+                                float amplitude, const int32_t* __restrict__ tok_pos, const int32_t* __restrict__ tok_seq,
                                 const int32_t* __restrict__ page_table, int table_width, T* __restrict__ k_pages, int heads,
                                 int kv_heads, int dim, int page_size) {
-    extern __shared__ __align__(16) float turn[];          // [half] cosines, [half] sines
+    extern __shared__ __align__(16) float turn[];          // [half] cosines, [half] sines, [heads + kv_heads] factors
     const int t = blockIdx.x, pos = tok_pos[t];
+    T* row = proj + (size_t)t * row_len;
+    if (q_gain) {
+        for (int hh = threadIdx.x / RI_WAVE; hh < heads + kv_heads; hh += blockDim.x / RI_WAVE) {
+            const bool is_q = hh < heads;
+            const T* x = row + (is_q ? q_off + (size_t)hh * dim : k_off + (size_t)(hh - heads) * dim);
+            const float* bias = is_q ? q_bias : k_bias;
+            if (bias) bias += (size_t)(is_q ? hh : hh - heads) * dim;
+            float ss = 0.f;
+            for (int i = (threadIdx.x & (RI_WAVE - 1)) * 8; i < dim; i += RI_WAVE * 8) {
+                float u[8], b[8];
+                Eight<T>::load(x + i, u);
+                if (bias) {
+                    Eight<float>::load(bias + i, b);
+#pragma unroll
+                    for (int k = 0; k < 8; ++k) u[k] += b[k];
+                }
+#pragma unroll
+                for (int k = 0; k < 8; ++k) ss += u[k] * u[k];
+            }
+            ss = wave_sum(ss);
+            if ((threadIdx.x & (RI_WAVE - 1)) == 0) turn[2 * half + hh] = 1.f / sqrtf(ss / (float)dim + eps);
+        }
+    }
     for (int i = threadIdx.x; i < half; i += blockDim.x) {
         float sn, cs;
         sincosf((float)pos * inv_freq[i], &sn, &cs);
@@ -80,7 +123,6 @@ qk_half_bias_k_write_vec_kernel(T* __restrict__ proj, size_t row_len, int q_off,
     }
     __syncthreads();
     const long page = kv_heads > 0 ? page_table[(size_t)tok_seq[t] * table_width + pos / page_size] : 0;
-    T* row = proj + (size_t)t * row_len;
     const int turning = half / 8, pieces = turning + (dim - 2 * half) / 8;      // of a head
     for (int e = threadIdx.x; e < (heads + kv_heads) * pieces; e += blockDim.x) {
         const int hh = e / pieces, piece = e - hh * pieces;
@@ -97,6 +139,13 @@ qk_half_bias_k_write_vec_kernel(T* __restrict__ proj, size_t row_len, int q_off,
 #pragma unroll
             for (int k = 0; k < 8; ++k) u[k] += b[k];
         }
+        const float* gain = is_q ? q_gain : k_gain;
+        const float inv = gain ? turn[2 * half + hh] : 1.f;
+        if (gain) {
+            Eight<float>::load(gain + i, b);
+#pragma unroll
+            for (int k = 0; k < 8; ++k) u[k] = u[k] * inv * b[k];
+        }
         if (piece < turning) {
             float v[8];
             Eight<T>::load(x + i + half, v);
@@ -104,6 +153,11 @@ qk_half_bias_k_write_vec_kernel(T* __restrict__ proj, size_t row_len, int q_off,
                 Eight<float>::load(bias + i + half, b);
 #pragma unroll
                 for (int k = 0; k < 8; ++k) v[k] += b[k];
+            }
+            if (gain) {
+                Eight<float>::load(gain + i + half, b);
+#pragma unroll
+                for (int k = 0; k < 8; ++k) v[k] = v[k] * inv * b[k];
             }
             float cs[8], sn[8];
             Eight<float>::load(turn + i, cs);
@@ -122,8 +176,8 @@ qk_half_bias_k_write_vec_kernel(T* __restrict__ proj, size_t row_len, int q_off,
 
 template <typename T>
 static void launch_qk_half(T* proj, size_t row_len, int q_off, int k_off, int v_off, const float* q_bias, const float* k_bias,
-                           const float* v_bias, const float* inv_freq, int half, float amplitude, const int32_t* tok_pos,
-                           const int32_t* tok_seq, const int32_t* cu_seqlens, int seqs, int max_new,
+                           const float* v_bias, const float* q_gain, const float* k_gain, float eps, const float* inv_freq, int half,
+                           float amplitude, const int32_t* tok_pos, const int32_t* tok_seq, const int32_t* cu_seqlens, int seqs, int max_new,
                            const int32_t* page_table, int table_width, T* k_pages, T* v_pages, int tokens, int heads,
                            int kv_heads, int dim, int vdim, int page_size, hipStream_t s) {
     const bool prompt = cu_seqlens && max_new > 1;
@@ -133,15 +187,16 @@ static void launch_qk_half(T* proj, size_t row_len, int q_off, int k_off, int v_
     const int unit = 16 / (int)sizeof(T);
     const bool pieces = prompt && (paged_values || kv_heads == 0) && half % 8 == 0 && dim % 8 == 0 &&
                         (row_len | q_off | k_off) % unit == 0 && (uintptr_t)proj % 16 == 0 && (uintptr_t)k_pages % 16 == 0 &&
-                        ((uintptr_t)q_bias | (uintptr_t)k_bias) % 16 == 0;
+                        ((uintptr_t)q_bias | (uintptr_t)k_bias | (uintptr_t)q_gain | (uintptr_t)k_gain) % 16 == 0 &&
+                        (2L * half + heads + kv_heads + 4) * (long)sizeof(float) <= 65536;
     if (pieces)
-        qk_half_bias_k_write_vec_kernel<T><<<tokens, 256, (2 * half + 4) * sizeof(float), s>>>(
-            proj, row_len, q_off, k_off, q_bias, k_bias, inv_freq, half, amplitude, tok_pos, tok_seq, page_table, table_width,
+        qk_half_bias_k_write_vec_kernel<T><<<tokens, 256, (2 * half + heads + kv_heads + 4) * sizeof(float), s>>>(
+            proj, row_len, q_off, k_off, q_bias, k_bias, q_gain, k_gain, eps, inv_freq, half, amplitude, tok_pos, tok_seq, page_table, table_width,
             k_pages, heads, kv_heads, dim, page_size);
     else {
         const long items = (long)tokens * (heads + (paged_values ? 1 : 2) * kv_heads);
         qk_half_bias_kv_write_kernel<T><<<(unsigned)((items + 3) / 4), 256, 0, s>>>(
-            proj, row_len, q_off, k_off, v_off, q_bias, k_bias, v_bias, inv_freq, half, amplitude, tok_pos, tok_seq, page_table,
+            proj, row_len, q_off, k_off, v_off, q_bias, k_bias, v_bias, q_gain, k_gain, eps, inv_freq, half, amplitude, tok_pos, tok_seq, page_table,
             table_width, k_pages, v_pages, tokens, heads, kv_heads, dim, vdim, page_size, !paged_values);
     }
     if (paged_values) {
@@ -152,8 +207,8 @@ static void launch_qk_half(T* proj, size_t row_len, int q_off, int k_off, int v_
 }
 
 extern "C" int ri_qk_half_bias_kv_write(void* proj, int act_dtype, long row_len, int q_off, int k_off, int v_off,
-                                        const float* q_bias, const float* k_bias, const float* v_bias, const float* inv_freq,
-                                        int half, float amplitude, const int32_t* tok_pos, const int32_t* tok_seq,
+                                        const float* q_bias, const float* k_bias, const float* v_bias, const float* q_gain,
+                                        const float* k_gain, float eps, const float* inv_freq, int half, float amplitude, const int32_t* tok_pos, const int32_t* tok_seq,
                                         const int32_t* cu_seqlens, int seqs, int max_new, const int32_t* page_table,
                                         int table_width, void* k_pages, void* v_pages, int cache_dtype, int tokens, int heads,
                                         int kv_heads, int dim, int vdim, int page_size, void* stream) {
@@ -170,11 +225,12 @@ extern "C" int ri_qk_half_bias_kv_write(void* proj, int act_dtype, long row_len,
     RI_REQUIRE(kv_heads == 0 || (page_size > 0 && table_width > 0 && k_pages && v_pages), "qk_half_bias_kv_write: page geometry");
     RI_REQUIRE(((long)tokens * (heads + 2 * kv_heads) + 3) / 4 <= 2147483647L, "qk_half_bias_kv_write: %ld heads exceed one launch",
                (long)tokens * (heads + 2 * kv_heads));
+    RI_REQUIRE(kv_heads == 0 || (q_gain == nullptr) == (k_gain == nullptr), "qk_half_bias_kv_write: gains of q and k come together");
     RI_REQUIRE(!cu_seqlens || (seqs > 0 && max_new > 0), "qk_half_bias_kv_write: seqs %d, max_new %d", seqs, max_new);
     hipStream_t s = (hipStream_t)stream;
 #define RI_GO(T)                                                                                                          \
     launch_qk_half<T>((T*)proj, (size_t)row_len, q_off, kv_heads ? k_off : 0, kv_heads ? v_off : 0, q_bias, k_bias, v_bias, \
-                      inv_freq, half, amplitude, tok_pos, tok_seq, cu_seqlens, seqs, max_new, page_table, table_width,      \
+                      q_gain, k_gain, eps, inv_freq, half, amplitude, tok_pos, tok_seq, cu_seqlens, seqs, max_new, page_table, table_width,      \
                       (T*)k_pages, (T*)v_pages, tokens, heads, kv_heads, dim, vdim, page_size, s)
     if (act_dtype == RI_F32) RI_GO(float); else RI_GO(bf16_t);
 #undef RI_GO

@@ -67,7 +67,7 @@ _SIGNATURES = {
                                  c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_void_p, c_int,
                                  c_void_p],
     "ri_attention_decode_kept_bf16": [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
-                                      c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_void_p, c_int,
+                                      c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_void_p, c_int,
                                       c_int, c_void_p, c_void_p],
     "ri_attention_decode_fused_bf16": [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_float,
                                        c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int,
@@ -101,10 +101,10 @@ _SIGNATURES = {
     "ri_finish_norm": [c_void_p, c_void_p, c_void_p, c_int, c_float, c_int, c_int, c_int, c_void_p],
     "ri_argmax": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p],
     "ri_attention_prefill_kept_bf16": [c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int,
-                                       c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_void_p, c_int,
+                                       c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_void_p, c_int,
                                        c_void_p, c_void_p],
     "ri_attention_kept": [c_void_p, c_void_p, c_int, c_int, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int,
-                          c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_void_p, c_int, c_void_p,
+                          c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_void_p, c_int, c_void_p,
                           c_void_p],
     "ri_qk_pairs_norm_kv_write": [c_void_p, c_int, ctypes.c_long, c_int, c_int, c_int, c_void_p, c_int, c_void_p, c_void_p,
                                   c_int, c_float, c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p, c_int, c_void_p,
@@ -120,20 +120,33 @@ _SIGNATURES = {
                            c_int, c_int, c_void_p],
     "ri_attention_padded_fits": [c_int, c_int, c_int, c_int],
     "ri_attention_prefill_padded_bf16": [c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int,
-                                         c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_void_p, c_int,
+                                         c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_void_p, c_int,
                                          c_void_p, c_void_p],
     "ri_attention_decode_padded_bf16": [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int,
-                                        c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_void_p, c_int,
+                                        c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_void_p, c_int,
                                         c_int, c_void_p, c_void_p],
     "ri_branch_norm_add_norm": [c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_void_p, c_void_p, c_float, c_int, c_void_p,
                                 c_void_p, c_float, c_int, c_int, c_int, c_void_p],
     "ri_embed_bigram": [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
                         ctypes.c_long, ctypes.c_long, ctypes.c_long, c_int, c_int, c_void_p],
-    "ri_qk_half_bias_kv_write": [c_void_p, c_int, ctypes.c_long, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int,
-                                 c_float, c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p, c_int, c_void_p, c_void_p, c_int,
+    "ri_qk_half_bias_kv_write": [c_void_p, c_int, ctypes.c_long, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_float,
+                                 c_void_p, c_int, c_float, c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p, c_int, c_void_p, c_void_p, c_int,
                                  c_int, c_int, c_int, c_int, c_int, c_int, c_void_p],
     "ri_experts_few_tokens_plain": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int,
                                     c_int, c_int, c_int, c_void_p],
+    "ri_head_norm_gate": [c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p, c_float, c_int, c_int, c_int, c_int,
+                          c_void_p],
+    "ri_normed_sum": [c_void_p, c_int, c_void_p, c_int, c_int, c_void_p, c_float, c_void_p, c_int, c_int, c_void_p, c_float, c_float,
+                      c_int, c_int, c_void_p],
+    "ri_experts_by_table": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_void_p],
+    "ri_delta_prepare_channels": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p, c_int, c_void_p, c_void_p, c_int,
+                                  c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int,
+                                  c_int, c_int, c_void_p],
+    "ri_delta_scan_channels": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int,
+                               c_int, c_void_p],
+    "ri_delta_step_channels": [c_void_p, c_void_p, c_int, c_int, c_int, c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_void_p,
+                               c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_float, c_int, c_int, c_int,
+                               c_int, c_int, c_void_p],
     "ri_gate_rows": [c_void_p, c_int, c_int, c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_float, c_int, c_int, c_int,
                      c_void_p],
     "ri_row_norm_gate": [c_void_p, c_int, c_int, c_void_p, c_void_p, c_float, c_void_p, c_int, c_int, c_int, c_float, c_int,
@@ -141,7 +154,7 @@ _SIGNATURES = {
     "ri_experts_route_general": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_int,
                                  c_int, c_int, c_int, c_int, c_int, c_int, c_void_p],
     "ri_experts_activate_strided": [c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_int, c_float, c_void_p],
-    "ri_experts_finish": [c_void_p, c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_int, c_void_p, c_int, c_int,
+    "ri_experts_finish": [c_void_p, c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_int, c_void_p, c_void_p, c_int, c_int, c_int,
                           c_void_p],
     "ri_scaled_sum_norm": [c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_void_p, c_float, c_void_p, c_void_p, c_float,
                            c_int, c_int, c_int, c_void_p],
@@ -481,11 +494,11 @@ def qk_norm_rope_kv_write(qkv, q_gain, k_gain, eps, inv_freq, tok_pos, tok_seq, 
 
 def attention(qkv, k_pages, v_pages, tok_pos, tok_seq, page_table, heads: int, kv_heads: int, head_dim: int,
               window: int | None, scale: float, softcap: float | None = None, slopes: torch.Tensor | None = None,
-              keep_first: int = 0, sinks: torch.Tensor | None = None, q_off: int = 0) -> torch.Tensor:
+              keep_first: int = 0, sinks: torch.Tensor | None = None, q_off: int = 0, chunk: int | None = None) -> torch.Tensor:
     """Attention of every new token over its sequence's pages; q is the first ``H dh`` columns of ``qkv``.
     With a window, ``keep_first`` first tokens of the sequence stay visible behind it; ``sinks`` (float32 ``[heads]``)
     adds ``exp(sinks[h])`` to the denominator of head ``h``'s softmax.  ``q_off``: the queries' first column in ``qkv``'s rows
-    where it is not 0.
+    where it is not 0.  ``chunk``: a query sees the keys of its own run of that many positions alone (no window beside it).
     The size of a value head is read from ``v_pages [pages, kv_heads, v_dim, page]``; with ``softcap`` a score
     ``s`` becomes ``softcap * tanh(s / softcap)`` before the softmax; with ``slopes`` (float32 ``[heads]``) the score of
     head ``h`` at position ``p`` for the key at ``j`` then loses ``slopes[h] * (p - j)``."""
@@ -500,7 +513,7 @@ def attention(qkv, k_pages, v_pages, tok_pos, tok_seq, page_table, heads: int, k
           _dev(v_pages, "v_pages"), code(k_pages.dtype), _dev(tok_pos, "tok_pos", torch.int32, (tokens,)),
           _dev(tok_seq, "tok_seq", torch.int32, (tokens,)), _dev(page_table, "page_table", torch.int32),
           page_table.shape[1], tokens, heads, kv_heads, head_dim, v_dim, k_pages.shape[2], int(window or 0),
-          float(scale), float(softcap or 0.0), _opt(slopes, "slopes", torch.float32, (heads,)), int(keep_first or 0),
+          int(chunk or 0), float(scale), float(softcap or 0.0), _opt(slopes, "slopes", torch.float32, (heads,)), int(keep_first or 0),
           _opt(sinks, "sinks", torch.float32, (heads,)), _stream())
     return out
 
@@ -529,9 +542,10 @@ def qk_pairs_norm_kv_write(proj, q_off: int, k_off: int, v_off: int, inv_freq, q
 
 def qk_half_bias_kv_write(proj, q_off: int, k_off: int, v_off: int, bias, inv_freq, amplitude: float, tok_pos, tok_seq, page_table,
                           k_pages, v_pages, heads: int, kv_heads: int, dim: int, vdim: int, cu_seqlens=None,
-                          max_new: int = 0) -> None:
+                          max_new: int = 0, q_gain=None, k_gain=None, eps: float = 0.0) -> None:
     """In place on the projection rows ``proj [T, row]`` (q heads at column ``q_off``, k heads at ``k_off``, v heads at ``v_off``):
-    the biases (float32, q's then k's then v's, or None) are added, the elements ``(i, i + r)`` of every q and k head, ``r =
+    the biases (float32, q's then k's then v's, or None) are added, with ``q_gain`` and ``k_gain`` (float32 ``[dim]``) every q and k
+    head goes through an RMS norm, the elements ``(i, i + r)`` of every q and k head, ``r =
     len(inv_freq)``, turn by ``pos * inv_freq[i]`` with cosine and sine times ``amplitude``; q stays in ``proj``, k and v go to their
     pages.  ``kv_heads`` 0: queries alone (their layer reads another one's keys and values)."""
     tokens, row = proj.shape
@@ -548,7 +562,8 @@ def qk_half_bias_kv_write(proj, q_off: int, k_off: int, v_off: int, bias, inv_fr
         kv = (_dev(k_pages, "k_pages", proj.dtype, (pages, kv_heads, page_size, dim)),
               _dev(v_pages, "v_pages", proj.dtype, (pages, kv_heads, vdim, page_size)), k_pages.dtype)
     _call("ri_qk_half_bias_kv_write", _dev(proj, "proj"), code(proj.dtype), row, int(q_off), int(k_off), int(v_off), q_bias, k_bias,
-          v_bias, _opt(inv_freq, "inv_freq", torch.float32), half, float(amplitude), _dev(tok_pos, "tok_pos", torch.int32, (tokens,)),
+          v_bias, _opt(q_gain, "q_gain", torch.float32, (dim,)), _opt(k_gain, "k_gain", torch.float32, (dim,)), float(eps),
+          _opt(inv_freq, "inv_freq", torch.float32), half, float(amplitude), _dev(tok_pos, "tok_pos", torch.int32, (tokens,)),
           _dev(tok_seq, "tok_seq", torch.int32, (tokens,)), _opt(cu_seqlens, "cu_seqlens", torch.int32), seqs, int(max_new),
           _dev(page_table, "page_table", torch.int32), page_table.shape[1], kv[0], kv[1], code(kv[2]), tokens, heads, kv_heads, dim,
           vdim, page_size, _stream())
@@ -747,6 +762,17 @@ def gla_norm_gate(o, proj, g_off: int, gain, eps: float, heads: int, vdim: int) 
     return out
 
 
+def head_norm_gate(o, gate, g_off: int, gain, eps: float, heads: int, vdim: int, out_dtype, kind: int) -> torch.Tensor:
+    """``rms_norm(o[t, h]) * gain * act(gate[t, h])`` in ``out_dtype``, ``act`` silu or the sigmoid (``kind``); the gate's rows,
+    float32 or ``out_dtype``, hold it at column ``g_off``; ``o``: float32 ``[T, heads * vdim]``."""
+    tokens, row = gate.shape
+    out = torch.empty((tokens, heads * vdim), dtype=out_dtype, device=gate.device)
+    _call("ri_head_norm_gate", _dev(out, "out"), code(out_dtype), _dev(o, "o", torch.float32, (tokens, heads * vdim)),
+          _dev(gate, "gate"), code(gate.dtype), row, g_off, _dev(gain, "gain", torch.float32, (vdim,)), float(eps), tokens, heads,
+          vdim, int(kind == GATE_SIGMOID), _stream())
+    return out
+
+
 def relu_squared(y: torch.Tensor) -> torch.Tensor:
     """``max(y, 0)^2`` elementwise."""
     out = torch.empty(y.shape, dtype=y.dtype, device=y.device)
@@ -848,6 +874,71 @@ def delta_step(proj, q_off: int, g_off: int, taps, tails, ab, a_log, dt_bias, st
     return out
 
 
+def _check_delta(tails, state, ntaps: int, channels: int, heads: int, dim: int, vdim: int) -> None:
+    if tails is not None and (tails.dim() != 3 or tuple(tails.shape[1:]) != (ntaps - 1, channels)):
+        raise ShapeError(f"the convolutions' tails are {list(tails.shape)}, not [slots, {ntaps - 1}, {channels}]")
+    if state is not None and (state.dim() != 4 or tuple(state.shape[1:]) != (heads, dim, vdim)):
+        raise ShapeError(f"the state is {list(state.shape)}, not [slots, {heads}, {dim}, {vdim}]")
+
+
+def _beta_logits(mid, b_off: int, heads: int, dtype):
+    """The address and row length of the logits of beta, ``heads`` columns of ``mid`` from ``b_off`` on."""
+    if b_off < 0 or b_off + heads > mid.shape[1]:
+        raise ShapeError(f"betas at column {b_off} of rows of {mid.shape[1]} for {heads} heads")
+    return _dev(mid, "mid", dtype) + b_off * mid.element_size(), mid.shape[1]
+
+
+def delta_prepare_channels(proj, q_off: int, taps, tails, z, mid, b_off: int, a_log, dt_bias, tok_seq, cu_seqlens, slots,
+                           heads: int, kv_heads: int, dim: int, vdim: int):
+    """``delta_prepare`` for a decay per head and key channel: ``z [T, >= heads * dim]`` float32 are the decays'
+    pre-activations, ``g = exp(-exp(a_log_h) softplus(z + dt_bias))`` with ``dt_bias [heads * dim]``; the logits of beta are the
+    columns ``b_off ..`` of ``mid`` (in the format of ``proj``).  ``gates`` is ``[T, heads * dim + heads]``."""
+    tokens, row = proj.shape
+    seqs, channels, ntaps = slots.shape[0], 2 * kv_heads * dim + heads * vdim, taps.shape[1]
+    _check_delta(tails, None, ntaps, channels, heads, dim, vdim)
+    qkv = torch.empty((tokens, channels), dtype=torch.float32, device=proj.device)
+    gates = torch.empty((tokens, heads * dim + heads), dtype=torch.float32, device=proj.device)
+    b, b_row = _beta_logits(mid, b_off, heads, proj.dtype)
+    _call("ri_delta_prepare_channels", _dev(qkv, "qkv"), _dev(gates, "gates"), _dev(proj, "proj"), code(proj.dtype), row, q_off,
+          _dev(taps, "taps", torch.float32, (channels, ntaps)), ntaps, _dev(tails, "tails", torch.float32),
+          _dev(z, "z", torch.float32, (tokens, z.shape[1])), z.shape[1], b, b_row, _dev(a_log, "a_log", torch.float32, (heads,)),
+          _dev(dt_bias, "dt_bias", torch.float32, (heads * dim,)), _dev(tok_seq, "tok_seq", torch.int32, (tokens,)),
+          _dev(cu_seqlens, "cu_seqlens", torch.int32, (seqs + 1,)), _dev(slots, "slots", torch.int32, (seqs,)),
+          seqs, tokens, heads, kv_heads, dim, vdim, _stream())
+    return qkv, gates
+
+
+def delta_scan_channels(qkv, gates, state, cu_seqlens, slots, heads: int, kv_heads: int, dim: int, vdim: int,
+                        slices: int = 0) -> torch.Tensor:
+    """``delta_scan`` for a decay per head and key channel (``gates`` of ``delta_prepare_channels``): ``S <- diag(g) S`` first."""
+    tokens, seqs = qkv.shape[0], slots.shape[0]
+    _check_delta(None, state, 1, 0, heads, dim, vdim)
+    out = torch.empty((tokens, heads * vdim), dtype=torch.float32, device=qkv.device)
+    _call("ri_delta_scan_channels", _dev(out, "out"), _dev(qkv, "qkv", torch.float32, (tokens, 2 * kv_heads * dim + heads * vdim)),
+          _dev(gates, "gates", torch.float32, (tokens, heads * dim + heads)), _dev(state, "state", torch.float32),
+          _dev(cu_seqlens, "cu_seqlens", torch.int32, (seqs + 1,)), _dev(slots, "slots", torch.int32, (seqs,)),
+          seqs, tokens, heads, kv_heads, dim, vdim, int(slices), _stream())
+    return out
+
+
+def delta_step_channels(proj, q_off: int, taps, tails, z, gate_at: int, mid, b_off: int, a_log, dt_bias, state, cu_seqlens, slots,
+                        gain, eps: float, heads: int, kv_heads: int, dim: int, vdim: int) -> torch.Tensor:
+    """``delta_step`` for a decay per head and key channel; the output gate is the sigmoid of ``z``'s columns ``gate_at ..``."""
+    seqs, row = proj.shape
+    channels, ntaps = 2 * kv_heads * dim + heads * vdim, taps.shape[1]
+    _check_delta(tails, state, ntaps, channels, heads, dim, vdim)
+    out = torch.empty((seqs, heads * vdim), dtype=proj.dtype, device=proj.device)
+    b, b_row = _beta_logits(mid, b_off, heads, proj.dtype)
+    _call("ri_delta_step_channels", _dev(out, "out"), _dev(proj, "proj"), code(proj.dtype), row, q_off,
+          _dev(taps, "taps", torch.float32, (channels, ntaps)), ntaps, _dev(tails, "tails", torch.float32),
+          _dev(z, "z", torch.float32, (seqs, z.shape[1])), z.shape[1], int(gate_at), b, b_row,
+          _dev(a_log, "a_log", torch.float32, (heads,)), _dev(dt_bias, "dt_bias", torch.float32, (heads * dim,)),
+          _dev(state, "state", torch.float32), _dev(cu_seqlens, "cu_seqlens", torch.int32, (seqs + 1,)),
+          _dev(slots, "slots", torch.int32, (seqs,)), _dev(gain, "gain", torch.float32, (vdim,)), float(eps), seqs, heads, kv_heads,
+          dim, vdim, _stream())
+    return out
+
+
 EXPERTS_MAX = 1024
 
 
@@ -887,16 +978,47 @@ def experts_route_general(z: torch.Tensor, correction: torch.Tensor, outs: int, 
     return ids, weights, dense, extra
 
 
-def experts_finish(routed: torch.Tensor, x, shared, extra: torch.Tensor) -> torch.Tensor:
-    """float32 ``routed + extra[:, 0] * x + extra[:, 1] * shared`` row by row; ``routed`` (float32) and ``shared`` may
-    be ``[parts, T, dim]`` (added in order); ``x`` and ``shared`` may be None."""
+def experts_finish(routed: torch.Tensor, x, shared, extra, plus: torch.Tensor | None = None) -> torch.Tensor:
+    """float32 ``routed + extra[:, 0] * x + extra[:, 1] * shared + plus`` row by row; ``routed`` (float32), ``shared`` and ``plus``
+    (float32) may be ``[parts, T, dim]`` (added in order); ``x``, ``shared`` and ``plus`` may be None, and so may ``extra`` where
+    ``x`` is (the shared expert's factor is then 1)."""
     tokens, dim = routed.shape[-2:]
     parts = routed.shape[0] if routed.dim() == 3 else 1
     shared_parts = shared.shape[0] if shared is not None and shared.dim() == 3 else 1
     out = torch.empty((tokens, dim), dtype=torch.float32, device=routed.device)
     _call("ri_experts_finish", _dev(out, "out"), _dev(routed, "routed", torch.float32), parts, _opt(x, "x"),
           code(x.dtype) if x is not None else F32, _opt(shared, "shared"), code(shared.dtype) if shared is not None else F32,
-          shared_parts, _dev(extra, "extra", torch.float32, (tokens, 2)), tokens, dim, _stream())
+          shared_parts, _opt(extra, "extra", torch.float32, (tokens, 2)), _opt(plus, "plus", torch.float32),
+          0 if plus is None else plus.shape[0] if plus.dim() == 3 else 1, tokens, dim, _stream())
+    return out
+
+
+def experts_by_table(table: torch.Tensor, token_ids: torch.Tensor, experts: int, dense: bool = True):
+    """The experts of tokens that a table gives: ``table [vocab, top]`` int32 (the entries of a row differ and are below
+    ``experts``).  Returns ``ids [T, top]``, ``weights [T, top]`` (all ``1 / top``) and, with ``dense``, the same as ``[T, experts]``."""
+    tokens, (vocab, top) = token_ids.shape[0], table.shape
+    ids = torch.empty((tokens, top), dtype=torch.int32, device=table.device)
+    weights = torch.empty((tokens, top), dtype=torch.float32, device=table.device)
+    spread = torch.empty((tokens, experts), dtype=torch.float32, device=table.device) if dense else None
+    _call("ri_experts_by_table", _dev(ids, "ids"), _dev(weights, "weights"), _opt(spread, "dense"), _dev(table, "table", torch.int32),
+          _dev(token_ids, "token_ids", torch.int32, (tokens,)), tokens, vocab, int(experts), top, _stream())
+    return ids, weights, spread
+
+
+def normed_sum(branches, gains, scales, eps: float) -> torch.Tensor:
+    """float32 ``sum_i scales[i] * rms_norm(branches[i]) * gains[i]`` over rows of the model's width: a branch is a product's
+    result, ``[T, dim]`` in either format or ``[parts, T, dim]`` float32 (the parts are added in order before the norm)."""
+    tokens, dim = branches[0].shape[-2:]
+    out = torch.empty((tokens, dim), dtype=torch.float32, device=branches[0].device)
+
+    def one(i):
+        if i >= len(branches):
+            return None, F32, 0, None, 0.0
+        y = branches[i]
+        return (_dev(y, "branch", None, y.shape[:-2] + (tokens, dim)), code(y.dtype), y.shape[0] if y.dim() == 3 else 1,
+                _dev(gains[i], "gain", torch.float32, (dim,)), float(scales[i]))
+    for i in range(0, len(branches), 2):
+        _call("ri_normed_sum", _dev(out, "out"), int(i > 0), *one(i), *one(i + 1), float(eps), tokens, dim, _stream())
     return out
 
 
@@ -1002,11 +1124,11 @@ def mfma_attention_fits(dtype, head_dim: int, group: int, page_size: int, decode
 def attention_prefill_bf16(qkv, k_pages, v_pages, cu_seqlens, tok_pos, page_table, seqs: int, max_new: int,
                            heads: int, kv_heads: int, head_dim: int, window: int | None, scale: float,
                            softcap: float | None = None, slopes: torch.Tensor | None = None, keep_first: int = 0,
-                           sinks: torch.Tensor | None = None, q_off: int = 0) -> torch.Tensor:
+                           sinks: torch.Tensor | None = None, q_off: int = 0, chunk: int | None = None) -> torch.Tensor:
     """Matrix-core attention for any number of new tokens per sequence (bfloat16, pages of 32).  With ``softcap`` a
     score ``s`` becomes ``softcap * tanh(s / softcap)`` before the softmax; with ``slopes`` (float32 ``[heads]``) head
-    ``h``'s score at position ``p`` for the key at ``j`` then loses ``slopes[h] * (p - j)``.  ``keep_first``, ``sinks`` and
-    ``q_off`` as in ``attention``."""
+    ``h``'s score at position ``p`` for the key at ``j`` then loses ``slopes[h] * (p - j)``.  ``keep_first``, ``sinks``,
+    ``q_off`` and ``chunk`` as in ``attention``."""
     tokens, stride = qkv.shape
     if q_off < 0 or q_off + heads * head_dim > stride or q_off % 8:
         raise ShapeError(f"attention: queries at column {q_off} of rows of {stride} for {heads} heads of {head_dim}")
@@ -1015,7 +1137,7 @@ def attention_prefill_bf16(qkv, k_pages, v_pages, cu_seqlens, tok_pos, page_tabl
           _dev(k_pages, "k_pages", torch.bfloat16), _dev(v_pages, "v_pages", torch.bfloat16),
           _dev(cu_seqlens, "cu_seqlens", torch.int32, (seqs + 1,)), _dev(tok_pos, "tok_pos", torch.int32, (tokens,)),
           _dev(page_table, "page_table", torch.int32), page_table.shape[1], seqs, max_new, heads, kv_heads, head_dim,
-          k_pages.shape[2], int(window or 0), float(scale), float(softcap or 0.0),
+          k_pages.shape[2], int(window or 0), int(chunk or 0), float(scale), float(softcap or 0.0),
           _opt(slopes, "slopes", torch.float32, (heads,)), int(keep_first or 0), _opt(sinks, "sinks", torch.float32, (heads,)),
           _stream())
     return out
@@ -1040,7 +1162,7 @@ def _padded_sizes(k_pages, v_pages, heads: int, kv_heads: int, stride: int, q_of
 def attention_prefill_padded(qkv, k_pages, v_pages, cu_seqlens, tok_pos, page_table, seqs: int, max_new: int, heads: int,
                              kv_heads: int, window: int | None, scale: float, softcap: float | None = None,
                              slopes: torch.Tensor | None = None, keep_first: int = 0, sinks: torch.Tensor | None = None,
-                             q_off: int = 0) -> torch.Tensor:
+                             q_off: int = 0, chunk: int | None = None) -> torch.Tensor:
     """``attention_prefill_bf16`` for key and value heads of their own sizes, which the pages give."""
     tokens, stride = qkv.shape
     dim, vdim, page_size = _padded_sizes(k_pages, v_pages, heads, kv_heads, stride, q_off)
@@ -1049,7 +1171,7 @@ def attention_prefill_padded(qkv, k_pages, v_pages, cu_seqlens, tok_pos, page_ta
           _dev(k_pages, "k_pages", torch.bfloat16), _dev(v_pages, "v_pages", torch.bfloat16),
           _dev(cu_seqlens, "cu_seqlens", torch.int32, (seqs + 1,)), _dev(tok_pos, "tok_pos", torch.int32, (tokens,)),
           _dev(page_table, "page_table", torch.int32), page_table.shape[1], seqs, max_new, heads, kv_heads, dim, vdim, page_size,
-          int(window or 0), float(scale), float(softcap or 0.0), _opt(slopes, "slopes", torch.float32, (heads,)),
+          int(window or 0), int(chunk or 0), float(scale), float(softcap or 0.0), _opt(slopes, "slopes", torch.float32, (heads,)),
           int(keep_first or 0), _opt(sinks, "sinks", torch.float32, (heads,)), _stream())
     return out
 
@@ -1057,7 +1179,7 @@ def attention_prefill_padded(qkv, k_pages, v_pages, cu_seqlens, tok_pos, page_ta
 def attention_decode_padded(qkv, k_pages, v_pages, tok_pos, page_table, seqs: int, max_len: int, heads: int, kv_heads: int,
                             window: int | None, scale: float, tiled_out: bool = False, softcap: float | None = None,
                             slopes: torch.Tensor | None = None, keep_first: int = 0, sinks: torch.Tensor | None = None,
-                            q_off: int = 0):
+                            q_off: int = 0, chunk: int | None = None):
     """``attention_decode_bf16`` for key and value heads of their own sizes, which the pages give."""
     tokens, stride = qkv.shape
     if tokens != seqs:
@@ -1072,7 +1194,7 @@ def attention_decode_padded(qkv, k_pages, v_pages, tok_pos, page_table, seqs: in
           _dev(qkv, "qkv", torch.bfloat16) + 2 * int(q_off), stride, _dev(k_pages, "k_pages", torch.bfloat16),
           _dev(v_pages, "v_pages", torch.bfloat16), _dev(tok_pos, "tok_pos", torch.int32, (tokens,)),
           _dev(page_table, "page_table", torch.int32), page_table.shape[1], seqs, chunks, heads, kv_heads, dim, vdim, page_size,
-          int(window or 0), float(scale), float(softcap or 0.0), _opt(slopes, "slopes", torch.float32, (heads,)), int(tiled_out),
+          int(window or 0), int(chunk or 0), float(scale), float(softcap or 0.0), _opt(slopes, "slopes", torch.float32, (heads,)), int(tiled_out),
           int(keep_first or 0), _opt(sinks, "sinks", torch.float32, (heads,)), _stream())
     return out
 
@@ -1093,11 +1215,11 @@ def decode_attention_streams(seqs: int, kv_heads: int, max_len: int) -> bool:
 def attention_decode_bf16(qkv, k_pages, v_pages, cu_seqlens, tok_pos, page_table, seqs: int, max_len: int,
                           heads: int, kv_heads: int, head_dim: int, window: int | None, scale: float,
                           tiled_out: bool = False, softcap: float | None = None, slopes: torch.Tensor | None = None,
-                          keep_first: int = 0, sinks: torch.Tensor | None = None, q_off: int = 0):
+                          keep_first: int = 0, sinks: torch.Tensor | None = None, q_off: int = 0, chunk: int | None = None):
     """Matrix-core attention for one new token per sequence; ``max_len`` bounds every sequence's length
     after this step (it sizes the grid and the workspace, not the result).  ``tiled_out``: the result as
     ``TiledRows`` (at most 64 sequences).  ``softcap`` and ``slopes`` as in ``attention_prefill_bf16``; ``keep_first``,
-    ``sinks`` and ``q_off`` as in ``attention`` (``keep_first`` in steps for which ``decode_attention_streams`` is false)."""
+    ``sinks``, ``q_off`` and ``chunk`` as in ``attention`` (``keep_first`` in steps for which ``decode_attention_streams`` is false)."""
     tokens, stride = qkv.shape
     if tokens != seqs:
         raise ShapeError(f"decode attention takes one token per sequence, got {tokens} tokens for {seqs} sequences")
@@ -1113,7 +1235,7 @@ def attention_decode_bf16(qkv, k_pages, v_pages, cu_seqlens, tok_pos, page_table
           _dev(k_pages, "k_pages", torch.bfloat16), _dev(v_pages, "v_pages", torch.bfloat16),
           _dev(cu_seqlens, "cu_seqlens", torch.int32, (seqs + 1,)), _dev(tok_pos, "tok_pos", torch.int32, (tokens,)),
           _dev(page_table, "page_table", torch.int32), page_table.shape[1], seqs, chunks, heads, kv_heads, head_dim,
-          k_pages.shape[2], int(window or 0), float(scale), float(softcap or 0.0),
+          k_pages.shape[2], int(window or 0), int(chunk or 0), float(scale), float(softcap or 0.0),
           _opt(slopes, "slopes", torch.float32, (heads,)), int(tiled_out), int(keep_first or 0),
           _opt(sinks, "sinks", torch.float32, (heads,)), _stream())
     return out

@@ -1,5 +1,6 @@
 from . import (attention, block, decay_attention, delta, experts, feed_forward, gla, latent, norm, parallel, position,
-               postnorm, sandwich, ssd, streams, talking, timemix, qwen3, zidepel, pisulorn, zakelorn, dagezen, notadra)  # noqa: F401  (registers the parts)
+               postnorm, sandwich, ssd, streams, talking, timemix, qwen3, zidepel, pisulorn, zakelorn, dagezen, notadra,
+               kisepel)  # noqa: F401  (registers the parts)
 from .base import Embedding, FeedForward, Head, Mixer, Norm, Part, PositionEncoding
 from .block import PreNormBlock, ResidualStream
 from .context import StepContext

@@ -11,6 +11,7 @@ from ..errors import ConfigError
 from ..kernels import ops
 from ..weights.loader import BIAS, GAIN, MATRIX, TensorSpec
 from .base import Mixer
+from .position import RotateHalf
 from .registry import build_part, register_part
 from .spec import PartSpec
 
@@ -66,8 +67,11 @@ class GroupedQueryAttention(Mixer):
     ``v_dim``, a ``softcap``, a ``window`` (with ``keep_first``) and sinks; a rotation with an ``amplitude`` or over part of a head;
     ``sinks="zero"``, a sink whose score is 0 for every head and which has no tensor (the softmax's denominator grows by
     one); ``reads_kv``, a layer without keys and values of its own: its run names the cache entry of an earlier layer of
-    the same geometry, whose keys it reads as they lie there, rotated, with its own queries.  ``sinks="zero"``, ``reads_kv``
-    or a rotation with an amplitude sends the mixer through ``ops.qk_half_bias_kv_write``.
+    the same geometry, whose keys it reads as they lie there, rotated, with its own queries.  ``chunk``: positions form runs of
+    that many, counted from the sequence's start, and a query sees the keys of its own run alone; the q/k norm with gains comes
+    before the rotation, as in the first family.  ``sinks="zero"``, ``reads_kv``, ``chunk``, a rotation with an amplitude, or one of
+    halves beside a ``v_dim``, sends the mixer through ``ops.qk_half_bias_kv_write``.  Such a mixer can share one input product with
+    others (``in_matrix``, ``heads_from``).
     """
 
     links_norms = True
@@ -77,7 +81,7 @@ class GroupedQueryAttention(Mixer):
                  qkv_bias: bool = False, o_bias: bool = False, v_dim: int | None = None, scale: float | None = None,
                  softcap: float | None = None, q_temper: tuple | None = None, names: dict | None = None,
                  distance_slopes: tuple | None = None, keep_first: int = 0, sinks: bool | str = False, gate: str | None = None,
-                 reads_kv: bool = False):
+                 reads_kv: bool = False, chunk: int | None = None):
         if heads < 1 or kv_heads < 1 or heads % kv_heads:
             raise ConfigError(f"{heads} attention heads not divisible by {kv_heads} kv heads")
         if not 1 <= head_dim <= ops.MAX_HEAD_DIM:
@@ -106,11 +110,17 @@ class GroupedQueryAttention(Mixer):
         self.keep_first, self.sinks, self.gate = int(keep_first or 0), bool(sinks) and not self.zero_sink, gate
         self.reads_kv, self.amplitude = bool(reads_kv), float(getattr(self.position, "amplitude", 1.0))
         # biases, halves and the rest in one kernel: the fourth family
-        self.halved = self.zero_sink or self.reads_kv or self.amplitude != 1.0
-        if self.halved and (qk_norm or gate is not None or self.q_temper is not None or o_bias
+        self.chunk = int(chunk) if chunk is not None else None
+        if self.chunk is not None and (self.chunk < 1 or window is not None):
+            raise ConfigError(f"chunks of {chunk} positions: a positive number, and no window beside it ({window})")
+        halves = isinstance(self.position, RotateHalf)
+        self.halved = (self.zero_sink or self.reads_kv or self.amplitude != 1.0 or self.chunk is not None
+                       or (halves and self.v_dim != head_dim))
+        if self.halved and (qk_norm == "unit" or (qk_norm and self.reads_kv) or gate is not None or self.q_temper is not None or o_bias
                             or getattr(self.position, "pairs", False) or getattr(self.position, "acts_after_norm", False)):
-            raise ConfigError("an attention that reads another layer's keys, has a sink of score 0 or a rotation with an "
-                              "amplitude takes no q/k norm, gate, query temperature or output bias, and rotates halves or not at all")
+            raise ConfigError("an attention that reads another layer's keys, has a sink of score 0, chunks or a rotation with an "
+                              "amplitude takes no unit norm (and none beside another layer's keys), gate, query temperature or output "
+                              "bias, and rotates halves or not at all")
         if gate not in (None, "sigmoid", "silu"):
             raise ConfigError(f"an output gate {gate!r} is neither 'sigmoid' nor 'silu'")
         if self.keep_first < 0 or (self.keep_first and window is None):
@@ -201,7 +211,7 @@ class GroupedQueryAttention(Mixer):
 
     def bind_plain(self, weights):
         if self.halved:
-            raise ConfigError("an attention that reads another layer's keys, has a sink of score 0 or a rotation with an "
+            raise ConfigError("an attention that reads another layer's keys, has a sink of score 0, chunks or a rotation with an "
                               "amplitude has no plain form")
         if self.tempered or self.softcap is not None:
             raise ConfigError("an attention with a score cap, a query temperature or value heads of their own size has "
@@ -243,7 +253,7 @@ class GroupedQueryAttention(Mixer):
 
     def cache_need(self):
         return KVNeed(self.kv_heads, self.head_dim, self.window, None if self.v_dim == self.head_dim else self.v_dim,
-                      self.keep_first or None)
+                      self.keep_first or None, self.chunk)
 
     def forward(self, x, ctx, store, page_table, link=None):
         rt = self.rt
@@ -299,17 +309,22 @@ class GroupedQueryAttention(Mixer):
         return self.project_out(o, link)
 
     def forward_halved(self, proj, ctx, store, page_table):
-        """Biases, rotation in halves and the write of k and v in one kernel (queries alone where the keys are another
-        layer's), then the attention over the entry the run names."""
-        own = 0 if self.reads_kv else self.kv_heads
-        with profiler.section(profiler.QK_NORM_ROPE_APPEND):
-            ops.qk_half_bias_kv_write(proj, 0, self.q_width, self.q_width + self.k_width, self.b_qkv, self.position.rotation_table(),
-                                      self.amplitude, ctx.tok_pos, ctx.tok_seq, page_table, store.k_pages, store.v_pages, self.heads,
-                                      own, self.head_dim, self.v_dim, ctx.cu_seqlens, ctx.max_new)
-        with profiler.section(profiler.ATTENTION):
-            o = self.attend_kept(proj, 0, ctx, store, page_table)
+        o = self.heads_from(None, proj, 0, ctx, store, page_table)
         with profiler.section(profiler.OUT_PROJECTION):
             return self.rt.linear_packed(o, self.w_o, out_dtype=torch.float32, parts_ok=True)
+
+    def heads_from(self, x, proj, col0: int, ctx, store, page_table):
+        """The fourth family between its two products: ``proj [T, row]`` holds q, k and v from column ``col0`` on.  Biases, q/k
+        norm, rotation in halves and the write of k and v in one kernel (queries alone where the keys are another layer's), then
+        the attention over the entry the run names: the heads side by side, ready for the output product."""
+        own = 0 if self.reads_kv else self.kv_heads
+        k_at = col0 + self.q_width
+        with profiler.section(profiler.QK_NORM_ROPE_APPEND):
+            ops.qk_half_bias_kv_write(proj, col0, k_at, k_at + self.k_width, self.b_qkv, self.position.rotation_table(),
+                                      self.amplitude, ctx.tok_pos, ctx.tok_seq, page_table, store.k_pages, store.v_pages, self.heads,
+                                      own, self.head_dim, self.v_dim, ctx.cu_seqlens, ctx.max_new, self.q_gain, self.k_gain, self.eps)
+        with profiler.section(profiler.ATTENTION):
+            return self.attend_kept(proj, col0, ctx, store, page_table)
 
     def core(self, proj, col0: int, ctx, store, page_table, out, out_col: int, out_scale: float) -> None:
         """The mixer between its two products: ``proj [T, row]`` holds this mixer's q, k, v (and g) from column
@@ -336,7 +351,8 @@ class GroupedQueryAttention(Mixer):
         tiled = self.halved and ctx.is_decode and not self.rt.invariant and self.rt.takes_tiled(self.w_o, ctx.B, True)
         if self.halved and (self.v_dim != self.head_dim or self.head_dim not in ops.MFMA_HEAD_DIMS):
             args = (self.heads, self.kv_heads, self.window, self.scale)
-            kw = {"softcap": self.softcap, "slopes": slopes, "keep_first": self.keep_first, "sinks": self.sink, "q_off": q_at}
+            kw = {"softcap": self.softcap, "slopes": slopes, "keep_first": self.keep_first, "sinks": self.sink, "q_off": q_at,
+                  "chunk": self.chunk}
             sizes = (proj.dtype, self.head_dim, self.v_dim, group, store.page_size)
             if aligned and ctx.is_decode and not self.rt.invariant and ops.padded_attention_fits(*sizes, True):
                 return ops.attention_decode_padded(proj, store.k_pages, store.v_pages, ctx.tok_pos, page_table, ctx.B, ctx.max_len, *args,
@@ -353,16 +369,16 @@ class GroupedQueryAttention(Mixer):
             return ops.attention_decode_bf16(proj, store.k_pages, store.v_pages, ctx.cu_seqlens, ctx.tok_pos, page_table,
                                              ctx.B, ctx.max_len, self.heads, self.kv_heads, self.head_dim, self.window,
                                              self.scale, tiled_out=tiled, softcap=self.softcap, slopes=slopes,
-                                             keep_first=self.keep_first, sinks=self.sink, q_off=q_at)
+                                             keep_first=self.keep_first, sinks=self.sink, q_off=q_at, chunk=self.chunk)
         if fits and ops.mfma_attention_fits(proj.dtype, self.head_dim, group, store.page_size, False):
             # the matrix cores' prompt kernel, also for the single tokens of a step that fills the machine: a
             # wavefront walks a sequence's pages in their order
             return ops.attention_prefill_bf16(proj, store.k_pages, store.v_pages, ctx.cu_seqlens, ctx.tok_pos, page_table,
                                               ctx.B, ctx.max_new, self.heads, self.kv_heads, self.head_dim, self.window,
-                                              self.scale, self.softcap, slopes, self.keep_first, self.sink, q_at)
+                                              self.scale, self.softcap, slopes, self.keep_first, self.sink, q_at, self.chunk)
         return ops.attention(proj, store.k_pages, store.v_pages, ctx.tok_pos, ctx.tok_seq, page_table, self.heads,
                              self.kv_heads, self.head_dim, self.window, self.scale, self.softcap, slopes,
-                             keep_first=self.keep_first, sinks=self.sink, q_off=q_at)
+                             keep_first=self.keep_first, sinks=self.sink, q_off=q_at, chunk=self.chunk)
 
     def forward_tempered(self, qkv, ctx, store, page_table, link):
         """No rotation: per-head norm, query temperature and the write of k and v in one kernel, then the attention

@@ -83,6 +83,12 @@ class ResidualStream:
             self.pending = None      # the kernel wrote sum + pending back
         return out
 
+    def add(self, rows) -> None:
+        """``x <- x + rows`` (float32) outside any sublayer.  A branch that waits goes on waiting; what was prepared from the sum
+        as it was is dropped."""
+        self.later = self.as_act = self.prepared = None
+        ops.add_rows(self.sum, rows, in_place=True)
+
     def flush(self) -> None:
         """Add the waiting branch without a norm (only arrangements that push twice need it)."""
         self.later = None            # its sum is in the stream already
@@ -152,6 +158,37 @@ class PreNormBlock:
             stream.push(self.feed_forward.forward(h, ctx, link=link))
         else:
             h = stream.normed(self.feed_forward_norm, act_dtype)
+            stream.push(self.feed_forward.forward(h, ctx))
+
+
+@register_part("arrangement", "parallel_prenorm")
+class ParallelPreNormBlock:
+    """``x <- x + (mixer(h) + ff(h))`` with ``h = norm(x)``: one norm, whose rows both sublayers read.  Parts: ``mixer_norm``,
+    ``mixer`` and, for a layer that has one, ``feed_forward``.  A feed-forward that sets ``adds_branch`` adds the mixer's result
+    where it adds up its own (``plus=``); the sum then waits for the next norm as one branch."""
+
+    def __init__(self, layer_spec):
+        self.mixer_norm = build_part("norm", layer_spec.mixer_norm)
+        self.mixer = build_part("mixer", layer_spec.mixer)
+        self.feed_forward = build_part("feed_forward", layer_spec.feed_forward) if "feed_forward" in layer_spec.parts else None
+
+    def parts(self):
+        first = (self.mixer_norm, self.mixer)
+        return first if self.feed_forward is None else first + (self.feed_forward,)
+
+    def entry_norm(self):
+        """The norm through which this layer first reads the stream."""
+        return self.mixer_norm
+
+    def forward(self, stream: ResidualStream, ctx, store, page_table, act_dtype) -> None:
+        h = stream.normed(self.mixer_norm, act_dtype)
+        y = self.mixer.forward(h, ctx, store, page_table)
+        if self.feed_forward is None:
+            stream.push(y)
+        elif getattr(self.feed_forward, "adds_branch", False) and isinstance(y, torch.Tensor) and y.dtype == torch.float32:
+            stream.push(self.feed_forward.forward(h, ctx, plus=y))
+        else:
+            stream.push(y)
             stream.push(self.feed_forward.forward(h, ctx))
 
 

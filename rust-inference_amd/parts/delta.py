@@ -32,10 +32,19 @@ class GatedDeltaRule(Mixer):
     ``names``: checkpoint names of ``q, k, v, g, o, a, b, norm, A_log, dt_bias`` where they are not ``<prefix>q`` and
     so on; the taps of q, k and v are ``<name>.conv``.  q, k, v and g are one product with the row-concatenated
     weight, a and b another whose result is float32.
+
+    ``decay="channel"``: a decay per value head and key channel, through a narrow middle whose width the checkpoint gives
+    (unless ``rank`` names it): ``g = exp(-exp(A_log_h) softplus(W_a2 (W_a1 h) + dt_bias))`` with ``dt_bias [heads * dim]``, and
+    ``S <- diag(g) S``; the output gate then is ``sigmoid(W_g2 (W_g1 h))``, through a middle of its own.  Names ``a1, a2, g1, g2`` in
+    the place of ``a`` and ``g``.  Both middles and the logits of beta are one product (``[a1; g1; b]``), both second steps
+    another, with the block-diagonal of ``a2`` and ``g2``, whose result is float32.  This form can share one input product with
+    other mixers (``in_matrix``, ``heads_from``).
     """
 
     def __init__(self, hidden: int, heads: int, kv_heads: int, dim: int, vdim: int, taps: int, prefix: str,
-                 eps: float = 1e-5, names: dict | None = None):
+                 eps: float = 1e-5, names: dict | None = None, decay: str = "head", rank: int | None = None):
+        if decay not in ("head", "channel"):
+            raise ConfigError(f"a delta rule's decay {decay!r} is neither 'head' nor 'channel'")
         if heads < 1 or kv_heads < 1 or heads % kv_heads:
             raise ConfigError(f"{heads} delta-rule heads not divisible by {kv_heads} query/key heads")
         if not 1 <= dim <= ops.DELTA_MAX_DIM or vdim < 1:
@@ -45,12 +54,24 @@ class GatedDeltaRule(Mixer):
         self.hidden, self.heads, self.kv_heads, self.dim, self.vdim, self.taps = hidden, heads, kv_heads, dim, vdim, taps
         self.prefix, self.eps = prefix, eps
         p = prefix
-        self.names = {n: p + n for n in ("q", "k", "v", "g", "o", "a", "b", "norm", "A_log", "dt_bias")}
+        self.per_channel, self.rank = decay == "channel", rank
+        self.names = {n: p + n for n in ("q", "k", "v", "g", "o", "a", "b", "norm", "A_log", "dt_bias", "a1", "a2", "g1", "g2")}
         self.names.update(names or {})
-        self.channels = 2 * kv_heads * dim + heads * vdim
+        self.in_width = self.channels = 2 * kv_heads * dim + heads * vdim
 
     def tensors(self):
         n, d, hk, hv, h = self.names, self.hidden, self.kv_heads * self.dim, self.heads * self.vdim, self.heads
+        if self.per_channel:
+            hd = h * self.dim
+            return {
+                n["q"]: TensorSpec((hk, d), MATRIX), n["k"]: TensorSpec((hk, d), MATRIX), n["v"]: TensorSpec((hv, d), MATRIX),
+                n["q"] + ".conv": TensorSpec((hk, self.taps), MATRIX), n["k"] + ".conv": TensorSpec((hk, self.taps), MATRIX),
+                n["v"] + ".conv": TensorSpec((hv, self.taps), MATRIX), n["o"]: TensorSpec((d, hv), MATRIX),
+                n["a1"]: TensorSpec((self.rank, d), MATRIX), n["a2"]: TensorSpec((hd, self.rank), MATRIX),
+                n["g1"]: TensorSpec((self.rank, d), MATRIX), n["g2"]: TensorSpec((hv, self.rank), MATRIX),
+                n["b"]: TensorSpec((h, d), MATRIX), n["A_log"]: TensorSpec((h,), BIAS), n["dt_bias"]: TensorSpec((hd,), BIAS),
+                n["norm"]: TensorSpec((self.vdim,), GAIN),
+            }
         return {
             n["q"]: TensorSpec((hk, d), MATRIX), n["k"]: TensorSpec((hk, d), MATRIX), n["v"]: TensorSpec((hv, d), MATRIX),
             n["q"] + ".conv": TensorSpec((hk, self.taps), MATRIX), n["k"] + ".conv": TensorSpec((hk, self.taps), MATRIX),
@@ -61,9 +82,42 @@ class GatedDeltaRule(Mixer):
             n["norm"]: TensorSpec((self.vdim,), GAIN),
         }
 
-    def bind(self, weights, rt):
+    def in_matrix(self, weights):
+        """The rows of this mixer's input product (of the form with a decay per channel), ``[q; k; v]``."""
+        return torch.cat([weights[self.names[x]] for x in "qkv"], 0)
+
+    def out_matrix(self, weights):
+        return weights[self.names["o"]]
+
+    def bind_channels(self, weights, rt, alone: bool) -> None:
+        n = self.names
+        a1, a2, g1, g2 = (weights[n[x]] for x in ("a1", "a2", "g1", "g2"))
+        for one, two in (("a1", "a2"), ("g1", "g2")):
+            if weights[n[one]].shape[0] != weights[n[two]].shape[1]:
+                raise ConfigError(f"{n[one]} has {weights[n[one]].shape[0]} rows, {n[two]} {weights[n[two]].shape[1]} columns")
+        ra, rg = a1.shape[0], g1.shape[0]
+        self.b_at = ra + rg
+        width = -(-(self.b_at + self.heads) // 8) * 8                  # the next product's rows in 16-byte pieces
+        mid = torch.zeros((width, self.hidden), dtype=a1.dtype, device=a1.device)
+        mid[:ra], mid[ra:self.b_at], mid[self.b_at:self.b_at + self.heads] = a1, g1, weights[n["b"]]
+        second = torch.zeros((a2.shape[0] + g2.shape[0], width), dtype=a1.dtype, device=a1.device)
+        second[:a2.shape[0], :ra], second[a2.shape[0]:, ra:self.b_at] = a2, g2
+        self.w_mid, self.w_second = rt.pack(rt.place_matrix(mid)), rt.pack(rt.place_matrix(second))
+        if alone:
+            self.w_in = rt.pack(rt.place_matrix(self.in_matrix(weights)), always=True)
+
+    def bind(self, weights, rt, alone: bool = True):
+        """``alone`` False: another part owns the products before and after (mixers side by side)."""
         self.rt = rt
         n = self.names
+        if self.per_channel:
+            self.bind_channels(weights, rt, alone)
+            self.conv_taps = rt.place_gain(torch.cat([weights[n[x] + ".conv"] for x in "qkv"], 0))
+            self.a_log, self.dt_bias = rt.place_gain(weights[n["A_log"]]), rt.place_gain(weights[n["dt_bias"]])
+            self.gain = rt.place_gain(weights[n["norm"]])
+            if alone:
+                self.w_o = rt.pack(rt.place_matrix(weights[n["o"]]), parts_ok=True)
+            return
         fused = torch.cat([weights[n["q"]], weights[n["k"]], weights[n["v"]], weights[n["g"]]], 0)
         self.w_qkvg = rt.pack(rt.place_matrix(fused), always=True)      # four projections in one
         self.w_ab = rt.pack(rt.place_matrix(torch.cat([weights[n["a"]], weights[n["b"]]], 0)))
@@ -76,8 +130,34 @@ class GatedDeltaRule(Mixer):
         return (StateNeed((self.heads, self.dim, self.vdim), torch.float32),
                 StateNeed((self.taps - 1, self.channels), torch.float32))
 
+    def heads_from(self, x, proj, col0: int, ctx, store, page_table):
+        """The form with a decay per channel between its two products: ``proj [T, row]`` holds q, k and v from column ``col0``
+        on, ``x`` is the mixer's input; the normed and gated heads, ready for the output product."""
+        rt = self.rt
+        state, tails = store
+        sizes = (self.heads, self.kv_heads, self.dim, self.vdim)
+        with profiler.section(profiler.QKV_PROJECTION):
+            mid = ops.as_rows(rt.linear_packed(x, self.w_mid))                        # [T, a1 | g1 | b]
+            z = ops.as_rows(rt.linear_packed(mid, self.w_second, out_dtype=torch.float32))      # [T, decays | gates]
+        gate_at = self.heads * self.dim
+        one_form = rt.dtype == torch.float32 or rt.invariant
+        with profiler.section(profiler.ATTENTION):
+            if ctx.is_decode and not one_form and ops.delta_step_fits(self.dim, self.vdim):
+                return ops.delta_step_channels(proj, col0, self.conv_taps, tails, z, gate_at, mid, self.b_at, self.a_log, self.dt_bias,
+                                               state, ctx.cu_seqlens, ctx.slots, self.gain, self.eps, *sizes)
+            qkv, gates = ops.delta_prepare_channels(proj, col0, self.conv_taps, tails, z, mid, self.b_at, self.a_log, self.dt_bias,
+                                                    ctx.tok_seq, ctx.cu_seqlens, ctx.slots, *sizes)
+            o = ops.delta_scan_channels(qkv, gates, state, ctx.cu_seqlens, ctx.slots, *sizes, slices=4 if one_form else 0)
+            return ops.head_norm_gate(o, z, gate_at, self.gain, self.eps, self.heads, self.vdim, rt.dtype, ops.GATE_SIGMOID)
+
     def forward(self, x, ctx, store, page_table):
         rt = self.rt
+        if self.per_channel:
+            with profiler.section(profiler.QKV_PROJECTION):
+                proj = ops.as_rows(rt.linear_packed(x, self.w_in))
+            heads = self.heads_from(x, proj, 0, ctx, store, page_table)
+            with profiler.section(profiler.OUT_PROJECTION):
+                return rt.linear_packed(heads, self.w_o, out_dtype=torch.float32, parts_ok=True)
         state, tails = store
         with profiler.section(profiler.QKV_PROJECTION):
             proj = ops.as_rows(rt.linear_packed(x, self.w_qkvg))          # [T, q | k | v | g]

@@ -6,7 +6,7 @@ import torch
 from .. import profiler
 from ..errors import ConfigError
 from ..kernels import ops
-from ..weights.loader import BIAS, MATRIX, TensorSpec
+from ..weights.loader import BIAS, MATRIX, TABLE, TensorSpec
 from .base import FeedForward
 from .registry import register_part
 
@@ -42,13 +42,19 @@ class RoutedExperts(FeedForward):
     correction; with ``scores="softmax"`` and ``normalize=True`` the weights are then the softmax over the chosen logits alone.
     ``shared=ff``: one more expert of that width and form, ``<prefix>shared.gate`` / ``.up`` / ``.down``, runs for
     every token and is added times ``sigmoid(W_sg h)``, one number a token (``<prefix>shared.sg [1, hidden]``; its row
-    rides as the last row of the router's matrix).
+    rides as the last row of the router's matrix); ``shared_gate=False``: it is added as it is and has no such tensor.
+    ``scores="table"``: no router.  ``<prefix>table [vocab, top]`` (integers, the entries of a row differ) gives every token id its
+    experts, each with the weight ``1 / top``.
+
+    ``forward(..., plus=y)``: another sublayer's float32 result, ``[T, hidden]`` or in parts, to be added to this one's.
     """
+
+    adds_branch = True
 
     def __init__(self, hidden: int, inter: int, experts: int, top: int, limit: float | None, prefix: str,
                  scores: str = "sigmoid", normalize: bool = True, groups: tuple | None = None, identity: int = 0,
                  shared: int | None = None, gated: bool = True, activation: str | None = None, router_bias: bool = False,
-                 group_score: str = "best"):
+                 group_score: str = "best", shared_gate: bool = True, vocab: int | None = None):
         self.outs = experts + int(identity)
         self.gated, self.activation, self.router_bias = bool(gated), activation, bool(router_bias)
         if not self.gated:
@@ -61,8 +67,11 @@ class RoutedExperts(FeedForward):
                               f"{ops.EXPERTS_MAX} outputs")
         if limit is not None and not limit > 0:
             raise ConfigError(f"the experts' limit {limit} must be positive")
-        if scores not in ("sigmoid", "softmax"):
-            raise ConfigError(f"router scores {scores!r} are neither 'sigmoid' nor 'softmax'")
+        if scores not in ("sigmoid", "softmax", "table"):
+            raise ConfigError(f"router scores {scores!r} are none of 'sigmoid', 'softmax' and 'table'")
+        self.by_table, self.vocab, self.shared_gate = scores == "table", vocab, bool(shared_gate) and shared is not None
+        if self.by_table and (groups or identity or router_bias or self.shared_gate or not vocab):
+            raise ConfigError("experts by a table of token ids need the number of ids and take no groups, identity experts, bias or gate")
         self.hidden, self.inter, self.experts, self.top, self.prefix = hidden, inter, experts, top, prefix
         self.limit = float(limit) if limit is not None else 0.0          # 0: the plain gated form
         self.scores, self.normalize, self.identity, self.shared = scores, bool(normalize), int(identity), shared
@@ -73,12 +82,17 @@ class RoutedExperts(FeedForward):
         if self.outs % self.groups or not 1 <= self.keep <= self.groups or top > self.keep * (self.outs // self.groups):
             raise ConfigError(f"{self.outs} router outputs in {self.groups} groups of which {self.keep} stay, for the {top} best")
         # the router of the first designs: one kernel call and no extras
-        self.simple = (scores == "sigmoid" and self.normalize and self.groups == 1 and not self.identity and shared is None)
+        self.simple = (scores == "sigmoid" and self.shared is None and self.normalize and self.groups == 1 and not self.identity and shared is None)
 
     def tensors(self):
         p, t = self.prefix, {}
-        t[p + "router"] = TensorSpec((self.outs, self.hidden), MATRIX)
-        if self.router_bias:
+        if self.by_table:
+            t[p + "table"] = TensorSpec((self.vocab, self.top), TABLE, below=self.experts)
+        else:
+            t[p + "router"] = TensorSpec((self.outs, self.hidden), MATRIX)
+        if self.by_table:
+            pass
+        elif self.router_bias:
             t[p + "router.b"] = TensorSpec((self.outs,), BIAS)
         else:
             t[p + "correction"] = TensorSpec((self.outs,), BIAS)
@@ -86,7 +100,8 @@ class RoutedExperts(FeedForward):
             t[p + "shared.gate"] = TensorSpec((self.shared, self.hidden), MATRIX)
             t[p + "shared.up"] = TensorSpec((self.shared, self.hidden), MATRIX)
             t[p + "shared.down"] = TensorSpec((self.hidden, self.shared), MATRIX)
-            t[p + "shared.sg"] = TensorSpec((1, self.hidden), MATRIX)
+            if self.shared_gate:
+                t[p + "shared.sg"] = TensorSpec((1, self.hidden), MATRIX)
         for e in range(self.experts):
             if self.gated:
                 t[f"{p}e{e}.gate"] = TensorSpec((self.inter, self.hidden), MATRIX)
@@ -97,14 +112,23 @@ class RoutedExperts(FeedForward):
     def bind(self, weights, rt):
         self.rt = rt
         p = self.prefix
-        router = weights[p + "router"]
-        if self.shared is not None:                       # the shared expert's gate: one more row of logits
-            router = torch.cat([router, weights[p + "shared.sg"].to(router.dtype)], 0)
+        if self.shared is not None:
             self.w_shared_in = rt.pack(rt.place_matrix(torch.cat([weights[p + "shared.gate"], weights[p + "shared.up"]], 0)),
                                        swiglu=True)
             self.w_shared_down = rt.pack(rt.place_matrix(weights[p + "shared.down"]), parts_ok=True)
-        self.w_router = rt.pack(rt.place_matrix(router))
-        if self.router_bias:
+        if self.by_table:
+            table = weights[p + "table"]
+            if table.numel() and not (0 <= int(table.min()) and int(table.max()) < self.experts):
+                raise ConfigError(f"{p}table names experts {int(table.min())} to {int(table.max())}, there are {self.experts}")
+            self.table = table.to(device=rt.device, dtype=torch.int32).contiguous()
+        else:
+            router = weights[p + "router"]
+            if self.shared_gate:                          # the shared expert's gate: one more row of logits
+                router = torch.cat([router, weights[p + "shared.sg"].to(router.dtype)], 0)
+            self.w_router = rt.pack(rt.place_matrix(router))
+        if self.by_table:
+            self.z_bias = self.correction = None
+        elif self.router_bias:
             # a bias of the router's product: it moves the logits themselves, so choice and weights both see it
             self.z_bias = rt.place_gain(weights[p + "router.b"])
             self.correction = torch.zeros_like(self.z_bias)
@@ -124,21 +148,25 @@ class RoutedExperts(FeedForward):
     # experts are computed for all tokens as two products, with zeros where a token did not choose.
     SORTED_MIN_TOKENS = 256
 
-    def forward(self, x, ctx):
+    def route(self, x, ctx):
+        """The choice of a step's tokens: ``ids``, ``weights`` ``[T, top]``, ``dense [T, outs]``, and ``extra`` (the identity experts'
+        weight and the shared expert's gate) where the router has one."""
+        if self.by_table:
+            return (*ops.experts_by_table(self.table, ctx.tokens, self.experts), None)
+        z = ops.as_rows(self.rt.linear_packed(x, self.w_router, out_dtype=torch.float32))
+        if self.z_bias is not None:
+            z = ops.add_bias(z, self.z_bias)
+        if self.simple:
+            return (*ops.experts_route(z, self.correction, self.top), None)
+        return ops.experts_route_general(z, self.correction, self.outs, self.experts, self.top,
+                                         ops.ROUTE_SOFTMAX if self.scores == "softmax" else ops.ROUTE_SIGMOID, self.normalize,
+                                         self.groups, self.keep, self.best_of)
+
+    def forward(self, x, ctx, plus=None):
         rt = self.rt
         with profiler.section(profiler.MLP):
-            z = ops.as_rows(rt.linear_packed(x, self.w_router, out_dtype=torch.float32))
-            if self.z_bias is not None:
-                z = ops.add_bias(z, self.z_bias)
-            extra = None
-            if self.simple:
-                ids, weights, dense = ops.experts_route(z, self.correction, self.top)
-            else:
-                ids, weights, dense, extra = ops.experts_route_general(
-                    z, self.correction, self.outs, self.experts, self.top,
-                    ops.ROUTE_SOFTMAX if self.scores == "softmax" else ops.ROUTE_SIGMOID, self.normalize, self.groups, self.keep,
-                    self.best_of)
-            tokens = z.shape[0]
+            ids, weights, dense, extra = self.route(x, ctx)
+            tokens = ids.shape[0]
             routed = (rt.dtype == torch.bfloat16 and not rt.invariant and self.top < self.experts
                       and self.hidden % 8 == 0 and self.inter % 8 == 0)
             own = self.identity > 0                   # whether the identity experts' share is still to be added
@@ -158,13 +186,14 @@ class RoutedExperts(FeedForward):
                      else ops.experts_activate_plain(gu, dense, self.inter, self.activation))
                 # float32 into the residual (or in parts that the stream's next read adds)
                 y = rt.linear_packed(a, self.w_down, out_dtype=torch.float32, parts_ok=True)
-            if not own and self.shared is None:
+            if not own and self.shared is None and plus is None:
                 return y
             shared = None
             if self.shared is not None:
                 act = rt.linear_packed(x, self.w_shared_in)
                 shared = rt.linear_packed(act, self.w_shared_down, out_dtype=torch.float32, parts_ok=True)
-            return ops.experts_finish(y, rt.normed_now(x) if own else None, shared, extra)
+            # (without a gate the shared expert is added as it is)
+            return ops.experts_finish(y, rt.normed_now(x) if own else None, shared, extra if own or self.shared_gate else None, plus)
 
     def forward_sorted(self, x, ids, weights):
         """A prompt: every expert's tokens as rows side by side, two library products an expert, the weighted sum in

@@ -213,6 +213,8 @@ class DecoderModel:
         for r in self.schedule:
             if not 0 <= r.layer < len(self.layers):
                 raise ConfigError(f"schedule names layer {r.layer}, the model has {len(self.layers)}")
+            if r.add_embedding and self.stream_kind is not None and self.stream_kind.kind != "residual":
+                raise ConfigError("the embedding's output is added again to a plain residual only")
         self.rt = None
 
     # ---- weights
@@ -272,8 +274,8 @@ class DecoderModel:
         h = self.embedding.plain(ctx)
         for run in self.schedule:
             entries = run.entries()
-            if len(entries) != 1:
-                raise ConfigError("the plain backend runs layers with one cache entry")
+            if len(entries) != 1 or run.add_embedding:
+                raise ConfigError("the plain backend runs layers with one cache entry and adds nothing between them")
             store, group = stores[entries[0]]
             h = self.layers[run.layer].plain(h, ctx, store, page_tables[group])
         return self.head.plain(self.final_norm.plain(h[ctx.want_rows]))
@@ -324,9 +326,17 @@ class DecoderModel:
             stream.links_ok = not rt.invariant
         else:
             stream = part_class("stream", self.stream_kind.kind)(hidden, **self.stream_kind.params)
+        embedded = None
+        if any(run.add_embedding for run in self.schedule):      # the residual is changed in place: later runs add a copy
+            embedded = torch.empty_like(hidden)
+            ops.gate_rows(embedded, 0, hidden, None, 0, 1.0)
         for at, run in enumerate(self.schedule):
             layer = self.layers[run.layer]
-            follower = self.layers[self.schedule[at + 1].layer] if at + 1 < len(self.schedule) else None
+            if run.add_embedding:
+                stream.add(embedded)
+            # (a run before which something is added reads another sum than this run's last product could prepare)
+            after = self.schedule[at + 1] if at + 1 < len(self.schedule) else None
+            follower = self.layers[after.layer] if after is not None and not after.add_embedding else None
             entry = getattr(follower, "entry_norm", None)
             stream.next_entry_norm = entry() if entry else None
             tiled = getattr(follower, "entry_takes_tiled", None)

@@ -26,26 +26,39 @@ class ParallelMixers(Mixer):
     projections each read a mix of their own) share the output product alone.  Other members run whole, and their float32
     results are added.
 
+    ``norms``: the checkpoint names of one gain of the model's width per member; each member's result then goes through an RMS
+    norm over that width (``eps``) before it is scaled and added.  The members keep output products of their own, and share the
+    input product where they all can (``in_matrix``, ``heads_from``: an attention of the fourth family, the delta rule with a decay
+    per channel).
+
     A member that keeps several things per sequence (a tuple of needs) gets its stores as a tuple; the layer's run names
     the members' entries one after the other.  A member that sets ``wants_residual`` also gets the float32 residual the
     layer hands over (``residual=``)."""
 
     wants_residual = True
 
-    def __init__(self, mixers: tuple, scales: tuple):
+    def __init__(self, mixers: tuple, scales: tuple, norms: tuple | None = None, hidden: int = 0, eps: float = 1e-6):
+        self.norms, self.hidden, self.eps = tuple(norms) if norms is not None else None, hidden, eps
+        if self.norms is not None and (len(self.norms) != len(mixers) or hidden < 1):
+            raise ConfigError(f"{len(self.norms)} norms over {hidden} elements for {len(mixers)} mixers side by side")
         if len(mixers) < 1 or len(mixers) != len(scales):
             raise ConfigError(f"{len(mixers)} mixers side by side with {len(scales)} constants")
         self.members = [build_part("mixer", m) for m in mixers]
         self.scales = tuple(float(s) for s in scales)
-        self.fused = all(hasattr(m, "core") and hasattr(m, "in_matrix") and hasattr(m, "out_matrix") and
+        self.fused = self.norms is None and all(hasattr(m, "core") and hasattr(m, "in_matrix") and hasattr(m, "out_matrix") and
                          (getattr(m, "paired", True)) for m in self.members)
         # members that write their heads into one row for one output product, each after input products of its own
-        self.shares_out = not self.fused and all(hasattr(m, "run_into") and hasattr(m, "out_matrix") for m in self.members)
+        self.shares_out = self.norms is None and not self.fused and all(hasattr(m, "run_into") and hasattr(m, "out_matrix") for m in self.members)
+        # members with a norm behind each: one input product for all that hand their heads over
+        self.shares_in = self.norms is not None and all(hasattr(m, "heads_from") and hasattr(m, "in_matrix") and (
+            getattr(m, "halved", False) or getattr(m, "per_channel", False)) for m in self.members)
 
     def tensors(self):
         t = {}
         for m in self.members:
             t.update(m.tensors())
+        if self.norms is not None:
+            t.update({name: TensorSpec((self.hidden,), GAIN) for name in self.norms})
         return t
 
     def bind(self, weights, rt):
@@ -59,6 +72,20 @@ class ParallelMixers(Mixer):
                 self.out_at.append(b)
                 b += m.out_width
             self.out_width = b
+            return
+        if self.norms is not None:
+            self.gains = [rt.place_gain(weights[name]) for name in self.norms]
+        if self.shares_in:
+            for m in self.members:
+                m.bind(weights, rt, alone=False)
+                m.w_o = rt.pack(rt.place_matrix(m.out_matrix(weights)), parts_ok=True)
+            rows, self.in_at, a = [], [], 0
+            for m in self.members:                       # every member's columns start on a multiple of 8 (zero rows between)
+                w = m.in_matrix(weights)
+                rows += [w, w.new_zeros((-w.shape[0] % 8, w.shape[1]))]
+                self.in_at.append(a)
+                a += w.shape[0] + rows[-1].shape[0]
+            self.w_in = rt.pack(rt.place_matrix(torch.cat(rows, 0)), always=True)
             return
         if not self.fused:
             for m in self.members:
@@ -108,6 +135,8 @@ class ParallelMixers(Mixer):
                 m.run_into(x, ctx, store, table, heads, b, scale, **extra(m))
             with profiler.section(profiler.OUT_PROJECTION):
                 return rt.linear_packed(heads, self.w_out, out_dtype=torch.float32, parts_ok=True)
+        if self.norms is not None:
+            return self.forward_normed(x, ctx, dealt, extra)
         if not self.fused:
             total = None
             for m, scale, (store, table) in zip(self.members, self.scales, dealt):
@@ -126,6 +155,24 @@ class ParallelMixers(Mixer):
             m.core(proj, a, ctx, store, table, heads, b, scale)
         with profiler.section(profiler.OUT_PROJECTION):
             return rt.linear_packed(heads, self.w_out, out_dtype=torch.float32, parts_ok=True)
+
+    def forward_normed(self, x, ctx, dealt, extra):
+        """The members' results, each through its own norm, times their constants, added: float32 ``[T, hidden]``."""
+        rt = self.rt
+        if self.shares_in:
+            with profiler.section(profiler.QKV_PROJECTION):
+                proj = ops.as_rows(rt.linear_packed(x, self.w_in))
+            results = []
+            for m, (store, table), a in zip(self.members, dealt, self.in_at):
+                heads = m.heads_from(x, proj, a, ctx, store, table)
+                with profiler.section(profiler.OUT_PROJECTION):
+                    results.append(rt.linear_packed(heads, m.w_o, out_dtype=torch.float32, parts_ok=True))
+        else:
+            results = [m.forward(x, ctx, store, table, **extra(m)) for m, (store, table) in zip(self.members, dealt)]
+            if any(isinstance(y, tuple) for y in results):
+                raise ConfigError("a mixer side by side with others hands back its result, not a link to a norm")
+        with profiler.section(profiler.NORM):
+            return ops.normed_sum([ops.as_rows(y) for y in results], self.gains, self.scales, self.eps)
 
 
 @register_part("arrangement", "norm_after")

@@ -21,11 +21,18 @@ class RotateHalf(PositionEncoding):
     64-bit and rounded once.  ``stretch = {factor, original, fast, slow}`` slows the pairs down for contexts ``factor`` times
     as long as ``original``: with ``i(t) = dims ln(original / (2 pi t)) / (2 ln theta)``, the place of a pair that turns ``t`` times
     in the original context, a pair's frequency runs from its own (``i <= floor(i(fast))``) to ``1/factor`` of it (``i >=
-    ceil(i(slow))``), linearly in ``i`` between; and ``amplitude = 0.1 ln(factor) + 1`` multiplies cosine and sine."""
+    ceil(i(slow))``), linearly in ``i`` between; and ``amplitude = 0.1 ln(factor) + 1`` multiplies cosine and sine.  ``factor``:
+    every pair's frequency is divided by it (linear scaling)."""
 
     amplitude = 1.0
 
-    def __init__(self, head_dim: int, theta: float, dims: int | None = None, stretch: dict | None = None):
+    def __init__(self, head_dim: int, theta: float, dims: int | None = None, stretch: dict | None = None,
+                 factor: float = 1.0):
+        if not factor > 0:
+            raise ConfigError(f"a rotation's frequencies divided by {factor}")
+        self.factor = float(factor)
+        if dims is None and self.factor != 1.0:
+            dims = head_dim
         if head_dim % 2 and dims is None:
             raise ConfigError(f"head_dim {head_dim} must be even for a rotation in pairs")
         if dims is not None and (dims % 2 or not 2 <= dims <= head_dim):
@@ -40,6 +47,7 @@ class RotateHalf(PositionEncoding):
         dims, base = self.dims, float(self.theta)
         i = torch.arange(dims // 2, dtype=torch.float64)
         f = torch.pow(torch.tensor(base, dtype=torch.float64), -2.0 * i / dims)
+        f = f / self.factor
         if self.stretch is None:
             return f
         s = self.stretch

@@ -62,9 +62,11 @@ class Run:
     reads what the earlier one wrote; its mixer must be one that does not write).
     A layer that keeps more than one thing per sequence (keys and values and a state
     of fixed size, or the caches of two mixers) names a tuple of entries, one for each
-    need its ``cache_need()`` lists, in that order."""
+    need its ``cache_need()`` lists, in that order.  ``add_embedding``: the embedding's output (the residual as it was before
+    the first layer) is added to the residual before this run."""
     layer: int
     cache: Union[None, int, Tuple[int, ...]] = None
+    add_embedding: bool = False
 
     def entries(self) -> Tuple[int, ...]:
         if self.cache is None:

@@ -32,6 +32,7 @@ class TensorSpec:
     shape: tuple               # a size of None is given by the file alone (a rank that no configuration key names)
     kind: str = MATRIX
     optional: bool = False     # absent is fine (e.g. lm_head.weight of a tied model)
+    below: int | None = None   # a table of choices: the entries of a row differ and lie in [0, below)
 
 
 _KEPT = (torch.bfloat16, torch.float32)

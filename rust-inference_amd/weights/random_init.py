@@ -34,6 +34,9 @@ def random_tensor(seed: int, name: str, spec: TensorSpec, dtype=torch.bfloat16, 
         raise ConfigError(f"{name}: a size that only a checkpoint gives ({list(spec.shape)}); a configuration that is to be "
                           "filled with random weights must name it (a gla mixer's 'rank')")
     g = _generator(seed, name, device)
+    if spec.kind == TABLE and spec.below is not None:           # a row of different entries: the first of a random order
+        order = torch.rand((spec.shape[0], spec.below), generator=g, device=device).argsort(dim=1)
+        return order[:, :spec.shape[1]].to(torch.int32).contiguous()
     if spec.kind == TABLE:
         return torch.zeros(spec.shape, dtype=torch.int32, device=device)
     x = torch.randn(spec.shape, generator=g, dtype=torch.float32, device=device)
