@@ -2,7 +2,7 @@
 """Decode and prefill throughput of the Qwen3-8B-shaped model on one MI355X.
 
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--layers L] [--batch B] [--context C] [--model 8b|0.6b|1.7b|4b|14b|32b]
-    python bench.py --design zidepel|pisulorn|zakelorn|dagezen|notadra [--size 0.6b|8b] [--layers L]      # another workload: see design_comparison below
+    python bench.py --design zidepel|pisulorn|zakelorn|dagezen|notadra|kisepel [--size 0.6b|8b] [--layers L]      # another workload: see design_comparison below
 
 The default run has the layer sizes of Qwen3-8B with random weights
 (N(0, 0.02), norm gains 1 + N(0, 0.1), seed 2), a batch of 8 and prompts of 2,048 tokens in a
@@ -284,6 +284,32 @@ def notadra_like(q, layers, vocab, context, vdim=None):
                        for i in range(layers)]}
 
 
+def kisepel_like(q, layers, vocab, context):
+    """A Kisepel configuration with the layer sizes of a Qwen3 one: the same width; of every four layers the first is a
+    state-space mixer with Qwen3's heads and head size, a state of one head size, its key heads as groups and four taps; the
+    second and the fourth are softmax attention in chunks of 1,024 tokens with Qwen3's heads and head size beside the delta rule
+    with a quarter as many heads of the same size and a middle of one head size; the third is linear attention with Qwen3's heads
+    and no feed-forward; the others have eight experts of half Qwen3's width, two a token, and a shared expert of a quarter of it
+    (the experts of the Zakelorn model)."""
+    d, h, g, dh, ff = q["hidden_size"], q["num_attention_heads"], q["num_key_value_heads"], q["head_dim"], q["intermediate_size"]
+    moe = {"kind": "moe", "expert": {"ff": ff // 2}, "shared": {"ff": ff // 4}, "router": {"experts": 8, "top": 2}}
+    ssm = {"type": "mamba2", "mlp": moe,
+           "mixer": {"heads": h, "vdim": dh, "state": dh, "groups": g, "conv": 4, "norm_groups": g}}
+    par = {"type": "parallel", "mlp": moe,
+           "mixer": {"left": {"heads": h, "kv_heads": g, "dim": dh, "vdim": dh, "scale": dh ** -0.5, "mask": {"size": 1024},
+                              "rot": {"dims": dh, "base": 1e6, "scaling": {"factor": 4.0}}},
+                     "right": {"heads": max(1, h // 4), "kv_heads": max(1, h // 4), "dim": dh, "vdim": dh, "conv": 4, "rank": dh}}}
+    lin = {"type": "lightning", "mlp": None,
+           "mixer": {"heads": h, "dim": dh, "vdim": dh, "decay": [1.0 - 2.0 ** -(3 + 5 * i / max(1, h - 1)) for i in range(h)]}}
+    return {"architecture": "Kisepel", "vocab": vocab, "width": d, "norm": {"eps": 1e-5}, "embedding": {"scale": 8.0},
+            "logit_scale": 0.5, "layers": [(ssm, par, lin, par)[i % 4] for i in range(layers)]}
+
+
+# What is measured beside a design, and which of them it is compared with in the line's `vs_...` key.
+BESIDE = {"notadra": ("qwen3", "zakelorn", "notadra", "notadra_vdim_5_4"),
+          "kisepel": ("qwen3", "pisulorn", "zakelorn", "dagezen", "kisepel")}
+
+
 def design_comparison(args) -> int:
     """`--design zidepel`, `--design pisulorn` or `--design zakelorn`: prefill and decode of a model of that design beside the Qwen3 model
     of the same layer sizes (and, for Pisulorn, beside the Zidepel model of those sizes, the design closest to it)
@@ -291,17 +317,24 @@ def design_comparison(args) -> int:
     the output matrix are what is timed).  One JSON line; the default workload and its line are not touched."""
     sizes = {"0.6b": QWEN3_0_6B, "8b": QWEN3_8B}
     layers, vocab, context = args.layers or 8, 32768, args.context
-    if args.design == "notadra":
-        out = {"metric": "prefill and decode of the Notadra design beside Zakelorn and Qwen3 at equal layer sizes", "unit": "tok/s",
+    if args.design in BESIDE:
+        own = args.design
+        others = "Zakelorn and Qwen3" if own == "notadra" else "Dagezen, Zakelorn, Pisulorn and Qwen3"
+        out = {"metric": f"prefill and decode of the {own.capitalize()} design beside {others} at equal layer sizes", "unit": "tok/s",
                "n_gpus": 1, "dtype": "bf16", "data": "synthetic: random weights, uniform random token ids", "layers": layers,
                "vocab": vocab, "steps": args.steps, "warmup": args.warmup, "sizes": {}}
         for size in ([args.size] if args.size else ["0.6b", "8b"]):
             q = dict(sizes[size], num_hidden_layers=layers, vocab_size=vocab, max_position_embeddings=context,
                      tie_word_embeddings=False)
             got = {}
-            for name, cfg in (("qwen3", q), ("zakelorn", zakelorn_like(q, layers, vocab, context)),
-                              ("notadra", notadra_like(q, layers, vocab, context)),
-                              ("notadra_vdim_5_4", notadra_like(q, layers, vocab, context, q["head_dim"] * 5 // 4))):
+            shapes = {"qwen3": lambda: q, "pisulorn": lambda: pisulorn_like(q, layers, vocab, context),
+                      "zakelorn": lambda: zakelorn_like(q, layers, vocab, context),
+                      "dagezen": lambda: dagezen_like(q, layers, vocab, context),
+                      "notadra": lambda: notadra_like(q, layers, vocab, context),
+                      "notadra_vdim_5_4": lambda: notadra_like(q, layers, vocab, context, q["head_dim"] * 5 // 4),
+                      "kisepel": lambda: kisepel_like(q, layers, vocab, context)}
+            for name in BESIDE[own]:
+                cfg = shapes[name]()
                 if args.only and name != args.only:
                     continue
                 b = ShapeBench(f"{name} at Qwen3-{size} layer sizes", cfg, vocab, 11, context, not args.no_graphs)
@@ -309,10 +342,10 @@ def design_comparison(args) -> int:
                 b.close()
             out["sizes"][size] = got
         first = out["sizes"][next(iter(out["sizes"]))]
-        if "notadra" in first:
-            out["value"], out["higher_is_better"] = first["notadra"]["decode_b8"]["tok_s"], True
-        if "notadra" in first and "zakelorn" in first:
-            out["vs_zakelorn_decode_b8"] = round(first["notadra"]["decode_b8"]["tok_s"] / first["zakelorn"]["decode_b8"]["tok_s"], 3)
+        if own in first:
+            out["value"], out["higher_is_better"] = first[own]["decode_b8"]["tok_s"], True
+        if own in first and "zakelorn" in first:
+            out["vs_zakelorn_decode_b8"] = round(first[own]["decode_b8"]["tok_s"] / first["zakelorn"]["decode_b8"]["tok_s"], 3)
         print(json.dumps(out))
         return 0
     if args.design == "dagezen":
@@ -409,10 +442,10 @@ def main() -> int:
     ap.add_argument("--no-points", action="store_true", help="skip the batch 1 and 64 points and the other models")
     ap.add_argument("--no-other-models", action="store_true", help="skip the Qwen3-0.6B and Qwen3-32B points")
     ap.add_argument("--no-graphs", action="store_true", help="launch every kernel of a decode step from the host")
-    ap.add_argument("--design", choices=["zidepel", "pisulorn", "zakelorn", "dagezen", "notadra"], default=None,
+    ap.add_argument("--design", choices=["zidepel", "pisulorn", "zakelorn", "dagezen", "notadra", "kisepel"], default=None,
                     help="another workload: this design beside Qwen3 at equal layer sizes (prefill, decode at batch 1, 8, 32)")
     ap.add_argument("--size", choices=["0.6b", "8b"], default=None, help="with --design: one of the two layer sizes only")
-    ap.add_argument("--only", default=None, help="with --design dagezen or notadra: one of the models only (qwen3, zakelorn, dagezen, notadra, notadra_vdim_5_4)")
+    ap.add_argument("--only", default=None, help="with --design dagezen, notadra or kisepel: one of the models measured only (qwen3, zakelorn, dagezen, ...)")
     args = ap.parse_args()
     if args.gpus != 1:
         print(f"bench.py measures one GPU: this library is single-GPU, --gpus {args.gpus} is not run")

@@ -517,6 +517,12 @@ int ri_attention_decode_padded_bf16(void* out, float* workspace, const void* qkv
                                     int window, int chunk, float scale, float softcap, const float* slopes, int tiled_out,
                                     int keep_first, const float* sinks, void* stream);
 
+// ri_add_rmsnorm for n results that wait (parts: n host-side addresses of [total rows, dim] float32), added in their order.
+int ri_add_branches_rmsnorm(void* out, int out_dtype, float* residual, const void* const* parts, int n, const float* gain, float eps,
+                            const int32_t* rows, int n_rows, int dim, void* stream);
+// out [rows, width] = x[:, col .. col + width] of rows of `row` elements.
+int ri_take_columns(void* out, const void* x, int dtype, int row, int col, int width, int rows, void* stream);
+
 // out (+)= a_scale * norm(a) * a_gain + b_scale * norm(b) * b_gain, row by row: RMS norms over `dim` of products' results a and b
 // ([parts, rows, dim] float32, added in order, or one part of either format; b may be NULL); out float32 [rows, dim].
 int ri_normed_sum(float* out, int accumulate, const void* a, int a_dtype, int a_parts, const float* a_gain, float a_scale,

@@ -481,54 +481,73 @@ extern "C" int ri_row_norm_gate(void* out, int out_stride, int out_off, const fl
 // ------------------------------------------------------------------ normed results of mixers side by side, added
 // out (+)= a_scale * rms_norm(a) * a_gain + b_scale * rms_norm(b) * b_gain: a and b are the results of two output products,
 // each [parts, rows, dim] (the parts added in order) or one part in the activations' format; b may be absent.
-template <typename T>
-__device__ __forceinline__ float4 parts4(const T* x, int parts, size_t stride, size_t at) {
-    float4 v = ld4(x + at);
-    for (int p = 1; p < parts; ++p) {
-        const float4 w = ld4(x + p * stride + at);
-        v = make_float4(v.x + w.x, v.y + w.y, v.z + w.z, v.w + w.w);
+// (four parts are asked for together, each from an address that exists, and added in their order)
+template <typename T, int VPT>
+__device__ __forceinline__ void parts4(float4 (&v)[VPT], const T* x, int parts, size_t stride, size_t row, const int (&at)[VPT]) {
+    for (int q0 = 0; q0 < parts; q0 += 4) {
+        float4 p[4][VPT];
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+#pragma unroll
+            for (int i = 0; i < VPT; ++i) p[j][i] = ld4(x + (size_t)min(q0 + j, parts - 1) * stride + row + at[i]);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            const bool live = q0 + j < parts;
+#pragma unroll
+            for (int i = 0; i < VPT; ++i) {
+                v[i].x = live ? v[i].x + p[j][i].x : v[i].x;
+                v[i].y = live ? v[i].y + p[j][i].y : v[i].y;
+                v[i].z = live ? v[i].z + p[j][i].z : v[i].z;
+                v[i].w = live ? v[i].w + p[j][i].w : v[i].w;
+            }
+        }
     }
-    return v;
 }
 
-// Rows of up to 1,024 VPT elements in a multiple of 4: both rows in registers, one trip; one workgroup a row.
-template <typename TX, typename TY, int VPT>
-__global__ void __launch_bounds__(256)
+// Rows of up to 4 THREADS VPT elements in a multiple of 4: both rows in registers, one trip; one workgroup a row, whose threads
+// depend on the width alone.
+template <typename TX, typename TY, int VPT, int THREADS>
+__global__ void __launch_bounds__(THREADS)
 normed_sum_vec_kernel(float* __restrict__ out, int accumulate, const TX* __restrict__ a, int a_parts, const float* __restrict__ a_gain,
                       float a_scale, const TY* __restrict__ b, int b_parts, const float* __restrict__ b_gain, float b_scale,
                       float eps, size_t stride, int dim) {
     __shared__ float scratch[16];
     const size_t t = (size_t)blockIdx.x * dim;
-    float4 va[VPT], vb[VPT];
+    float4 va[VPT], vb[VPT], ga[VPT], gb[VPT];
+    int at[VPT];
+    bool ok[VPT];
+    const float* b_gain_there = b ? b_gain : a_gain;
+#pragma unroll
+    for (int i = 0; i < VPT; ++i) {
+        const int c = (threadIdx.x + i * THREADS) * 4;
+        ok[i] = c < dim;
+        at[i] = ok[i] ? c : 0;
+        va[i] = vb[i] = make_float4(0.f, 0.f, 0.f, 0.f);
+        ga[i] = ld4(a_gain + at[i]);
+        gb[i] = ld4(b_gain_there + at[i]);
+    }
+    parts4<TX, VPT>(va, a, a_parts, stride, t, at);
+    if (b) parts4<TY, VPT>(vb, b, b_parts, stride, t, at);
     float sa = 0.f, sb = 0.f;
 #pragma unroll
     for (int i = 0; i < VPT; ++i) {
-        const int c = (threadIdx.x + i * 256) * 4;
-        const bool ok = c < dim;
-        va[i] = parts4(a, a_parts, stride, t + (ok ? c : 0));
-        vb[i] = b ? parts4(b, b_parts, stride, t + (ok ? c : 0)) : make_float4(0.f, 0.f, 0.f, 0.f);
-        if (ok) {
-            sa += (va[i].x * va[i].x + va[i].y * va[i].y) + (va[i].z * va[i].z + va[i].w * va[i].w);
-            sb += (vb[i].x * vb[i].x + vb[i].y * vb[i].y) + (vb[i].z * vb[i].z + vb[i].w * vb[i].w);
-        }
+        if (!ok[i]) continue;
+        sa += (va[i].x * va[i].x + va[i].y * va[i].y) + (va[i].z * va[i].z + va[i].w * va[i].w);
+        sb += (vb[i].x * vb[i].x + vb[i].y * vb[i].y) + (vb[i].z * vb[i].z + vb[i].w * vb[i].w);
     }
     const float fa = a_scale / sqrtf(block_sum(sa, scratch) / (float)dim + eps);
     const float fb = b ? b_scale / sqrtf(block_sum(sb, scratch) / (float)dim + eps) : 0.f;
 #pragma unroll
     for (int i = 0; i < VPT; ++i) {
-        const int c = (threadIdx.x + i * 256) * 4;
-        if (c >= dim) continue;
-        const float4 g = ld4(a_gain + c);
-        float4 v = make_float4(fa * va[i].x * g.x, fa * va[i].y * g.y, fa * va[i].z * g.z, fa * va[i].w * g.w);
-        if (b) {
-            const float4 h = ld4(b_gain + c);
-            v = make_float4(v.x + fb * vb[i].x * h.x, v.y + fb * vb[i].y * h.y, v.z + fb * vb[i].z * h.z, v.w + fb * vb[i].w * h.w);
-        }
+        if (!ok[i]) continue;
+        float4 v = make_float4(fa * va[i].x * ga[i].x, fa * va[i].y * ga[i].y, fa * va[i].z * ga[i].z, fa * va[i].w * ga[i].w);
+        if (b) v = make_float4(v.x + fb * vb[i].x * gb[i].x, v.y + fb * vb[i].y * gb[i].y, v.z + fb * vb[i].z * gb[i].z,
+                               v.w + fb * vb[i].w * gb[i].w);
         if (accumulate) {
-            const float4 o = ld4(out + t + c);
+            const float4 o = ld4(out + t + at[i]);
             v = make_float4(v.x + o.x, v.y + o.y, v.z + o.z, v.w + o.w);
         }
-        st4(out + t + c, v);
+        st4(out + t + at[i], v);
     }
 }
 
@@ -571,9 +590,12 @@ extern "C" int ri_normed_sum(float* out, int accumulate, const void* a, int a_dt
     hipStream_t s = (hipStream_t)stream;
     const size_t stride = (size_t)rows * dim;
     const bool vec = dim % 4 == 0 && dim <= 8192;
-    const int vpt = (dim / 4 + 255) / 256;
 #define RI_ARGS(TX, TY) out, accumulate, (const TX*)a, a_parts, a_gain, a_scale, (const TY*)b, b_parts, b_gain, b_scale, eps, stride, dim
-#define RI_GO(TX, TY)                                                                                       if (!vec) normed_sum_kernel<TX, TY><<<rows, 256, 0, s>>>(RI_ARGS(TX, TY));                              else if (vpt <= 1) normed_sum_vec_kernel<TX, TY, 1><<<rows, 256, 0, s>>>(RI_ARGS(TX, TY));              else if (vpt <= 2) normed_sum_vec_kernel<TX, TY, 2><<<rows, 256, 0, s>>>(RI_ARGS(TX, TY));              else if (vpt <= 4) normed_sum_vec_kernel<TX, TY, 4><<<rows, 256, 0, s>>>(RI_ARGS(TX, TY));              else normed_sum_vec_kernel<TX, TY, 8><<<rows, 256, 0, s>>>(RI_ARGS(TX, TY))
+#define RI_GO(TX, TY)                                                                                       if (!vec) normed_sum_kernel<TX, TY><<<rows, 256, 0, s>>>(RI_ARGS(TX, TY));                               \
+    else if (dim <= 1024) normed_sum_vec_kernel<TX, TY, 1, 256><<<rows, 256, 0, s>>>(RI_ARGS(TX, TY));       \
+    else if (dim <= 2048) normed_sum_vec_kernel<TX, TY, 1, 512><<<rows, 512, 0, s>>>(RI_ARGS(TX, TY));       \
+    else if (dim <= 4096) normed_sum_vec_kernel<TX, TY, 1, 1024><<<rows, 1024, 0, s>>>(RI_ARGS(TX, TY));     \
+    else normed_sum_vec_kernel<TX, TY, 2, 1024><<<rows, 1024, 0, s>>>(RI_ARGS(TX, TY))
     if (a_dtype == RI_F32) { if (!b || b_dtype == RI_F32) { RI_GO(float, float); } else { RI_GO(float, bf16_t); } }
     else                   { if (!b || b_dtype == RI_F32) { RI_GO(bf16_t, float); } else { RI_GO(bf16_t, bf16_t); } }
 #undef RI_GO

@@ -443,7 +443,7 @@ template <typename TX, typename TS>
 __global__ void __launch_bounds__(256)
 experts_finish_kernel(float* __restrict__ out, const float* __restrict__ routed, int parts, size_t part_stride,
                       const TX* __restrict__ x, const TS* __restrict__ shared, int shared_parts,
-                      const float* __restrict__ extra, const float* __restrict__ plus, int plus_parts, int dim) {
+                      const float* __restrict__ extra, int dim) {
     const size_t at = (size_t)blockIdx.x * dim;
     const float own = extra ? extra[(size_t)blockIdx.x * 2] : 1.f, gate = extra ? extra[(size_t)blockIdx.x * 2 + 1] : 1.f;
     for (int d = threadIdx.x; d < dim; d += blockDim.x) {
@@ -455,7 +455,6 @@ experts_finish_kernel(float* __restrict__ out, const float* __restrict__ routed,
             for (int p = 1; p < shared_parts; ++p) sv += to_f32(shared[p * part_stride + at + d]);
             v += gate * sv;
         }
-        for (int p = 0; p < plus_parts; ++p) v += plus[p * part_stride + at + d];
         out[at + d] = v;
     }
 }
@@ -473,7 +472,7 @@ template <typename TX, typename TS>
 __global__ void __launch_bounds__(256)
 experts_finish_vec_kernel(float* __restrict__ out, const float* __restrict__ routed, int parts, size_t part_stride,
                           const TX* __restrict__ x, const TS* __restrict__ shared, int shared_parts,
-                          const float* __restrict__ extra, const float* __restrict__ plus, int plus_parts, int dim) {
+                          const float* __restrict__ extra, int dim) {
     const int d = (blockIdx.y * 256 + threadIdx.x) * 4;
     if (d >= dim) return;
     const size_t at = (size_t)blockIdx.x * dim + d;
@@ -495,17 +494,11 @@ experts_finish_vec_kernel(float* __restrict__ out, const float* __restrict__ rou
         }
         v = make_float4(v.x + gate * sv.x, v.y + gate * sv.y, v.z + gate * sv.z, v.w + gate * sv.w);
     }
-    for (int p = 0; p < plus_parts; ++p) {
-        const float4 w = fin_ld4(plus + p * part_stride + at);
-        v = make_float4(v.x + w.x, v.y + w.y, v.z + w.z, v.w + w.w);
-    }
     *reinterpret_cast<float4*>(out + at) = v;
 }
 
 extern "C" int ri_experts_finish(float* out, const float* routed, int parts, const void* x, int x_dtype, const void* shared,
-                                 int shared_dtype, int shared_parts, const float* extra, const float* plus, int plus_parts,
-                                 int tokens, int dim, void* stream) {
-    RI_REQUIRE(plus_parts >= 0 && (plus_parts == 0 || plus), "experts_finish: %d more parts", plus_parts);
+                                 int shared_dtype, int shared_parts, const float* extra, int tokens, int dim, void* stream) {
     RI_REQUIRE(tokens > 0 && dim > 0 && parts >= 1 && shared_parts >= 1 && (extra || !x) && routed, "experts_finish: %d tokens of %d", tokens, dim);
     RI_REQUIRE((x_dtype == RI_F32 || x_dtype == RI_BF16) && (shared_dtype == RI_F32 || shared_dtype == RI_BF16),
                "experts_finish: dtypes %d and %d", x_dtype, shared_dtype);
@@ -516,10 +509,10 @@ extern "C" int ri_experts_finish(float* out, const float* routed, int parts, con
 #define RI_GO(TX, TS)                                                                                                   \
     if (dim % 4 == 0 && vgrid.y <= 65535)                                                                               \
         experts_finish_vec_kernel<TX, TS><<<vgrid, 256, 0, s>>>(out, routed, parts, stride, (const TX*)x,                 \
-                                                                (const TS*)shared, shared_parts, extra, plus, plus_parts, dim);            \
+                                                                (const TS*)shared, shared_parts, extra, dim);            \
     else                                                                                                                \
         experts_finish_kernel<TX, TS><<<tokens, 256, 0, s>>>(out, routed, parts, stride, (const TX*)x,                    \
-                                                             (const TS*)shared, shared_parts, extra, plus, plus_parts, dim)
+                                                             (const TS*)shared, shared_parts, extra, dim)
     if (x_dtype == RI_F32) { if (shared_dtype == RI_F32) RI_GO(float, float); else RI_GO(float, bf16_t); }
     else                   { if (shared_dtype == RI_F32) RI_GO(bf16_t, float); else RI_GO(bf16_t, bf16_t); }
 #undef RI_GO

@@ -201,6 +201,155 @@ extern "C" int ri_add_rmsnorm(void* out, int out_dtype, float* residual, const v
     return 0;
 }
 
+// The same for several results that wait to be added, up to BRANCH_PARTS parts of products in all, at addresses of their own:
+// the sum is taken in the order of the list.  The threads of a row depend on its width alone, so a row's sums do too.
+#define BRANCH_PARTS 32
+struct BranchParts {
+    const float* at[BRANCH_PARTS];
+    int n;
+};
+
+template <typename TO, int VPT, int THREADS>
+__global__ void __launch_bounds__(THREADS)
+add_branches_rmsnorm_vec_kernel(TO* __restrict__ out, float* __restrict__ residual, BranchParts parts,
+                                const float* __restrict__ gain, float eps, const int32_t* __restrict__ rows, int dim) {
+    __shared__ float scratch[16];
+    constexpr int PQ = 4;
+    const int row = blockIdx.x;
+    const size_t src = (size_t)(rows ? rows[row] : row) * dim;
+    float4 v[VPT], g[VPT];
+    int at[VPT];
+    bool ok[VPT];
+#pragma unroll
+    for (int i = 0; i < VPT; ++i) {
+        const int d = (i * THREADS + threadIdx.x) * 4;
+        ok[i] = d < dim;
+        at[i] = ok[i] ? d : 0;
+        v[i] = load4(residual + src + at[i]);
+        g[i] = load4(gain + at[i]);
+    }
+    for (int q0 = 0; q0 < parts.n; q0 += PQ) {
+        float4 p[PQ][VPT];
+#pragma unroll
+        for (int j = 0; j < PQ; ++j) {
+            const float* from = parts.at[min(q0 + j, parts.n - 1)] + src;
+#pragma unroll
+            for (int i = 0; i < VPT; ++i) p[j][i] = load4(from + at[i]);
+        }
+#pragma unroll
+        for (int j = 0; j < PQ; ++j) {
+            const bool live = q0 + j < parts.n;
+#pragma unroll
+            for (int i = 0; i < VPT; ++i) {
+                v[i].x = live ? v[i].x + p[j][i].x : v[i].x;
+                v[i].y = live ? v[i].y + p[j][i].y : v[i].y;
+                v[i].z = live ? v[i].z + p[j][i].z : v[i].z;
+                v[i].w = live ? v[i].w + p[j][i].w : v[i].w;
+            }
+        }
+    }
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < VPT; ++i) {
+        if (ok[i]) {
+            if (!rows) store4(residual + src + at[i], v[i]);
+            ss += v[i].x * v[i].x + v[i].y * v[i].y + v[i].z * v[i].z + v[i].w * v[i].w;
+        }
+    }
+    const float inv = 1.0f / sqrtf(block_sum(ss, scratch) / (float)dim + eps);
+#pragma unroll
+    for (int i = 0; i < VPT; ++i)
+        if (ok[i])
+            store4(out + (size_t)row * dim + at[i], make_float4(v[i].x * inv * g[i].x, v[i].y * inv * g[i].y, v[i].z * inv * g[i].z,
+                                                                v[i].w * inv * g[i].w));
+}
+
+template <typename TO>
+__global__ void __launch_bounds__(256)
+add_branches_rmsnorm_kernel(TO* __restrict__ out, float* __restrict__ residual, BranchParts parts, const float* __restrict__ gain,
+                            float eps, const int32_t* __restrict__ rows, int dim) {
+    __shared__ float scratch[16];
+    const int row = blockIdx.x;
+    const size_t src = (size_t)(rows ? rows[row] : row) * dim;
+    auto sum = [&](int d) {
+        float v = residual[src + d];
+        for (int p = 0; p < parts.n; ++p) v += parts.at[p][src + d];
+        return v;
+    };
+    float ss = 0.f;
+    for (int d = threadIdx.x; d < dim; d += blockDim.x) {
+        const float v = sum(d);
+        ss += v * v;
+    }
+    const float inv = 1.0f / sqrtf(block_sum(ss, scratch) / (float)dim + eps);
+    for (int d = threadIdx.x; d < dim; d += blockDim.x) {
+        const float v = sum(d);
+        if (!rows) residual[src + d] = v;                  // (read and written by this thread alone)
+        from_f32(out + (size_t)row * dim + d, v * inv * gain[d]);
+    }
+}
+
+template <typename TO>
+static void launch_add_branches(TO* out, float* residual, const BranchParts& parts, const float* gain, float eps, const int32_t* rows,
+                                int n_rows, int dim, hipStream_t s) {
+    if (dim % 4 || dim > 8192)
+        add_branches_rmsnorm_kernel<TO><<<n_rows, 256, 0, s>>>(out, residual, parts, gain, eps, rows, dim);
+    else if (dim <= 1024)
+        add_branches_rmsnorm_vec_kernel<TO, 1, 256><<<n_rows, 256, 0, s>>>(out, residual, parts, gain, eps, rows, dim);
+    else if (dim <= 2048)
+        add_branches_rmsnorm_vec_kernel<TO, 1, 512><<<n_rows, 512, 0, s>>>(out, residual, parts, gain, eps, rows, dim);
+    else if (dim <= 4096)
+        add_branches_rmsnorm_vec_kernel<TO, 1, 1024><<<n_rows, 1024, 0, s>>>(out, residual, parts, gain, eps, rows, dim);
+    else
+        add_branches_rmsnorm_vec_kernel<TO, 2, 1024><<<n_rows, 1024, 0, s>>>(out, residual, parts, gain, eps, rows, dim);
+}
+
+// parts: n addresses in host memory, each of [total rows, dim] float32.
+extern "C" int ri_add_branches_rmsnorm(void* out, int out_dtype, float* residual, const void* const* parts, int n, const float* gain,
+                                       float eps, const int32_t* rows, int n_rows, int dim, void* stream) {
+    RI_REQUIRE(n_rows > 0 && dim > 0 && n >= 1 && n <= BRANCH_PARTS && parts, "add_branches_rmsnorm: %d parts, %d rows of %d", n, n_rows, dim);
+    RI_REQUIRE(out_dtype == RI_F32 || out_dtype == RI_BF16, "add_branches_rmsnorm: out dtype %d", out_dtype);
+    BranchParts list = {};
+    list.n = n;
+    for (int i = 0; i < n; ++i) list.at[i] = (const float*)parts[i];
+    for (int i = n; i < BRANCH_PARTS; ++i) list.at[i] = list.at[0];
+    if (out_dtype == RI_F32)
+        launch_add_branches<float>((float*)out, residual, list, gain, eps, rows, n_rows, dim, (hipStream_t)stream);
+    else
+        launch_add_branches<bf16_t>((bf16_t*)out, residual, list, gain, eps, rows, n_rows, dim, (hipStream_t)stream);
+    RI_LAUNCH_CHECK("add_branches_rmsnorm");
+    return 0;
+}
+
+// Columns of wider rows as rows of their own: 16 bytes a thread where everything is a multiple of that, else an element.
+template <typename U>
+__global__ void __launch_bounds__(256)
+take_columns_kernel(U* __restrict__ out, const U* __restrict__ x, int row, int col, int width, long total) {
+    const long e = (long)blockIdx.x * 256 + threadIdx.x;
+    if (e >= total) return;
+    const long t = e / width;
+    out[e] = x[t * row + col + (e - t * width)];
+}
+
+extern "C" int ri_take_columns(void* out, const void* x, int dtype, int row, int col, int width, int rows, void* stream) {
+    RI_REQUIRE(rows > 0 && width > 0 && col >= 0 && col + (long)width <= row, "take_columns: columns %d ..+%d of %d rows of %d", col, width,
+               rows, row);
+    RI_REQUIRE(dtype == RI_F32 || dtype == RI_BF16, "take_columns: dtype %d", dtype);
+    const int unit = dtype == RI_F32 ? 4 : 8;
+    hipStream_t s = (hipStream_t)stream;
+    const bool pieces = (row | col | width) % unit == 0 && ((uintptr_t)out | (uintptr_t)x) % 16 == 0;
+    const long total = (long)rows * (pieces ? width / unit : width), blocks = (total + 255) / 256;
+    RI_REQUIRE(blocks <= 2147483647L, "take_columns: %ld elements exceed one launch", total);
+    if (pieces)
+        take_columns_kernel<uint4><<<(unsigned)blocks, 256, 0, s>>>((uint4*)out, (const uint4*)x, row / unit, col / unit, width / unit, total);
+    else if (dtype == RI_F32)
+        take_columns_kernel<float><<<(unsigned)blocks, 256, 0, s>>>((float*)out, (const float*)x, row, col, width, total);
+    else
+        take_columns_kernel<bf16_t><<<(unsigned)blocks, 256, 0, s>>>((bf16_t*)out, (const bf16_t*)x, row, col, width, total);
+    RI_LAUNCH_CHECK("take_columns");
+    return 0;
+}
+
 // (out may be residual itself when rows is NULL: every element is read and then written by one thread)
 template <typename TP>
 __global__ void add_rows_kernel(float* out, const float* residual,

@@ -134,6 +134,8 @@ _SIGNATURES = {
                                  c_int, c_int, c_int, c_int, c_int, c_int, c_void_p],
     "ri_experts_few_tokens_plain": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int,
                                     c_int, c_int, c_int, c_void_p],
+    "ri_add_branches_rmsnorm": [c_void_p, c_int, c_void_p, c_void_p, c_int, c_void_p, c_float, c_void_p, c_int, c_int, c_void_p],
+    "ri_take_columns": [c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p],
     "ri_head_norm_gate": [c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p, c_float, c_int, c_int, c_int, c_int,
                           c_void_p],
     "ri_normed_sum": [c_void_p, c_int, c_void_p, c_int, c_int, c_void_p, c_float, c_void_p, c_int, c_int, c_void_p, c_float, c_float,
@@ -154,7 +156,7 @@ _SIGNATURES = {
     "ri_experts_route_general": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_int,
                                  c_int, c_int, c_int, c_int, c_int, c_int, c_void_p],
     "ri_experts_activate_strided": [c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_int, c_float, c_void_p],
-    "ri_experts_finish": [c_void_p, c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_int, c_void_p, c_void_p, c_int, c_int, c_int,
+    "ri_experts_finish": [c_void_p, c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_int, c_void_p, c_int, c_int,
                           c_void_p],
     "ri_scaled_sum_norm": [c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_void_p, c_float, c_void_p, c_void_p, c_float,
                            c_int, c_int, c_int, c_void_p],
@@ -372,6 +374,38 @@ def add_rmsnorm(residual: torch.Tensor, pending, gain: torch.Tensor, eps: float,
           _opt(pending, "pending"), code(pending.dtype) if pending is not None else F32, parts, t,
           _dev(gain, "gain", torch.float32, (dim,)), float(eps), _opt(rows, "rows", torch.int32), n, dim, int(tiled),
           _stream())
+    return out
+
+
+MAX_BRANCH_PARTS = 32
+
+
+def add_branches_rmsnorm(residual: torch.Tensor, branches, gain: torch.Tensor, eps: float, out_dtype,
+                         rows: torch.Tensor | None = None) -> torch.Tensor:
+    """``add_rmsnorm`` for several results that wait to be added: float32 tensors ``[T, dim]`` or ``[parts, T, dim]``, up to
+    ``MAX_BRANCH_PARTS`` parts in all, added one after the other."""
+    t, dim = residual.shape
+    n = t if rows is None else rows.shape[0]
+    at = []
+    for y in branches:
+        base = _dev(y, "branch", torch.float32, (*y.shape[:-2], t, dim))
+        at += [base + 4 * t * dim * i for i in range(y.shape[0] if y.dim() == 3 else 1)]
+    if not 1 <= len(at) <= MAX_BRANCH_PARTS:
+        raise ShapeError(f"{len(at)} parts of branches: the kernel adds 1 to {MAX_BRANCH_PARTS}")
+    out = torch.empty((n, dim), dtype=out_dtype, device=residual.device)
+    _call("ri_add_branches_rmsnorm", _dev(out, "out"), code(out_dtype), _dev(residual, "residual", torch.float32),
+          (c_void_p * len(at))(*at), len(at), _dev(gain, "gain", torch.float32, (dim,)), float(eps),
+          _opt(rows, "rows", torch.int32), n, dim, _stream())
+    return out
+
+
+def take_columns(x: torch.Tensor, col: int, width: int) -> torch.Tensor:
+    """The columns ``col .. col + width`` of ``x [T, row]`` as rows of their own."""
+    tokens, row = x.shape
+    if col < 0 or width < 1 or col + width > row:
+        raise ShapeError(f"columns {col} ..+{width} of rows of {row}")
+    out = torch.empty((tokens, width), dtype=x.dtype, device=x.device)
+    _call("ri_take_columns", _dev(out, "out"), _dev(x, "x"), code(x.dtype), row, int(col), int(width), tokens, _stream())
     return out
 
 
@@ -892,7 +926,7 @@ def delta_prepare_channels(proj, q_off: int, taps, tails, z, mid, b_off: int, a_
                            heads: int, kv_heads: int, dim: int, vdim: int):
     """``delta_prepare`` for a decay per head and key channel: ``z [T, >= heads * dim]`` float32 are the decays'
     pre-activations, ``g = exp(-exp(a_log_h) softplus(z + dt_bias))`` with ``dt_bias [heads * dim]``; the logits of beta are the
-    columns ``b_off ..`` of ``mid`` (in the format of ``proj``).  ``gates`` is ``[T, heads * dim + heads]``."""
+    columns ``b_off ..`` of ``mid`` (in the format of ``proj``, or ``proj`` itself).  ``gates`` is ``[T, heads * dim + heads]``."""
     tokens, row = proj.shape
     seqs, channels, ntaps = slots.shape[0], 2 * kv_heads * dim + heads * vdim, taps.shape[1]
     _check_delta(tails, None, ntaps, channels, heads, dim, vdim)
@@ -978,18 +1012,17 @@ def experts_route_general(z: torch.Tensor, correction: torch.Tensor, outs: int, 
     return ids, weights, dense, extra
 
 
-def experts_finish(routed: torch.Tensor, x, shared, extra, plus: torch.Tensor | None = None) -> torch.Tensor:
-    """float32 ``routed + extra[:, 0] * x + extra[:, 1] * shared + plus`` row by row; ``routed`` (float32), ``shared`` and ``plus``
-    (float32) may be ``[parts, T, dim]`` (added in order); ``x``, ``shared`` and ``plus`` may be None, and so may ``extra`` where
-    ``x`` is (the shared expert's factor is then 1)."""
+def experts_finish(routed: torch.Tensor, x, shared, extra) -> torch.Tensor:
+    """float32 ``routed + extra[:, 0] * x + extra[:, 1] * shared`` row by row; ``routed`` (float32) and ``shared`` may
+    be ``[parts, T, dim]`` (added in order); ``x`` and ``shared`` may be None, and so may ``extra`` where ``x`` is (the shared
+    expert's factor is then 1)."""
     tokens, dim = routed.shape[-2:]
     parts = routed.shape[0] if routed.dim() == 3 else 1
     shared_parts = shared.shape[0] if shared is not None and shared.dim() == 3 else 1
     out = torch.empty((tokens, dim), dtype=torch.float32, device=routed.device)
     _call("ri_experts_finish", _dev(out, "out"), _dev(routed, "routed", torch.float32), parts, _opt(x, "x"),
           code(x.dtype) if x is not None else F32, _opt(shared, "shared"), code(shared.dtype) if shared is not None else F32,
-          shared_parts, _opt(extra, "extra", torch.float32, (tokens, 2)), _opt(plus, "plus", torch.float32),
-          0 if plus is None else plus.shape[0] if plus.dim() == 3 else 1, tokens, dim, _stream())
+          shared_parts, _opt(extra, "extra", torch.float32, (tokens, 2)), tokens, dim, _stream())
     return out
 
 

@@ -54,13 +54,23 @@ class ResidualStream:
             return None
         return NormLink(self.sum, norm, tiled)
 
-    def push(self, branch) -> None:
+    def push(self, branch, gather: bool = False) -> None:
+        """``gather``: a float32 branch may wait beside others (``pending`` is then a list) for a norm that adds them all."""
+        if (gather and self.pending is not None and self.later is None and not isinstance(branch, tuple)
+                and self._gathers(branch)):
+            self.pending = (self.pending if isinstance(self.pending, list) else [self.pending]) + [branch]
+            return
         if self.pending is not None or self.later is not None:
             self.flush()
         if isinstance(branch, tuple):        # (NormedLater, norm): the product took a NormLink
             self.later = branch
         else:
             self.pending = branch
+
+    def _gathers(self, branch) -> bool:
+        waiting = (self.pending if isinstance(self.pending, list) else [self.pending]) + [branch]
+        return (all(y.dtype == torch.float32 for y in waiting)
+                and sum(y.shape[0] if y.dim() == 3 else 1 for y in waiting) <= ops.MAX_BRANCH_PARTS)
 
     def normed(self, norm, out_dtype, rows=None, later_ok: bool = False, tiled: bool = False):
         """The stream through ``norm``.  With ``later_ok`` the caller takes a ``NormedLater`` too, with
@@ -71,6 +81,14 @@ class ResidualStream:
             if later_ok and for_norm is norm and rows is None:
                 return later
             # prepared for another reader: the sum is complete, norm it the plain way
+        if isinstance(self.pending, list):
+            if getattr(norm, "accepts_branches", False):
+                with profiler.section(profiler.NORM):
+                    out = norm.apply_branches(self.sum, self.pending, out_dtype, rows)
+                if rows is None:
+                    self.pending = None
+                return out
+            self.flush()
         if self.pending is not None and self.pending.dim() == 3 and not getattr(norm, "accepts_parts", False):
             self.flush()                             # a norm that does not know about parts: they go into the sum first
         with profiler.section(profiler.NORM):
@@ -84,17 +102,18 @@ class ResidualStream:
         return out
 
     def add(self, rows) -> None:
-        """``x <- x + rows`` (float32) outside any sublayer.  A branch that waits goes on waiting; what was prepared from the sum
-        as it was is dropped."""
+        """``x <- x + rows`` (float32) outside any sublayer: one more branch that waits.  What was prepared from the sum as it was
+        is dropped."""
         self.later = self.as_act = self.prepared = None
-        ops.add_rows(self.sum, rows, in_place=True)
+        self.push(rows, gather=True)
 
     def flush(self) -> None:
         """Add the waiting branch without a norm (only arrangements that push twice need it)."""
         self.later = None            # its sum is in the stream already
         if self.pending is not None:
-            for part in (self.pending.unbind(0) if self.pending.dim() == 3 else (self.pending,)):
-                ops.add_rows(self.sum, part, in_place=True)       # parts in order, each sum in float32
+            for branch in (self.pending if isinstance(self.pending, list) else (self.pending,)):
+                for part in (branch.unbind(0) if branch.dim() == 3 else (branch,)):
+                    ops.add_rows(self.sum, part, in_place=True)   # parts in order, each sum in float32
             self.pending = None
 
 
@@ -164,8 +183,8 @@ class PreNormBlock:
 @register_part("arrangement", "parallel_prenorm")
 class ParallelPreNormBlock:
     """``x <- x + (mixer(h) + ff(h))`` with ``h = norm(x)``: one norm, whose rows both sublayers read.  Parts: ``mixer_norm``,
-    ``mixer`` and, for a layer that has one, ``feed_forward``.  A feed-forward that sets ``adds_branch`` adds the mixer's result
-    where it adds up its own (``plus=``); the sum then waits for the next norm as one branch."""
+    ``mixer`` and, for a layer that has one, ``feed_forward``.  The results wait as branches of the stream, which the next norm
+    adds (``ops.add_branches_rmsnorm``); a feed-forward that sets ``separates`` hands back those of its own that are only added."""
 
     def __init__(self, layer_spec):
         self.mixer_norm = build_part("norm", layer_spec.mixer_norm)
@@ -185,11 +204,11 @@ class ParallelPreNormBlock:
         y = self.mixer.forward(h, ctx, store, page_table)
         if self.feed_forward is None:
             stream.push(y)
-        elif getattr(self.feed_forward, "adds_branch", False) and isinstance(y, torch.Tensor) and y.dtype == torch.float32:
-            stream.push(self.feed_forward.forward(h, ctx, plus=y))
-        else:
-            stream.push(y)
-            stream.push(self.feed_forward.forward(h, ctx))
+            return
+        z = (self.feed_forward.forward(h, ctx, separate=True) if getattr(self.feed_forward, "separates", False)
+             else self.feed_forward.forward(h, ctx))
+        for branch in [y] + (z if isinstance(z, list) else [z]):
+            stream.push(branch, gather=True)
 
 
 @register_part("arrangement", "hyper_prenorm")

@@ -36,9 +36,9 @@ class GatedDeltaRule(Mixer):
     ``decay="channel"``: a decay per value head and key channel, through a narrow middle whose width the checkpoint gives
     (unless ``rank`` names it): ``g = exp(-exp(A_log_h) softplus(W_a2 (W_a1 h) + dt_bias))`` with ``dt_bias [heads * dim]``, and
     ``S <- diag(g) S``; the output gate then is ``sigmoid(W_g2 (W_g1 h))``, through a middle of its own.  Names ``a1, a2, g1, g2`` in
-    the place of ``a`` and ``g``.  Both middles and the logits of beta are one product (``[a1; g1; b]``), both second steps
-    another, with the block-diagonal of ``a2`` and ``g2``, whose result is float32.  This form can share one input product with
-    other mixers (``in_matrix``, ``heads_from``).
+    the place of ``a`` and ``g``.  q, k, v, both middles and the logits of beta are one product, both second steps another, with
+    the block-diagonal of ``a2`` and ``g2``, whose result is float32.  This form can share one input product with other mixers
+    (``in_matrix``, ``heads_from``).
     """
 
     def __init__(self, hidden: int, heads: int, kv_heads: int, dim: int, vdim: int, taps: int, prefix: str,
@@ -57,7 +57,7 @@ class GatedDeltaRule(Mixer):
         self.per_channel, self.rank = decay == "channel", rank
         self.names = {n: p + n for n in ("q", "k", "v", "g", "o", "a", "b", "norm", "A_log", "dt_bias", "a1", "a2", "g1", "g2")}
         self.names.update(names or {})
-        self.in_width = self.channels = 2 * kv_heads * dim + heads * vdim
+        self.channels = 2 * kv_heads * dim + heads * vdim
 
     def tensors(self):
         n, d, hk, hv, h = self.names, self.hidden, self.kv_heads * self.dim, self.heads * self.vdim, self.heads
@@ -83,8 +83,15 @@ class GatedDeltaRule(Mixer):
         }
 
     def in_matrix(self, weights):
-        """The rows of this mixer's input product (of the form with a decay per channel), ``[q; k; v]``."""
-        return torch.cat([weights[self.names[x]] for x in "qkv"], 0)
+        """The rows of this mixer's input product (of the form with a decay per channel): q, k, v, the two middles, the logits of
+        beta, each group on a multiple of 8 (zero rows between)."""
+        n = self.names
+        groups = ([weights[n[x]] for x in "qkv"], [weights[n["a1"]], weights[n["g1"]]], [weights[n["b"]]])
+        rows = []
+        for group in groups:
+            rows += group
+            rows.append(group[0].new_zeros((-sum(w.shape[0] for w in group) % 8, group[0].shape[1])))
+        return torch.cat(rows, 0)
 
     def out_matrix(self, weights):
         return weights[self.names["o"]]
@@ -96,13 +103,11 @@ class GatedDeltaRule(Mixer):
             if weights[n[one]].shape[0] != weights[n[two]].shape[1]:
                 raise ConfigError(f"{n[one]} has {weights[n[one]].shape[0]} rows, {n[two]} {weights[n[two]].shape[1]} columns")
         ra, rg = a1.shape[0], g1.shape[0]
-        self.b_at = ra + rg
-        width = -(-(self.b_at + self.heads) // 8) * 8                  # the next product's rows in 16-byte pieces
-        mid = torch.zeros((width, self.hidden), dtype=a1.dtype, device=a1.device)
-        mid[:ra], mid[ra:self.b_at], mid[self.b_at:self.b_at + self.heads] = a1, g1, weights[n["b"]]
-        second = torch.zeros((a2.shape[0] + g2.shape[0], width), dtype=a1.dtype, device=a1.device)
-        second[:a2.shape[0], :ra], second[a2.shape[0]:, ra:self.b_at] = a2, g2
-        self.w_mid, self.w_second = rt.pack(rt.place_matrix(mid)), rt.pack(rt.place_matrix(second))
+        self.mid_at, self.mid_width = -(-self.channels // 8) * 8, -(-(ra + rg) // 8) * 8
+        self.b_at = self.mid_at + self.mid_width
+        second = torch.zeros((a2.shape[0] + g2.shape[0], self.mid_width), dtype=a1.dtype, device=a1.device)
+        second[:a2.shape[0], :ra], second[a2.shape[0]:, ra:ra + rg] = a2, g2
+        self.w_second = rt.pack(rt.place_matrix(second))
         if alone:
             self.w_in = rt.pack(rt.place_matrix(self.in_matrix(weights)), always=True)
 
@@ -131,21 +136,21 @@ class GatedDeltaRule(Mixer):
                 StateNeed((self.taps - 1, self.channels), torch.float32))
 
     def heads_from(self, x, proj, col0: int, ctx, store, page_table):
-        """The form with a decay per channel between its two products: ``proj [T, row]`` holds q, k and v from column ``col0``
-        on, ``x`` is the mixer's input; the normed and gated heads, ready for the output product."""
+        """The form with a decay per channel between its two products: ``proj [T, row]`` holds the columns of ``in_matrix`` from
+        ``col0`` on; the normed and gated heads, ready for the output product."""
         rt = self.rt
         state, tails = store
         sizes = (self.heads, self.kv_heads, self.dim, self.vdim)
         with profiler.section(profiler.QKV_PROJECTION):
-            mid = ops.as_rows(rt.linear_packed(x, self.w_mid))                        # [T, a1 | g1 | b]
+            mid = ops.take_columns(proj, col0 + self.mid_at, self.mid_width)         # [T, a1 | g1]
             z = ops.as_rows(rt.linear_packed(mid, self.w_second, out_dtype=torch.float32))      # [T, decays | gates]
         gate_at = self.heads * self.dim
         one_form = rt.dtype == torch.float32 or rt.invariant
         with profiler.section(profiler.ATTENTION):
             if ctx.is_decode and not one_form and ops.delta_step_fits(self.dim, self.vdim):
-                return ops.delta_step_channels(proj, col0, self.conv_taps, tails, z, gate_at, mid, self.b_at, self.a_log, self.dt_bias,
+                return ops.delta_step_channels(proj, col0, self.conv_taps, tails, z, gate_at, proj, col0 + self.b_at, self.a_log, self.dt_bias,
                                                state, ctx.cu_seqlens, ctx.slots, self.gain, self.eps, *sizes)
-            qkv, gates = ops.delta_prepare_channels(proj, col0, self.conv_taps, tails, z, mid, self.b_at, self.a_log, self.dt_bias,
+            qkv, gates = ops.delta_prepare_channels(proj, col0, self.conv_taps, tails, z, proj, col0 + self.b_at, self.a_log, self.dt_bias,
                                                     ctx.tok_seq, ctx.cu_seqlens, ctx.slots, *sizes)
             o = ops.delta_scan_channels(qkv, gates, state, ctx.cu_seqlens, ctx.slots, *sizes, slices=4 if one_form else 0)
             return ops.head_norm_gate(o, z, gate_at, self.gain, self.eps, self.heads, self.vdim, rt.dtype, ops.GATE_SIGMOID)

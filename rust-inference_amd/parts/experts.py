@@ -46,10 +46,11 @@ class RoutedExperts(FeedForward):
     ``scores="table"``: no router.  ``<prefix>table [vocab, top]`` (integers, the entries of a row differ) gives every token id its
     experts, each with the weight ``1 / top``.
 
-    ``forward(..., plus=y)``: another sublayer's float32 result, ``[T, hidden]`` or in parts, to be added to this one's.
+    ``forward(..., separate=True)``: the result may come as a list of branches that the residual stream adds (the routed
+    experts' and the shared expert's, where nothing but their sum is asked for).
     """
 
-    adds_branch = True
+    separates = True
 
     def __init__(self, hidden: int, inter: int, experts: int, top: int, limit: float | None, prefix: str,
                  scores: str = "sigmoid", normalize: bool = True, groups: tuple | None = None, identity: int = 0,
@@ -162,7 +163,7 @@ class RoutedExperts(FeedForward):
                                          ops.ROUTE_SOFTMAX if self.scores == "softmax" else ops.ROUTE_SIGMOID, self.normalize,
                                          self.groups, self.keep, self.best_of)
 
-    def forward(self, x, ctx, plus=None):
+    def forward(self, x, ctx, separate: bool = False):
         rt = self.rt
         with profiler.section(profiler.MLP):
             ids, weights, dense, extra = self.route(x, ctx)
@@ -186,14 +187,16 @@ class RoutedExperts(FeedForward):
                      else ops.experts_activate_plain(gu, dense, self.inter, self.activation))
                 # float32 into the residual (or in parts that the stream's next read adds)
                 y = rt.linear_packed(a, self.w_down, out_dtype=torch.float32, parts_ok=True)
-            if not own and self.shared is None and plus is None:
+            if not own and self.shared is None:
                 return y
             shared = None
             if self.shared is not None:
                 act = rt.linear_packed(x, self.w_shared_in)
                 shared = rt.linear_packed(act, self.w_shared_down, out_dtype=torch.float32, parts_ok=True)
+            if separate and not own and not self.shared_gate:
+                return [y, shared]
             # (without a gate the shared expert is added as it is)
-            return ops.experts_finish(y, rt.normed_now(x) if own else None, shared, extra if own or self.shared_gate else None, plus)
+            return ops.experts_finish(y, rt.normed_now(x) if own else None, shared, extra if own or self.shared_gate else None)
 
     def forward_sorted(self, x, ids, weights):
         """A prompt: every expert's tokens as rows side by side, two library products an expert, the weighted sum in

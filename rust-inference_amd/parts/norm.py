@@ -41,6 +41,12 @@ class RMSNorm(Norm):
     def plain(self, x):
         return plain.rms_norm(x, self.gain_plain, self.eps)
 
+    accepts_branches = True
+
+    def apply_branches(self, residual, branches, out_dtype, rows=None):
+        """``apply`` for several float32 branches that wait side by side."""
+        return ops.add_branches_rmsnorm(residual, branches, self.gain, self.eps, out_dtype, rows)
+
     def apply(self, residual, pending, out_dtype, rows=None, tiled=False):
         tiled = tiled and self.dim % 4 == 0 and self.dim <= 8192        # what the vectorised kernel takes
         return ops.add_rmsnorm(residual, pending, self.gain, self.eps, out_dtype, rows, tiled=tiled)

@@ -103,13 +103,29 @@ def mamba2_mixer(h, w, p, m, eps, state):
 
 
 # ---------------------------------------------------------------- softmax attention in chunks of the sequence
+def attention_core(q, keys, values, start, size, scale):
+    """q [T, heads, dim] at positions start ..; keys and values [start + T, groups, .] from position 0 on; a query sees the keys
+    of its own run of ``size`` positions up to itself."""
+    heads, groups = q.shape[1], keys.shape[1]
+    out = np.zeros((q.shape[0], heads, values.shape[2]))
+    for i in range(q.shape[0]):
+        at = start + i
+        lo = at // size * size                       # the first position of the query's chunk
+        for hd in range(heads):
+            g = hd // (heads // groups)
+            s = keys[lo:at + 1, g] @ q[i, hd] * scale
+            e = np.exp(s - s.max())
+            out[i, hd] = (e / e.sum()) @ values[lo:at + 1, g]
+    return out
+
+
 def chunked_attention(h, w, p, m, eps, state):
     t = h.shape[0]
     heads, groups, dim, vdim = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
-    size = m["mask"]["size"]
+    size = m["mask"]["size"] if m.get("mask") else 1 << 40
     start = state.get("len", 0)
     pos = np.arange(start, start + t, dtype=np.float64)
-    rot = (m["rot"]["dims"], m["rot"]["base"], m["rot"]["scaling"]["factor"])
+    rot = (m["rot"]["dims"], m["rot"]["base"], (m["rot"].get("scaling") or {"factor": 1.0})["factor"]) if m.get("rot") else (0, 1.0, 1.0)
     q = rms_unit((h @ w[p + "q"].T).reshape(t, heads, dim), eps) * w[p + "q.norm"]
     k = rms_unit((h @ w[p + "k"].T).reshape(t, groups, dim), eps) * w[p + "k.norm"]
     q, k = rotate_halves(q, pos, *rot), rotate_halves(k, pos, *rot)
@@ -117,39 +133,46 @@ def chunked_attention(h, w, p, m, eps, state):
     state["k"] = np.concatenate([state["k"], k]) if "k" in state else k
     state["v"] = np.concatenate([state["v"], v]) if "v" in state else v
     state["len"] = start + t
-    out = np.zeros((t, heads, vdim))
-    for i in range(t):
-        at = start + i
-        lo = at // size * size                       # the first position of the query's chunk
-        for hd in range(heads):
-            g = hd // (heads // groups)
-            s = state["k"][lo:at + 1, g] @ q[i, hd] * m["scale"]
-            e = np.exp(s - s.max())
-            out[i, hd] = (e / e.sum()) @ state["v"][lo:at + 1, g]
+    out = attention_core(q, state["k"], state["v"], start, size, m["scale"])
     return out.reshape(t, heads * vdim) @ w[p + "o"].T
 
 
 # ---------------------------------------------------------------- the delta rule with a decay a key channel
+def unit(x):
+    return x / np.sqrt((x * x).sum(-1, keepdims=True) + 1e-6)
+
+
+def decays(z, a_log, dt_bias):
+    """z [T, heads * dim] -> a factor per head and key channel."""
+    heads = a_log.shape[0]
+    return np.exp(-np.exp(a_log)[None, :, None] * softplus(z + dt_bias).reshape(len(z), heads, -1))
+
+
+def delta_walk(q, k, v, beta, g, s):
+    """q, k [T, kv, dim], v [T, heads, vdim], beta [T, heads], g [T, heads, dim]; the states s [heads, dim, vdim] change in place."""
+    out = np.zeros(v.shape)
+    share = v.shape[1] // q.shape[1]
+    for i in range(v.shape[0]):
+        for hd in range(v.shape[1]):
+            qi, ki = q[i, hd // share], k[i, hd // share]
+            s[hd] = g[i, hd][:, None] * s[hd]
+            u = beta[i, hd] * (v[i, hd] - s[hd].T @ ki)
+            s[hd] = s[hd] + np.outer(ki, u)
+            out[i, hd] = s[hd].T @ qi                # the read-out sees the token's own write
+    return out
+
+
 def delta_mixer(h, w, p, m, eps, state):
     t = h.shape[0]
     heads, kv, dim, vdim = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
     conv = lambda n: silu(short_conv(h @ w[p + n].T, w[p + n + ".conv"], None, state, n))
-    unit = lambda x: x / np.sqrt((x * x).sum(-1, keepdims=True) + 1e-6)
     q = unit(conv("q").reshape(t, kv, dim)) * dim ** -0.5
     k = unit(conv("k").reshape(t, kv, dim))
     v = conv("v").reshape(t, heads, vdim)
     beta = sigmoid(h @ w[p + "b"].T)
-    z = softplus((h @ w[p + "a1"].T) @ w[p + "a2"].T + w[p + "dt_bias"]).reshape(t, heads, dim)
-    g = np.exp(-np.exp(w[p + "A_log"])[None, :, None] * z)
+    g = decays((h @ w[p + "a1"].T) @ w[p + "a2"].T, w[p + "A_log"], w[p + "dt_bias"])
     s = state.get("S", np.zeros((heads, dim, vdim)))
-    out = np.zeros((t, heads, vdim))
-    for i in range(t):
-        for hd in range(heads):
-            qi, ki = q[i, hd // (heads // kv)], k[i, hd // (heads // kv)]
-            s[hd] = g[i, hd][:, None] * s[hd]
-            u = beta[i, hd] * (v[i, hd] - s[hd].T @ ki)
-            s[hd] = s[hd] + np.outer(ki, u)
-            out[i, hd] = s[hd].T @ qi
+    out = delta_walk(q, k, v, beta, g, s)
     state["S"] = s
     gate = sigmoid((h @ w[p + "g1"].T) @ w[p + "g2"].T)
     y = (rms_unit(out, eps) * w[p + "norm"]).reshape(t, heads * vdim) * gate

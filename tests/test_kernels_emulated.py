@@ -63,6 +63,9 @@ PISULORN_TESTS = os.path.join(HERE, "test_pisulorn_kernels_gpu.py")
 ZAKELORN_TESTS = os.path.join(HERE, "test_zakelorn_kernels_gpu.py")
 NOTADRA_TESTS = os.path.join(HERE, "test_notadra_kernels_gpu.py")
 DAGEZEN_TESTS = os.path.join(HERE, "test_dagezen_kernels_gpu.py")
+KISEPEL_TESTS = os.path.join(HERE, "test_kisepel_kernels_gpu.py")
+KISEPEL_SELECT = ("not many_sequences and not thousands and not 8200 and not 4100 and not lens7 "
+                  "and not (in_chunks and not (tokens-33 or prompts-100 or portions-64 or 31-6 or 100-3 or 33-2))")      # a chunk size a form
 PISULORN_SELECT = "not two_equal_keys and not many_sequences"      # not the 1,300 keys and the 512 workgroups on the emulated matrix cores (minutes)
 NOTADRA_SELECT = ("not many_sequences and not thousands_of_keys and not (matrix_core and not (64-88 or 24-36 or 128-252 or 40-64))"
                   " and not 8192 and not 8200 and not 4100")          # a size of every capacity, not every size (minutes each)
@@ -89,6 +92,8 @@ def runs():
         "zakelorn": _start([*PYTEST, *_workers(2), ZAKELORN_TESTS, "-k", "not thousands_of_keys"]),
         "dagezen": _start([*PYTEST, *_workers(2), DAGEZEN_TESTS]),
         "notadra": _start([*PYTEST, *_workers(3), NOTADRA_TESTS, "-k", NOTADRA_SELECT]),
+        "kisepel": _start([*PYTEST, *_workers(3), KISEPEL_TESTS, "-k", KISEPEL_SELECT]),
+        "kisepel, eight units": _start([*PYTEST, KISEPEL_TESTS, "-k", "many_sequences"], {"RI_EMU_COMPUTE_UNITS": "8"}),
         # (eight compute units: the decode attention then walks whole runs of keys for a few sequences already)
         "notadra, eight units": _start([*PYTEST, *_workers(2), NOTADRA_TESTS, "-k", "many_sequences and 64-88"], {"RI_EMU_COMPUTE_UNITS": "8"}),
         # (with one compute unit a prompt of 70 tokens already takes the form of the rotation kernel that gives a
@@ -160,6 +165,14 @@ def test_the_kernels_of_the_notadra_design_pass_on_the_cpu_build_between_guard_p
     sizes of their own), groups scored by their two best, experts without gates."""
     _passed(runs["notadra"])
     _passed(runs["notadra, eight units"], 2)
+
+
+def test_the_kernels_of_the_kisepel_design_pass_on_the_cpu_build_between_guard_pages(runs):
+    """tests/test_kisepel_kernels_gpu.py: the q/k norm with the scaled rotation and the cache write, attention in chunks of the
+    sequence (generic and on the emulated matrix cores), the delta rule with a decay per key channel, norms of mixers side by
+    side, branches that wait for a norm, experts by a table."""
+    _passed(runs["kisepel"])
+    _passed(runs["kisepel, eight units"], 6)
 
 
 @pytest.mark.parametrize("units, tests", [("sixteen units", 7), ("one unit", 61)])
