@@ -146,7 +146,7 @@ int ri_delta_prepare(float* qkv, float* gates, const void* proj, int act_dtype, 
 // Per sequence and head, over the sequence's new tokens in order: S <- g S; u = beta (v - S^T k); S <- S + k u^T;
 // o = S^T q.  state: float32 [slots, heads, dim, vdim]; out: float32 [tokens, heads * vdim].
 int ri_delta_max_dim();
-// slices: over how many lanes a column's rows are spread, 4 or 8; 0: by the size of the launch.
+// slices: over how many lanes a column's rows are spread, 4, 8 or 16; 0: by the size of the launch.
 int ri_delta_scan(float* out, const float* qkv, const float* gates, float* state, const int32_t* cu_seqlens,
                   const int32_t* slots, int seqs, int tokens, int heads, int kv_heads, int dim, int vdim, int slices,
                   void* stream);

@@ -20,6 +20,12 @@
 __device__ __forceinline__ float silu_f(float v) { return v / (1.f + expf(-v)); }
 __device__ __forceinline__ float softplus_f(float v) { return fmaxf(v, 0.f) + log1pf(expf(-fabsf(v))); }
 
+// A token's row of gates: g then beta per head; with CH the decays of every head and the betas, padded to a multiple of 4.
+template <bool CH>
+__host__ __device__ __forceinline__ int delta_gate_row(int heads, int dim) {
+    return CH ? heads * dim + ((heads + 3) & ~3) : 2 * heads;
+}
+
 // A workgroup takes one token and one unit of its channels: a q or k head (units 0 .. 2 kv_heads - 1), which it
 // norms, or a stretch of DELTA_V_UNIT channels of v.  conv[] (dynamic LDS, max(dim, DELTA_V_UNIT) floats) holds the
 // unit's activated convolutions.  (One workgroup a token walked its thousands of channels in turns of 256, each
@@ -43,7 +49,7 @@ delta_prepare_kernel(float* __restrict__ qkv, float* __restrict__ gates, const T
     const int qk = kv_heads * dim, channels = 2 * qk + heads * vdim;
     if (CH) {
         const int decays = heads * dim, at = (unit - 2 * kv_heads - (heads * vdim + DELTA_V_UNIT - 1) / DELTA_V_UNIT) * DELTA_V_UNIT;
-        float* to = gates + (size_t)t * (decays + heads);
+        float* to = gates + (size_t)t * delta_gate_row<CH>(heads, dim);
         if (at >= 0) {                                        // a stretch of decays (the whole workgroup)
             const int e = at + threadIdx.x;
             if (e < decays) to[e] = expf(-expf(a_log[e / dim]) * softplus_f(ab[(size_t)t * z_row + e] + dt_bias[e]));
@@ -128,7 +134,7 @@ delta_prepare_pieces_kernel(float* __restrict__ qkv, float* __restrict__ gates, 
                             const int32_t* __restrict__ slots, int heads, int kv_heads, int dim, int vdim, int z_row,
                             const T* __restrict__ bsrc, int b_row, int tokens) {
     const int qk = kv_heads * dim, channels = 2 * qk + heads * vdim, decays = CH ? heads * dim : 0;
-    const int pieces = channels / 4, lanes = dim / 4, t0 = blockIdx.y * TT, gate_row = CH ? decays + heads : 2 * heads;
+    const int pieces = channels / 4, lanes = dim / 4, t0 = blockIdx.y * TT, gate_row = delta_gate_row<CH>(heads, dim);
     if (blockIdx.x == 0) {                                    // a number a head: the betas and, without CH, the decays
         for (int e = threadIdx.x; e < TT * heads; e += 256) {
             const int t = t0 + e / heads, h = e % heads;
@@ -239,12 +245,13 @@ __device__ __forceinline__ float quad_sum(float v) {
     return v;
 }
 
-// The same over the SL = 4 or 8 lanes of a column: after the quads, the mirror image inside every eight lanes
-// (lane i takes lane 7 - i: the other quad, all of whose lanes hold its sum).
+// The same over the SL = 4, 8 or 16 lanes of a column: after the quads, the mirror image inside every eight lanes
+// (lane i takes lane 7 - i: the other quad, all of whose lanes hold its sum), then inside every sixteen.
 template <int SL>
 __device__ __forceinline__ float slices_sum(float v) {
     v = quad_sum(v);
-    if (SL == 8) v += __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0x141, 0xF, 0xF, true));
+    if (SL >= 8) v += __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0x141, 0xF, 0xF, true));
+    if (SL == 16) v += __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0x140, 0xF, 0xF, true));
     return v;
 }
 
@@ -256,7 +263,7 @@ __device__ __forceinline__ float slices_sum(float v) {
 // double the workgroups that each stage q and k, which is what counts once the machine is full: the launch chooses.
 template <int RPT, int SL, bool CH>
 struct DeltaLds {
-    static constexpr int DELTA_BLOCK = RPT * SL >= 256 ? 8 : 16;    // tokens a block: two buffers stay inside 64 KB
+    static constexpr int DELTA_BLOCK = RPT * SL >= (CH ? 128 : 256) ? 8 : 16;    // tokens a block: two buffers stay inside 64 KB
     static constexpr int QS = RPT + 4;                        // stride of a slice of q or k: no bank conflicts between the slices
     static constexpr int COLS = 256 / SL;
     float q[DELTA_BLOCK][SL][QS];
@@ -293,7 +300,7 @@ delta_scan_kernel(float* __restrict__ out, const float* __restrict__ qkv, const 
         S[i] = (has_col && rw < dim) ? v : 0.f;
     }
 
-    const int gate_row = CH ? heads * dim + heads : 2 * heads;
+    const int gate_row = delta_gate_row<CH>(heads, dim);
     float fq[QR], fk[QR], fgk[CH ? QR : 1], fv[VR], fg = 0.f;
     auto fetch = [&](int first) {                             // the block of tokens first ..+DELTA_BLOCK, into registers
 #pragma unroll
@@ -370,6 +377,138 @@ delta_scan_kernel(float* __restrict__ out, const float* __restrict__ qkv, const 
         __syncthreads();
         cur ^= 1;
     }
+#pragma unroll
+    for (int i = 0; i < RPT; ++i) {
+        const int rw = r * RPT + i;
+        if (has_col && rw < dim) st[(size_t)rw * vdim + col] = S[i];
+    }
+}
+
+// The walk of a launch of few heads: a workgroup is one wavefront with four columns and sixteen slices of rows, so that a head of
+// 128 columns is 32 workgroups, each on a vector unit of its own, and a token costs 5 RPT vector instructions of one wavefront.
+// What the chain from token to token waits for is short: with S' = g S, both sums of a token run over S' side by side (S'^T k
+// and S'^T q, beside k . q), then u = beta (v - S'^T k) and o = S'^T q + (k . q) u, and S = S' + k u is ready for the next token
+// without a sum of its own.  q, k and the decays come in 16-byte pieces (dim and the rows a multiple of 4), a block of tokens at a
+// time, the next block's in flight; a token's values are read from LDS while the token before it is walked.  A block's results
+// wait in LDS and leave before the next loads are asked for: a store among the walk's tokens would be waited for with those loads.
+template <int RPT, bool CH>
+struct DeltaToken {
+    float k[RPT], q[RPT], gk[CH ? RPT : 1], g, beta, v;
+};
+
+template <int RPT, bool CH>
+__global__ void __launch_bounds__(64)
+delta_scan_narrow_kernel(float* __restrict__ out, const float* __restrict__ qkv, const float* __restrict__ gates,
+                         float* __restrict__ state, const int32_t* __restrict__ cu_seqlens, const int32_t* __restrict__ slots,
+                         int heads, int kv_heads, int dim, int vdim) {
+    constexpr int B = RPT <= 8 ? 16 : 8, SL = 16, COLS = 4, PIECES = SL * RPT / 4, PR = B * PIECES / 64, QS = RPT + 4;
+    __shared__ __attribute__((aligned(16))) float lq[B][SL][QS], lk[B][SL][QS], lg[CH ? B : 1][SL][CH ? QS : 4];
+    __shared__ float lv[B][COLS], lo[B][COLS], lbeta[B], lgs[B];
+    const int b = blockIdx.x / heads, h = blockIdx.x % heads, col0 = blockIdx.y * COLS, hq = h / (heads / kv_heads);
+    const int tid = threadIdx.x, r = tid & (SL - 1), mine = tid / SL, col = col0 + mine;
+    const bool has_col = col < vdim;
+    const int t0 = cu_seqlens[b], n = cu_seqlens[b + 1] - t0;
+    if (n <= 0) return;
+    const int qk = kv_heads * dim, channels = 2 * qk + heads * vdim, gate_row = delta_gate_row<CH>(heads, dim);
+    float* st = state + (((size_t)slots[b] * heads + h) * dim) * vdim;
+
+    float S[RPT];
+#pragma unroll
+    for (int i = 0; i < RPT; ++i) {
+        const int rw = r * RPT + i;
+        const float v = st[(size_t)min(rw, dim - 1) * vdim + min(col, vdim - 1)];
+        S[i] = (has_col && rw < dim) ? v : 0.f;
+    }
+
+    float4 fq[PR], fk[PR], fg[CH ? PR : 1];
+    float fv, fbeta, fgs = 0.f;
+    auto fetch = [&](int first) {                             // the block of tokens first ..+B, into registers
+#pragma unroll
+        for (int e = 0; e < PR; ++e) {
+            const int at = e * 64 + tid, tk = at / PIECES, rw = (at % PIECES) * 4;
+            const int t = t0 + min(first + tk, n - 1), row = min(rw, dim - 4);
+            const float* p = qkv + (size_t)t * channels + hq * dim + row;
+            fq[e] = delta_ld4(p);
+            fk[e] = delta_ld4(p + qk);
+            if (CH) fg[e] = delta_ld4(gates + (size_t)t * gate_row + h * dim + row);
+        }
+        const int vt = t0 + min(first + (tid & (B * COLS - 1)) / COLS, n - 1);
+        fv = qkv[(size_t)vt * channels + 2 * qk + h * vdim + min(col0 + tid % COLS, vdim - 1)];
+        const float* gp = gates + (size_t)(t0 + min(first + (tid & (B - 1)), n - 1)) * gate_row + (CH ? heads * dim : heads) + h;
+        fbeta = gp[0];
+        if (!CH) fgs = gp[-heads];
+    };
+    auto stage = [&]() {
+#pragma unroll
+        for (int e = 0; e < PR; ++e) {
+            const int at = e * 64 + tid, tk = at / PIECES, rw = (at % PIECES) * 4;
+            const bool ok = rw < dim;                         // rows past dim: a state of zeros that stays so
+            // (component by component: a choice between whole structures would put the arrays into memory)
+            auto kept = [&](const float4& v) { return make_float4(ok ? v.x : 0.f, ok ? v.y : 0.f, ok ? v.z : 0.f, ok ? v.w : 0.f); };
+            *reinterpret_cast<float4*>(&lq[tk][rw / RPT][rw % RPT]) = kept(fq[e]);
+            *reinterpret_cast<float4*>(&lk[tk][rw / RPT][rw % RPT]) = kept(fk[e]);
+            if (CH) *reinterpret_cast<float4*>(&lg[tk][rw / RPT][rw % RPT]) = kept(fg[e]);
+        }
+        if (tid < B * COLS) lv[tid / COLS][tid % COLS] = fv;
+        if (tid < B) {
+            lbeta[tid] = fbeta;
+            if (!CH) lgs[tid] = fgs;
+        }
+    };
+    typedef DeltaToken<RPT, CH> Token;
+    auto read = [&](Token& x, int tk) {
+#pragma unroll
+        for (int i = 0; i < RPT; i += 4) {
+            const float4 k = delta_ld4(&lk[tk][r][i]), q = delta_ld4(&lq[tk][r][i]);
+            x.k[i] = k.x; x.k[i + 1] = k.y; x.k[i + 2] = k.z; x.k[i + 3] = k.w;
+            x.q[i] = q.x; x.q[i + 1] = q.y; x.q[i + 2] = q.z; x.q[i + 3] = q.w;
+            if (CH) {
+                const float4 g = delta_ld4(&lg[tk][r][i]);
+                x.gk[i] = g.x; x.gk[i + 1] = g.y; x.gk[i + 2] = g.z; x.gk[i + 3] = g.w;
+            }
+        }
+        x.g = CH ? 1.f : lgs[tk];
+        x.beta = lbeta[tk];
+        x.v = lv[tk][mine];
+    };
+    auto walk = [&](const Token& x, int tk) {
+        float a[2] = {0.f, 0.f}, o[2] = {0.f, 0.f}, c[2] = {0.f, 0.f};
+#pragma unroll
+        for (int i = 0; i < RPT; ++i) {
+            S[i] *= CH ? x.gk[i] : x.g;
+            a[i & 1] += S[i] * x.k[i];
+            o[i & 1] += S[i] * x.q[i];
+            c[i & 1] += x.k[i] * x.q[i];
+        }
+        const float sa = slices_sum<16>(a[0] + a[1]), so = slices_sum<16>(o[0] + o[1]), sc = slices_sum<16>(c[0] + c[1]);
+        const float u = x.beta * (x.v - sa);
+#pragma unroll
+        for (int i = 0; i < RPT; ++i) S[i] += x.k[i] * u;
+        if (r == 0) lo[tk][mine] = so + sc * u;
+    };
+    auto hand_on = [&](int first, int count) {                // the results of a block that was walked
+        if (tid < count * COLS && col0 + tid % COLS < vdim)
+            out[(size_t)(t0 + first + tid / COLS) * heads * vdim + (size_t)h * vdim + col0 + tid % COLS] = lo[tid / COLS][tid % COLS];
+    };
+
+    fetch(0);
+    for (int first = 0; first < n; first += B) {
+        stage();
+        if (first > 0) hand_on(first - B, B);
+        __syncthreads();                                      // (one wavefront: what it wrote is in place)
+        const int count = min(B, n - first);
+        fetch(first + B < n ? first + B : first);             // (always issued: no load in a branch)
+        Token x, y;
+        read(x, 0);
+        for (int tk = 0; tk < count; tk += 2) {               // (the last token's successor is read from its own place and not used)
+            read(y, min(tk + 1, B - 1));
+            walk(x, tk);
+            read(x, min(tk + 2, B - 1));
+            if (tk + 1 < count) walk(y, tk + 1);
+        }
+        __syncthreads();
+    }
+    hand_on((n - 1) / B * B, (n - 1) % B + 1);
 #pragma unroll
     for (int i = 0; i < RPT; ++i) {
         const int rw = r * RPT + i;
@@ -660,20 +799,31 @@ template <bool CH>
 static int launch_delta_scan(float* out, const float* qkv, const float* gates, float* state, const int32_t* cu_seqlens,
                              const int32_t* slots, int seqs, int tokens, int heads, int kv_heads, int dim, int vdim,
                              int slices, void* stream) {
-    RI_REQUIRE(slices == 0 || slices == 4 || slices == 8, "delta_scan: %d slices of rows (4, 8, or 0 for the launch's choice)", slices);
+    RI_REQUIRE(slices == 0 || slices == 4 || slices == 8 || slices == 16,
+               "delta_scan: %d slices of rows (4, 8, 16, or 0 for the launch's choice)", slices);
     RI_REQUIRE(tokens > 0 && seqs > 0 && heads > 0 && kv_heads > 0 && heads % kv_heads == 0 && vdim > 0,
                "delta_scan: tokens %d, sequences %d, heads %d, kv heads %d", tokens, seqs, heads, kv_heads);
     RI_REQUIRE(dim >= 1 && dim <= 256, "delta_scan: key heads of %d, the kernel takes 1 to 256", dim);
-    RI_REQUIRE((long)seqs * heads <= 2147483647L && (vdim + 31) / 32 <= 65535, "delta_scan: the grid");
+    RI_REQUIRE((long)seqs * heads <= 2147483647L && (vdim + 3) / 4 <= 65535, "delta_scan: the grid");
     hipStream_t s = (hipStream_t)stream;
-    // eight slices of rows while the workgroups of four would leave compute units idle (a token's time halves), four
-    // once they fill the machine (half the workgroups stage q and k)
-    const bool eight = slices ? slices == 8 : (long)seqs * heads * ((vdim + 63) / 64) <= (long)ri_compute_units() && dim >= 8;
-    const int sl = eight ? 8 : 4, cols = 256 / sl;
+    // sixteen slices of rows in workgroups of one wavefront while every wavefront has a vector unit of its own; else eight slices
+    // while the workgroups of four would leave compute units idle (a token's time halves), four once they fill the machine (half
+    // the workgroups stage q and k)
+    const long cus = ri_compute_units(), narrow = (long)seqs * heads * ((vdim + 3) / 4);
+    const bool pieces = dim % 4 == 0 && (heads * vdim) % 4 == 0 && ((uintptr_t)qkv | (uintptr_t)gates) % 16 == 0;
+    RI_REQUIRE(slices != 16 || pieces, "delta_scan: sixteen slices take heads in 16-byte pieces, not %d x %d", dim, vdim);
+    const int sl = slices ? slices : narrow <= 4 * cus && pieces && dim >= 16 ? 16
+                   : (long)seqs * heads * ((vdim + 63) / 64) <= cus && dim >= 8 ? 8 : 4;
+    const int cols = sl == 16 ? 4 : 256 / sl;
     const dim3 grid((unsigned)(seqs * heads), (unsigned)((vdim + cols - 1) / cols));
     const int need = (dim + sl - 1) / sl;
 #define RI_DELTA_GO(R, SL) delta_scan_kernel<R, SL, CH><<<grid, 256, 0, s>>>(out, qkv, gates, state, cu_seqlens, slots, heads, kv_heads, dim, vdim)
-    if (eight) {
+#define RI_DELTA_NARROW(R) delta_scan_narrow_kernel<R, CH><<<grid, 64, 0, s>>>(out, qkv, gates, state, cu_seqlens, slots, heads, kv_heads, dim, vdim)
+    if (sl == 16) {
+        if (need <= 4) RI_DELTA_NARROW(4);
+        else if (need <= 8) RI_DELTA_NARROW(8);
+        else RI_DELTA_NARROW(16);
+    } else if (sl == 8) {
         if (need <= 4) RI_DELTA_GO(4, 8);
         else if (need <= 8) RI_DELTA_GO(8, 8);
         else if (need <= 16) RI_DELTA_GO(16, 8);
@@ -686,6 +836,7 @@ static int launch_delta_scan(float* out, const float* qkv, const float* gates, f
         else RI_DELTA_GO(64, 4);
     }
 #undef RI_DELTA_GO
+#undef RI_DELTA_NARROW
     RI_LAUNCH_CHECK("delta_scan");
     return 0;
 }

@@ -165,6 +165,7 @@ static inline int emu_mov_dpp_quad(int v, int control) {
     emu::wave_gather(&v, sizeof(int), all);
     const int lane = emu::self->lane;
     if (control == 0x141) return all[(lane & ~7) | (7 - (lane & 7))];
+    if (control == 0x140) return all[(lane & ~15) | (15 - (lane & 15))];
     return all[(lane & ~3) | ((control >> (2 * (lane & 3))) & 3)];
 }
 #define __builtin_amdgcn_mov_dpp(v, control, row_mask, bank_mask, bound_ctrl) emu_mov_dpp_quad((v), (control))

@@ -866,7 +866,7 @@ def delta_scan(qkv, gates, state, cu_seqlens, slots, heads: int, kv_heads: int, 
                slices: int = 0) -> torch.Tensor:
     """The gated delta rule over every sequence's new tokens, ``S <- g S; u = beta (v - S^T k); S <- S + k u^T;
     o = S^T q``; float32 ``[T, heads * vdim]``.  ``state: [slots, heads, dim, vdim]`` float32 is read and written at
-    the sequences' slots.  ``slices``: the lanes a column's rows are spread over, 4 or 8 (0: chosen by the size of the
+    the sequences' slots.  ``slices``: the lanes a column's rows are spread over, 4, 8 or 16 (heads in 16-byte pieces; 0: chosen by the size of the
     launch, which depends on the sequences and heads and not on their tokens)."""
     tokens = qkv.shape[0]
     seqs = slots.shape[0]
@@ -908,6 +908,11 @@ def delta_step(proj, q_off: int, g_off: int, taps, tails, ab, a_log, dt_bias, st
     return out
 
 
+def delta_gate_row(heads: int, dim: int) -> int:
+    """Columns of the gates of a decay per key channel: the decays, then the betas, padded to a multiple of 4."""
+    return heads * dim + -(-heads // 4) * 4
+
+
 def _check_delta(tails, state, ntaps: int, channels: int, heads: int, dim: int, vdim: int) -> None:
     if tails is not None and (tails.dim() != 3 or tuple(tails.shape[1:]) != (ntaps - 1, channels)):
         raise ShapeError(f"the convolutions' tails are {list(tails.shape)}, not [slots, {ntaps - 1}, {channels}]")
@@ -926,12 +931,13 @@ def delta_prepare_channels(proj, q_off: int, taps, tails, z, mid, b_off: int, a_
                            heads: int, kv_heads: int, dim: int, vdim: int):
     """``delta_prepare`` for a decay per head and key channel: ``z [T, >= heads * dim]`` float32 are the decays'
     pre-activations, ``g = exp(-exp(a_log_h) softplus(z + dt_bias))`` with ``dt_bias [heads * dim]``; the logits of beta are the
-    columns ``b_off ..`` of ``mid`` (in the format of ``proj``, or ``proj`` itself).  ``gates`` is ``[T, heads * dim + heads]``."""
+    columns ``b_off ..`` of ``mid`` (in the format of ``proj``, or ``proj`` itself).  ``gates`` is ``[T, delta_gate_row]``: the
+    decays, then the betas."""
     tokens, row = proj.shape
     seqs, channels, ntaps = slots.shape[0], 2 * kv_heads * dim + heads * vdim, taps.shape[1]
     _check_delta(tails, None, ntaps, channels, heads, dim, vdim)
     qkv = torch.empty((tokens, channels), dtype=torch.float32, device=proj.device)
-    gates = torch.empty((tokens, heads * dim + heads), dtype=torch.float32, device=proj.device)
+    gates = torch.empty((tokens, delta_gate_row(heads, dim)), dtype=torch.float32, device=proj.device)
     b, b_row = _beta_logits(mid, b_off, heads, proj.dtype)
     _call("ri_delta_prepare_channels", _dev(qkv, "qkv"), _dev(gates, "gates"), _dev(proj, "proj"), code(proj.dtype), row, q_off,
           _dev(taps, "taps", torch.float32, (channels, ntaps)), ntaps, _dev(tails, "tails", torch.float32),
@@ -949,7 +955,7 @@ def delta_scan_channels(qkv, gates, state, cu_seqlens, slots, heads: int, kv_hea
     _check_delta(None, state, 1, 0, heads, dim, vdim)
     out = torch.empty((tokens, heads * vdim), dtype=torch.float32, device=qkv.device)
     _call("ri_delta_scan_channels", _dev(out, "out"), _dev(qkv, "qkv", torch.float32, (tokens, 2 * kv_heads * dim + heads * vdim)),
-          _dev(gates, "gates", torch.float32, (tokens, heads * dim + heads)), _dev(state, "state", torch.float32),
+          _dev(gates, "gates", torch.float32, (tokens, delta_gate_row(heads, dim))), _dev(state, "state", torch.float32),
           _dev(cu_seqlens, "cu_seqlens", torch.int32, (seqs + 1,)), _dev(slots, "slots", torch.int32, (seqs,)),
           seqs, tokens, heads, kv_heads, dim, vdim, int(slices), _stream())
     return out

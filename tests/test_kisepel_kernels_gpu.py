@@ -221,7 +221,7 @@ def test_single_tokens_of_many_sequences_walk_their_chunk_in_runs(ops, size, dim
     from rust_inference_amd.kernels.build import load
     rng = np.random.default_rng(dim + size)
     kv = 8
-    seqs = -(-2 * load().ri_compute_units() // kv)
+    seqs = max(4, -(-2 * load().ri_compute_units() // kv))
     heads = 2 * kv
     lens = [int(n) for n in rng.integers(1, 150, seqs)]
     lens[0], lens[1], lens[2] = 1, 97, 96                     # one past a chunk's edge, and its last token
@@ -275,6 +275,12 @@ def delta_case(rng, T, H, G, dk, dv, K, lead):
             "a_log": rng.normal(size=H) * 0.7 - 0.5, "dt_bias": rng.normal(size=H * dk) * 0.7}
 
 
+def lay_gates(ops, g, beta):
+    """[decays | betas | what pads a row]."""
+    T, H, dk = g.shape
+    return t(np.concatenate([g.reshape(T, -1), beta, np.full((T, ops.delta_gate_row(H, dk) - H * dk - H), 7.0)], 1))
+
+
 def plain_prepare(c, H, G, dk, dv, lens, tails, lead):
     """q, k, v, gates of the sequences one after the other; ``tails`` are moved on in place."""
     rows, gates, at, C = [], [], 0, c["C"]
@@ -310,7 +316,8 @@ def test_delta_prepare_with_a_decay_per_channel(ops, dtype, H, G, dk, dv, K, len
     qkv, gates = ops.delta_prepare_channels(proj, lead, t(c["taps"]), dev_tails, t(c["z"]), proj, lead + c["C"], t(c["a_log"]), t(c["dt_bias"]),
                                             t(seq, torch.int32), t(cu, torch.int32), t(slots, torch.int32), H, G, dk, dv)
     close(qkv, want_qkv, F32, "q, k, v")
-    close(gates, want_gates, F32, "gates")
+    assert gates.shape[1] == ops.delta_gate_row(H, dk)
+    close(gates[:, :H * dk + H], want_gates, F32, "gates")
     for s, want in zip(slots, plain_tails):
         if K > 1:
             close(dev_tails[s], want, 1e-7, "tail")
@@ -319,14 +326,16 @@ def test_delta_prepare_with_a_decay_per_channel(ops, dtype, H, G, dk, dv, K, len
 
 
 WALKS = [(4, 2, 12, 20, (1, 7, 3)), (2, 1, 64, 48, (45,)), (3, 3, 5, 70, (2, 18)), (2, 2, 100, 33, (17, 1)), (1, 1, 256, 40, (20,)), (2, 1, 130, 64, (9, 24)),
-         (6, 6, 8, 8, (40, 3))]
+         (6, 6, 8, 8, (40, 3)), (3, 1, 16, 12, (8, 7, 9)), (2, 2, 200, 10, (25,))]
 
 
 @pytest.mark.parametrize("H, G, dk, dv, lens", WALKS)
-@pytest.mark.parametrize("slices", [0, 4, 8])
+@pytest.mark.parametrize("slices", [0, 4, 8, 16])
 def test_delta_walk_with_a_decay_per_channel(ops, H, G, dk, dv, lens, slices):
     rng = np.random.default_rng(H * 11 + dk)
     T = sum(lens)
+    if slices == 16 and (dk % 4 or H * dv % 4):
+        pytest.skip("sixteen slices take heads in 16-byte pieces")
     q, k, v = P.unit(rng.normal(size=(T, G, dk))) * dk ** -0.5, P.unit(rng.normal(size=(T, G, dk))), rng.normal(size=(T, H, dv))
     g, beta = rng.uniform(0.3, 1.0, size=(T, H, dk)), rng.uniform(0.1, 1.0, size=(T, H))
     slots = [2, 0, 3][:len(lens)]
@@ -338,24 +347,24 @@ def test_delta_walk_with_a_decay_per_channel(ops, H, G, dk, dv, lens, slices):
     qkv = np.concatenate([q.reshape(T, -1), k.reshape(T, -1), v.reshape(T, -1)], 1)
     cu = np.concatenate([[0], np.cumsum(lens)])
     dev_state = t(state)
-    got = ops.delta_scan_channels(t(qkv), t(np.concatenate([g.reshape(T, -1), beta], 1)), dev_state, t(cu, torch.int32), t(slots, torch.int32),
+    got = ops.delta_scan_channels(t(qkv), lay_gates(ops, g, beta), dev_state, t(cu, torch.int32), t(slots, torch.int32),
                                   H, G, dk, dv, slices)
     close(got, np.concatenate(want).reshape(T, -1), 1e-5, "outputs")
     close(dev_state, want_state, 1e-5, "state")
 
 
-@pytest.mark.parametrize("slices", [4, 8])
+@pytest.mark.parametrize("slices", [4, 8, 16])
 def test_the_walk_token_by_token_is_the_walk_in_blocks(ops, slices):
     """The same 37 tokens in one step, and one at a time from the state the step before left: the same bits."""
     rng = np.random.default_rng(5)
     H, G, dk, dv, T = 2, 1, 24, 40, 37
     q, k = P.unit(rng.normal(size=(T, G, dk))) * dk ** -0.5, P.unit(rng.normal(size=(T, G, dk)))
     qkv = np.concatenate([q.reshape(T, -1), k.reshape(T, -1), rng.normal(size=(T, H * dv))], 1)
-    gates = np.concatenate([rng.uniform(0.3, 1.0, size=(T, H * dk)), rng.uniform(0.1, 1.0, size=(T, H))], 1)
+    gates = lay_gates(ops, rng.uniform(0.3, 1.0, size=(T, H, dk)), rng.uniform(0.1, 1.0, size=(T, H)))
     one, slot = t(np.zeros((2, H, dk, dv))), t([1], torch.int32)
-    whole = ops.delta_scan_channels(t(qkv), t(gates), one, t([0, T], torch.int32), slot, H, G, dk, dv, slices)
+    whole = ops.delta_scan_channels(t(qkv), gates, one, t([0, T], torch.int32), slot, H, G, dk, dv, slices)
     two = t(np.zeros((2, H, dk, dv)))
-    rows = [ops.delta_scan_channels(t(qkv[i:i + 1]), t(gates[i:i + 1]), two, t([0, 1], torch.int32), slot, H, G, dk, dv, slices) for i in range(T)]
+    rows = [ops.delta_scan_channels(t(qkv[i:i + 1]), t(f64(gates[i:i + 1])), two, t([0, 1], torch.int32), slot, H, G, dk, dv, slices) for i in range(T)]
     assert torch.equal(torch.cat([r.cpu() for r in rows]), whole.cpu()) and torch.equal(one.cpu(), two.cpu())
 
 
