@@ -117,7 +117,7 @@ delta_prepare_kernel(float* __restrict__ qkv, float* __restrict__ gates, const T
 // The same for q/k heads whose four-channel pieces are a power of two that divides a wavefront, up to four taps: a thread takes
 // four neighbouring channels (or decays) of TT tokens in turn and keeps the inputs before its token in registers, so that a row
 // is read once; a head's norm meets over its dim / 4 lanes, without a barrier.  (The form above reads every row once per tap and
-// leaves threads idle where a head has fewer channels than a workgroup threads: 64 us against 13 for 2,048 tokens of 8 heads of 128.)
+// leaves threads idle where a head has fewer channels than a workgroup threads: 64 us against 32 for 2,048 tokens of 8 heads of 128 with their decays.)
 __device__ __forceinline__ float4 delta_ld4(const float* p) { return *reinterpret_cast<const float4*>(p); }
 __device__ __forceinline__ float4 delta_ld4(const bf16_t* p) {
     const uint2 w = *reinterpret_cast<const uint2*>(p);
@@ -181,15 +181,19 @@ delta_prepare_pieces_kernel(float* __restrict__ qkv, float* __restrict__ gates, 
     float4 next[TT];                                          // the tokens' own inputs, all asked for at once
 #pragma unroll
     for (int k = 0; k < TT; ++k) next[k] = delta_ld4(proj + (size_t)min(t0 + k, tokens - 1) * row + q_off + c);
+    int seq[TT], place[TT];                                   // ... and whose they are (the same for the whole workgroup)
+#pragma unroll
+    for (int k = 0; k < TT; ++k) seq[k] = tok_seq[min(t0 + k, tokens - 1)];
+#pragma unroll
+    for (int k = 0; k < TT; ++k) place[k] = min(t0 + k, tokens - 1) - cu_seqlens[seq[k]];
     const bool normed = c < 2 * qk;
     const float scale = c < qk ? rsqrtf((float)dim) : 1.f;
 #pragma unroll
     for (int k = 0; k < TT; ++k) {
-        const int t = t0 + k;
+        const int t = t0 + k, i = place[k];
         if (t >= tokens) break;
-        const int b = tok_seq[t], i = t - cu_seqlens[b];
-        if (k == 0 || i == 0) {                               // (the same for the whole workgroup)
-            const float* tail = ntaps > 1 ? tails + (size_t)slots[b] * (ntaps - 1) * channels + c : nullptr;
+        if (k == 0 || i == 0) {
+            const float* tail = ntaps > 1 ? tails + (size_t)slots[seq[k]] * (ntaps - 1) * channels + c : nullptr;
 #pragma unroll
             for (int d = 1; d < 4; ++d) {
                 x[d] = make_float4(0.f, 0.f, 0.f, 0.f);

@@ -80,20 +80,21 @@ qk_half_bias_kv_write_kernel(T* __restrict__ proj, size_t row_len, int q_off, in
 }
 
 // A prompt whose halves and head sizes 16-byte pieces divide: a workgroup a token.  The token's sines and cosines are
-// made once, in LDS, as are, with gains, the heads' factors (a wavefront a head); a thread then takes a piece of eight from each half of a head (or one of the part that passes), every
+// made once, in LDS; with gains a head's norm meets over the lanes that hold its pieces, where they are a power of two (`lanes`),
+// and else in a pass of its own ahead (a wavefront a head, lanes 0); a thread takes a piece of eight from each half of a head (or one of the part that passes), every
 // load and store 16 bytes (32 for float32).  The values go a page at a time (values_to_pages_kernel).
 template <typename T>
-__global__ void __launch_bounds__(256)
+__global__ void __launch_bounds__(512)
 qk_half_bias_k_write_vec_kernel(T* __restrict__ proj, size_t row_len, int q_off, int k_off, const float* __restrict__ q_bias,
                                 const float* __restrict__ k_bias, const float* __restrict__ q_gain,
                                 const float* __restrict__ k_gain, float eps, const float* __restrict__ inv_freq, int half,
                                 float amplitude, const int32_t* __restrict__ tok_pos, const int32_t* __restrict__ tok_seq,
                                 const int32_t* __restrict__ page_table, int table_width, T* __restrict__ k_pages, int heads,
-                                int kv_heads, int dim, int page_size) {
+                                int kv_heads, int dim, int page_size, int lanes) {
     extern __shared__ __align__(16) float turn[];          // [half] cosines, [half] sines, [heads + kv_heads] factors
     const int t = blockIdx.x, pos = tok_pos[t];
     T* row = proj + (size_t)t * row_len;
-    if (q_gain) {
+    if (q_gain && !lanes) {
         for (int hh = threadIdx.x / RI_WAVE; hh < heads + kv_heads; hh += blockDim.x / RI_WAVE) {
             const bool is_q = hh < heads;
             const T* x = row + (is_q ? q_off + (size_t)hh * dim : k_off + (size_t)(hh - heads) * dim);
@@ -132,33 +133,38 @@ qk_half_bias_k_write_vec_kernel(T* __restrict__ proj, size_t row_len, int q_off,
         if (bias) bias += (size_t)(is_q ? hh : hh - heads) * dim;
         T* to = is_q ? x : k_pages + ((page * kv_heads + (hh - heads)) * page_size + pos % page_size) * dim;
         const int i = piece < turning ? piece * 8 : 2 * half + (piece - turning) * 8;
-        float u[8], b[8];
+        const bool turns = piece < turning;
+        float u[8], v[8], b[8];
         Eight<T>::load(x + i, u);
+        Eight<T>::load(x + (turns ? i + half : i), v);
         if (bias) {
             Eight<float>::load(bias + i, b);
 #pragma unroll
             for (int k = 0; k < 8; ++k) u[k] += b[k];
+            Eight<float>::load(bias + (turns ? i + half : i), b);
+#pragma unroll
+            for (int k = 0; k < 8; ++k) v[k] += b[k];
         }
         const float* gain = is_q ? q_gain : k_gain;
-        const float inv = gain ? turn[2 * half + hh] : 1.f;
         if (gain) {
+            float inv;
+            if (lanes) {                                      // (the lanes of a head run this loop together)
+                float ss = 0.f;
+#pragma unroll
+                for (int k = 0; k < 8; ++k) ss += u[k] * u[k] + (turns ? v[k] * v[k] : 0.f);
+                for (int m = lanes / 2; m > 0; m >>= 1) ss += __shfl_xor(ss, m, RI_WAVE);
+                inv = 1.f / sqrtf(ss / (float)dim + eps);
+            } else {
+                inv = turn[2 * half + hh];
+            }
             Eight<float>::load(gain + i, b);
 #pragma unroll
             for (int k = 0; k < 8; ++k) u[k] = u[k] * inv * b[k];
+            Eight<float>::load(gain + (turns ? i + half : i), b);
+#pragma unroll
+            for (int k = 0; k < 8; ++k) v[k] = v[k] * inv * b[k];
         }
-        if (piece < turning) {
-            float v[8];
-            Eight<T>::load(x + i + half, v);
-            if (bias) {
-                Eight<float>::load(bias + i + half, b);
-#pragma unroll
-                for (int k = 0; k < 8; ++k) v[k] += b[k];
-            }
-            if (gain) {
-                Eight<float>::load(gain + i + half, b);
-#pragma unroll
-                for (int k = 0; k < 8; ++k) v[k] = v[k] * inv * b[k];
-            }
+        if (turns) {
             float cs[8], sn[8];
             Eight<float>::load(turn + i, cs);
             Eight<float>::load(turn + half + i, sn);
@@ -189,11 +195,14 @@ static void launch_qk_half(T* proj, size_t row_len, int q_off, int k_off, int v_
                         (row_len | q_off | k_off) % unit == 0 && (uintptr_t)proj % 16 == 0 && (uintptr_t)k_pages % 16 == 0 &&
                         ((uintptr_t)q_bias | (uintptr_t)k_bias | (uintptr_t)q_gain | (uintptr_t)k_gain) % 16 == 0 &&
                         (2L * half + heads + kv_heads + 4) * (long)sizeof(float) <= 65536;
-    if (pieces)
-        qk_half_bias_k_write_vec_kernel<T><<<tokens, 256, (2 * half + heads + kv_heads + 4) * sizeof(float), s>>>(
+    if (pieces) {
+        const int of_head = half / 8 + (dim - 2 * half) / 8, all = (heads + kv_heads) * of_head;
+        const int lanes = of_head <= RI_WAVE && (of_head & (of_head - 1)) == 0 ? of_head : 0;
+        const int threads = all <= 512 && all > 256 ? (all + RI_WAVE - 1) / RI_WAVE * RI_WAVE : 256;      // (a token in one turn where that fits)
+        qk_half_bias_k_write_vec_kernel<T><<<tokens, threads, (2 * half + heads + kv_heads + 4) * sizeof(float), s>>>(
             proj, row_len, q_off, k_off, q_bias, k_bias, q_gain, k_gain, eps, inv_freq, half, amplitude, tok_pos, tok_seq, page_table, table_width,
-            k_pages, heads, kv_heads, dim, page_size);
-    else {
+            k_pages, heads, kv_heads, dim, page_size, lanes);
+    } else {
         const long items = (long)tokens * (heads + (paged_values ? 1 : 2) * kv_heads);
         qk_half_bias_kv_write_kernel<T><<<(unsigned)((items + 3) / 4), 256, 0, s>>>(
             proj, row_len, q_off, k_off, v_off, q_bias, k_bias, v_bias, q_gain, k_gain, eps, inv_freq, half, amplitude, tok_pos, tok_seq, page_table,
